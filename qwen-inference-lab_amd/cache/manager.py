@@ -17,7 +17,8 @@ One page more than the pool hands out lies behind every page group's storage, an
 are requests behind every state group's (``spare_page``, ``spare_slot``): no request ever gets them.  Inert rows
 that pad a captured step to its graph's size, and a new graph's warm-up run, write there.
 
-Per request the manager keeps ``computed``: how many tokens every layer has
+Per request the manager keeps ``last_tokens``, the last token of its steps so far (an embedding of token pairs
+needs the token before a step's first), and ``computed``: how many tokens every layer has
 cached.  A step must start exactly there (qil/cache.py:84-95,113-116) and
 ``advance`` moves it after the step ran.
 """
@@ -86,9 +87,10 @@ class CacheManager:
             raise ValueError(f'{len(self.kv_groups)} page groups, {len(pages)} page counts')
         for group, count in zip(self.kv_groups, pages):
             group['pool'] = PagePool(num_pages=count, page_size=page_size, window=group['need'].window,
-                                     max_step_tokens=max_step_tokens)
+                                     max_step_tokens=max_step_tokens, keep_first=getattr(group['need'], 'keep_first', 0))
         self.free_slots = deque(range(max_requests))
         self.slots, self.computed, self.limits = {}, {}, {}
+        self.last_tokens = {}            # request -> the last token its steps brought (None before the first)
         if allocate:
             self._allocate()
 
@@ -164,6 +166,7 @@ class CacheManager:
             group['pool'].admit(request, max_cached_tokens)
         self.slots[request] = self.free_slots.popleft()
         self.computed[request] = 0
+        self.last_tokens[request] = None
         self.limits[request] = max_cached_tokens
         return True
 
@@ -187,11 +190,13 @@ class CacheManager:
         for group in self.kv_groups:
             group['pool'].ensure(request, end)
 
-    def advance(self, request, end):
-        """The step has cached tokens up to ``end``; windows give passed pages back."""
+    def advance(self, request, end, last_token=None):
+        """The step has cached tokens up to ``end``, of which ``last_token`` is the last; windows give passed pages
+        back."""
         if end < self.computed[request]:
             raise ValueError('computed length cannot shrink')
         self.computed[request] = end
+        self.last_tokens[request] = last_token
         for group in self.kv_groups:
             group['pool'].pass_window(request, end)
 
@@ -201,7 +206,7 @@ class CacheManager:
         for group in self.kv_groups:
             group['pool'].release(request)
         self.free_slots.append(self.slots.pop(request))
-        del self.computed[request], self.limits[request]
+        del self.computed[request], self.limits[request], self.last_tokens[request]
 
     def owns(self, request):
         return request in self.slots

@@ -8,7 +8,7 @@ Admission reserves credits for a request's whole life, so partial prefills can
 never exhaust the pool and deadlock (qil/cache.py:1-5,54-68); physical pages are
 taken only as tokens are computed (qil/cache.py:70-77) and go back FIFO
 (qil/cache.py:43,77,184).  A windowed pool also gives pages back as soon as the
-window has passed them.
+window has passed them, but for the first ``keep_first`` tokens' pages, which stay.
 """
 from collections import deque
 
@@ -18,16 +18,19 @@ class CacheFull(RuntimeError):
 
 
 class PagePool:
-    def __init__(self, *, num_pages, page_size, window=None, max_step_tokens=None):
+    def __init__(self, *, num_pages, page_size, window=None, max_step_tokens=None, keep_first=0):
         if type(num_pages) is not int or num_pages < 1 or type(page_size) is not int or page_size < 1:
             raise ValueError('num_pages and page_size must be positive integers')
         if window is not None and (type(window) is not int or window < 1):
             raise ValueError('window must be a positive integer or None')
+        if type(keep_first) is not int or keep_first < 0:
+            raise ValueError('keep_first must be a non-negative integer')
         self.capacity, self.page_size, self.window = num_pages, page_size, window
+        self.kept_pages = self.pages_for(keep_first) if window is not None else 0     # first blocks that stay for good
         self.max_step_tokens = max_step_tokens
         self.free = deque(range(num_pages))
         self.tables = {}        # request -> list of page ids by logical block (-1: given back)
-        self.first_live = {}    # request -> first logical block still held
+        self.first_live = {}    # request -> first logical block still held (behind the kept ones)
         self.credits = {}       # request -> reserved pages (0 for unreserved admission)
 
     def pages_for(self, tokens):
@@ -39,7 +42,7 @@ class PagePool:
         if self.window is None or self.max_step_tokens is None:
             return whole
         # live span of a step: window - 1 old keys + the step's tokens, not block aligned
-        return min(whole, self.pages_for(self.window - 1 + self.max_step_tokens) + 1)
+        return min(whole, self.kept_pages + self.pages_for(self.window - 1 + self.max_step_tokens) + 1)
 
     @property
     def unreserved(self):
@@ -66,12 +69,12 @@ class PagePool:
 
     def pass_window(self, request, computed):
         """Give back blocks no later query can see: all their keys j satisfy
-        j <= p - window for every position p >= computed."""
+        j <= p - window for every position p >= computed, and none is among the kept first ones."""
         if self.window is None:
             return
         table = self.tables[request]
         horizon = computed - self.window + 1          # smallest key index still visible
-        block = self.first_live[request]
+        block = max(self.first_live[request], self.kept_pages)
         while block < len(table) and (block + 1) * self.page_size <= horizon:
             self.free.append(table[block])
             table[block] = -1

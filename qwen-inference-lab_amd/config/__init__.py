@@ -5,5 +5,7 @@ from .fubapel import FubapelConfig
 from .gerivik import GerivikConfig
 from .zinesun import ZinesunConfig
 from .dogozen import DogozenConfig
+from .tinuzen import TinuzenConfig
 
-__all__ = ['ConfigError', 'read_config_json', 'Qwen3Config', 'FubapelConfig', 'GerivikConfig', 'ZinesunConfig', 'DogozenConfig']
+__all__ = ['ConfigError', 'read_config_json', 'Qwen3Config', 'FubapelConfig', 'GerivikConfig', 'ZinesunConfig', 'DogozenConfig',
+           'TinuzenConfig']

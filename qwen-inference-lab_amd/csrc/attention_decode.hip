@@ -19,8 +19,12 @@
 // written or belong to someone else: their scores are replaced, not multiplied, and their V
 // elements are zeroed before the product, so garbage (even NaN) cannot enter a sum.
 //
+// keep > 0: the first `keep` keys stay visible behind a window; steps and parts then count places (key_span.h).
+// slopes: slopes[h] * (position - key) is taken off head h's scaled score.
+//
 // Takes page_size % 8 == 0, d % 16 == 0, d <= 256, g <= 16; other sizes go to the row kernel.
 #include "common.h"
+#include "key_span.h"
 #include "qk_math.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -46,6 +50,9 @@ struct FusedQKV {
   int writes;                                              // 0: the cache belongs to another layer, which wrote it
   int row_elems;                                           // elements of a row of qkv (more than q, k and v where another
                                                            // branch's columns follow; q alone for a reader without k and v)
+  int v_head;                                              // the head-sized piece of a row at which the values begin
+                                                           // (heads + kv_heads; heads: the values are the keys before norm
+                                                           // and rotation)
   const float* bias;                                       // null, or the projection's bias by column, added to the sums
   float temp_coef;                                         // temp_every > 0: the query at position p is multiplied by
   int temp_every;                                          // 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) last
@@ -73,7 +80,7 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
                    const int* __restrict__ row_index, float* __restrict__ part_acc, float* __restrict__ part_m,
                    float* __restrict__ part_l, bf16_t* __restrict__ out, int heads, int kv_heads, int d,
                    int page_size, int window, float scale, int P, int parts, float softcap,
-                   const float* __restrict__ sinks) {
+                   const float* __restrict__ sinks, const float* __restrict__ slopes, int keep) {
   constexpr int QFRAGS = DMAX / 32, DTILES = DMAX / 16;
   if (WHOLE) d = DMAX;                                      // what the host has checked, known to the compiler: no
                                                             // condition on the head size stays in the loops
@@ -82,17 +89,19 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
   const int row = row_index ? row_index[slot_row] : slot_row;
   const int g = heads / kv_heads;
   const int pos = positions[row], ctx = pos + 1;
-  const int lo = window > 0 ? max(0, ctx - window) : 0;
-  const int begin = max(part * P, lo), end = min((part + 1) * P, ctx);
+  const KeySpan span(pos, window, keep);
+  const int begin = max(part * P, span.first_place()), end = min((part + 1) * P, span.places());      // places
   if (begin >= end) return;
+  const int pos_place = pos - span.hole;                   // the row's own key lies behind the hole
 
   const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE, waves = blockDim.x / QIL_WAVE;
   const int r = lane & 15, kb = lane >> 4;
   const int dt = d / 16;
   const int* table = block_tables + (size_t)row_seq[row] * table_stride;
 
-  const int first_step = begin / 32;                       // 32-key steps, absolute numbering
+  const int first_step = begin / 32;                       // steps of 32 places, numbered from the first place
   const int last_step = (end - 1) / 32;
+  const float slope = (slopes && r < g) ? slopes[kvh * g + r] : 0.f;
 
   // Q fragments: B operand, column r = head kvh * g + r (filled below, after the first loads are on their way)
   bf16x8 qb[QFRAGS];
@@ -111,7 +120,7 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
     uint4 v[DTILES];                                        // V^T[dim 16 t + r][keys 8 kb .. 8 kb + 7]: 16 bytes of one page row
   };
   auto look_up = [&](int step, int (&page)[3]) {
-    const int k0 = step * 32;
+    const int k0 = span.key(step * 32);
 #pragma unroll
     for (int jt = 0; jt < 2; ++jt)
       // row r of sub-tile jt is key 8 (r / 4) + 4 jt + r % 4 of the step, so that a lane's eight
@@ -120,7 +129,7 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
     page[2] = table[(min(k0 + 8 * kb, ctx - 1) & ~7) / page_size];
   };
   auto request = [&](int step, const int (&page)[3], StepData& data) {
-    const int k0 = step * 32;
+    const int k0 = span.key(step * 32);
 #pragma unroll
     for (int jt = 0; jt < 2; ++jt) {
       const int key = min(k0 + 8 * (r >> 2) + 4 * jt + (r & 3), ctx - 1);
@@ -138,9 +147,9 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
       data.v[t] = t < dt ? once4(vbase + (size_t)(t * 16 + r) * page_size) : make_uint4(0, 0, 0, 0);
   };
   auto attend = [&](int step, StepData& data) {
-    const int k0 = step * 32;
+    const int k0 = span.key(step * 32);
     if constexpr (FUSED) {
-      if (owner && step == (pos >> 5)) {                   // the new key and value come from this wave's registers
+      if (owner && step == (pos_place >> 5)) {                   // the new key and value come from this wave's registers
         const int local = pos & 31;                          // key 8 (rr / 4) + 4 jt + rr % 4 of the step
         const int jt_new = (local >> 2) & 1, rr = ((local >> 3) << 2) | (local & 3);
 #pragma unroll
@@ -179,16 +188,17 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
       s[jt] = acc;
     }
     float mx = -INFINITY;
-    uint32_t keep[2][4];                                    // 0xffff where the key is visible
+    uint32_t seen[2][4];                                    // 0xffff where the key is visible
 #pragma unroll
     for (int jt = 0; jt < 2; ++jt)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = k0 + 8 * kb + 4 * jt + i;
-        const bool visible = key >= begin && key < end;
-        keep[jt][i] = visible ? 0xffffu : 0u;
+        const bool visible = span.visible(key);              // (a part ends at a whole step, or where the keys end)
+        seen[jt][i] = visible ? 0xffffu : 0u;
         float v = s[jt][i] * scale;
         if (softcap > 0.f) v = soft_cap_fast(v, softcap, 2.88539008177793f / softcap);
+        v = fmaf(slope, (float)(key - pos), v);
         if (!visible) v = -INFINITY;
         s[jt][i] = v;
         mx = fmaxf(mx, v);
@@ -216,8 +226,8 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
       for (int i = 0; i < 2; ++i)
         packed[jt * 2 + i] = pack_bf16(s[jt][2 * i], s[jt][2 * i + 1]);
     const bf16x8 pb = __builtin_bit_cast(bf16x8, make_uint4(packed[0], packed[1], packed[2], packed[3]));
-    const uint32_t mask[4] = {keep[0][0] | (keep[0][1] << 16), keep[0][2] | (keep[0][3] << 16),
-                              keep[1][0] | (keep[1][1] << 16), keep[1][2] | (keep[1][3] << 16)};
+    const uint32_t mask[4] = {seen[0][0] | (seen[0][1] << 16), seen[0][2] | (seen[0][3] << 16),
+                              seen[1][0] | (seen[1][1] << 16), seen[1][2] | (seen[1][3] << 16)};
 #pragma unroll
     for (int t = 0; t < DTILES; ++t) {
       if (t < dt) {
@@ -249,7 +259,7 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
         }
         if (base + sub < g) shared_q[(base + sub) * TG + chunk] = pack8(x);
       }
-      owner = fused.writes && pos >= begin && pos < end && wave == ((pos >> 5) - first_step) % waves;
+      owner = fused.writes && pos_place >= begin && pos_place < end && wave == ((pos_place >> 5) - first_step) % waves;
       if (owner) {                                           // wave-uniform
         float x[8];
         load8_sum_wide(fused.qkv, (size_t)row * fused.row_elems + (size_t)(heads + kvh) * DMAX + chunk * 8, fused.splits, fused.split_stride, x);
@@ -257,9 +267,9 @@ attn_decode_kernel(FusedQKV fused, const bf16_t* __restrict__ q, int q_stride, c
         norm_rope8<bf16_t>(x, chunk, TG, fused.k_weight, DMAX, fused.eps, fused.cos_table, fused.sin_table, pos, fused.rot,
                            fused.rotate_first != 0);
         new_k = pack8(x);
-        load8_sum_wide(fused.qkv, (size_t)row * fused.row_elems + (size_t)(heads + kv_heads + kvh) * DMAX + chunk * 8, fused.splits,
+        load8_sum_wide(fused.qkv, (size_t)row * fused.row_elems + (size_t)(fused.v_head + kvh) * DMAX + chunk * 8, fused.splits,
                        fused.split_stride, x);
-        add_bias8(x, fused.bias, (heads + kv_heads + kvh) * DMAX + chunk * 8);
+        add_bias8(x, fused.bias, (fused.v_head + kvh) * DMAX + chunk * 8);
         new_v = pack8(x);
         if (sub == 0) {                                      // into the pages (qil/cache.py:79-82)
           const size_t page = table[pos / page_size];
@@ -377,15 +387,17 @@ extern "C" int qil_attn_decode_takes(int heads, int kv_heads, int d, int page_si
 // the caller runs the row kernel's merge when parts > 1.  P must be a multiple of 32; a block has
 // `waves` waves (at most 8), best one or two 32-key steps of P for each.  pairs != 0: a wave loads two of
 // its steps at a time (twice the registers; for launches of at most one block a CU).  sinks: null, or float32 [heads]:
-// exp(sink) joins a head's divisor (here when parts == 1, else in the merge).
+// exp(sink) joins a head's divisor (here when parts == 1, else in the merge).  slopes: null, or float32 [heads]; keep > 0
+// (with a window): the kept first keys, and P and parts count places.
 extern "C" int qil_attn_decode(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                const int* block_tables, int table_stride, const int* row_seq, const int* positions,
                                const int* row_index, void* workspace, void* out, int rows, int heads, int kv_heads,
                                int d, int page_size, int window, float scale, int P, int parts, int waves,
-                               int pairs, float softcap, const float* sinks, hipStream_t s) {
+                               int pairs, float softcap, const float* sinks, const float* slopes, int keep,
+                               hipStream_t s) {
   if (rows == 0) return 0;
   if (!qil_attn_decode_takes(heads, kv_heads, d, page_size) || P % 32 || P < 32 || parts < 1 || parts > 65535 ||
-      kv_heads > 65535 || waves < 1 || waves > DEC_MAX_WAVES)
+      kv_heads > 65535 || waves < 1 || waves > DEC_MAX_WAVES || keep < 0 || (keep > 0 && window <= 0))
     return -1;
   const int g = heads / kv_heads;
   float* acc = (float*)workspace;
@@ -398,12 +410,12 @@ extern "C" int qil_attn_decode(const void* q, int q_stride, const void* k_cache,
   hipLaunchKernelGGL((attn_decode_kernel<DMAX, PAIRS, FUSED>), grid, dim3(waves * QIL_WAVE), lds, s, FIELDS,         \
                      (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables,       \
                      table_stride, row_seq, positions, row_index, acc, m, l, (bf16_t*)out, heads, kv_heads, d,        \
-                     page_size, window, scale, P, parts, softcap, sinks)
+                     page_size, window, scale, P, parts, softcap, sinks, slopes, keep)
 #define QIL_DEC_WHOLE(DMAX, PAIRS)                                                                                  \
   hipLaunchKernelGGL((attn_decode_kernel<DMAX, PAIRS, false, true>), grid, dim3(waves * QIL_WAVE), lds, s, none,     \
                      (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables,       \
                      table_stride, row_seq, positions, row_index, acc, m, l, (bf16_t*)out, heads, kv_heads, d,        \
-                     page_size, window, scale, P, parts, softcap, sinks)
+                     page_size, window, scale, P, parts, softcap, sinks, slopes, keep)
 #define QIL_DEC_CASE(DMAX)                                                                                          \
   if (d == DMAX && pairs) QIL_DEC_WHOLE(DMAX, true);                                                                \
   else if (d == DMAX) QIL_DEC_WHOLE(DMAX, false);                                                                   \
@@ -433,6 +445,8 @@ extern "C" int qil_attn_decode_fused_takes(int heads, int kv_heads, int d, int p
 // positions (the page comes from the block table).  has_kv 0: the rows of qkv hold queries only (a reader; writes must be 0).
 // extra_columns: so many more columns follow in every row and are skipped.  bias: null, or float32 by column of q, k and v.
 // temp_every > 0: the query temperature of qk_rope.hip.  sinks: null, or float32 [heads] (as in qil_attn_decode).
+// shared_kv: the rows hold no values of their own; a value is its key as projected, before norm and rotation.
+// slopes, keep: as in qil_attn_decode.
 extern "C" int qil_attn_decode_fused(const float* qkv, int splits, const float* q_weight, const float* k_weight,
                                      float eps, const float* cos_table, const float* sin_table, int rot, int writes,
                                      void* k_cache, void* v_cache, const int* block_tables, int table_stride,
@@ -440,8 +454,9 @@ extern "C" int qil_attn_decode_fused(const float* qkv, int splits, const float* 
                                      int heads, int kv_heads, int d, int page_size, int window, float scale, int P,
                                      int parts, int waves, int pairs, int rotate_first, float softcap,
                                      int has_kv, int extra_columns, const float* bias, float temp_coef, int temp_every,
-                                     const float* sinks, hipStream_t s) {
+                                     const float* sinks, int shared_kv, const float* slopes, int keep, hipStream_t s) {
   if (rows == 0) return 0;
+  if (keep < 0 || (keep > 0 && window <= 0) || (shared_kv && !has_kv)) return -1;
   if (extra_columns < 0 || temp_every < 0 || (writes && !has_kv) || ((uintptr_t)bias % 16) || extra_columns % 8) return -1;
   if (!qil_attn_decode_fused_takes(heads, kv_heads, d, page_size, cos_table ? rot : 0) || P % 32 || P < 32 ||
       parts < 1 || parts > 65535 || kv_heads > 65535 || waves < 1 || waves > DEC_MAX_WAVES || splits < 1 ||
@@ -457,7 +472,8 @@ extern "C" int qil_attn_decode_fused(const float* qkv, int splits, const float* 
   dim3 grid(rows, kv_heads, parts);
   FusedQKV fused;
   fused.qkv = qkv;
-  fused.row_elems = (heads + (has_kv ? 2 * kv_heads : 0)) * d + extra_columns;
+  fused.row_elems = (heads + (has_kv ? (shared_kv ? 1 : 2) * kv_heads : 0)) * d + extra_columns;
+  fused.v_head = shared_kv ? heads : heads + kv_heads;
   fused.split_stride = (size_t)rows * fused.row_elems;
   fused.bias = bias; fused.temp_coef = temp_coef; fused.temp_every = temp_every;
   fused.splits = splits;

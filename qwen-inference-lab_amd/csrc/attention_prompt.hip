@@ -51,16 +51,19 @@ __device__ __forceinline__ int prompt_row(int kl) {
 // of its SIMD's issue slots whether the wave is alone there or not, and 2,048 tokens are 33 wave-tiles a SIMD.)
 // CAP: scores are scaled and capped softly (softcap * tanh(score / softcap)) as they leave the matrix cores; the
 // exponent then scales nothing.
-template <int WAVES, bool SPLIT = false, bool CAP = false>
+// EXT (keys in one part): slopes[h] * (position - key) is taken off head h's scaled score as it leaves the matrix cores
+// (the exponent then scales nothing), and the first `keep` keys stay visible behind a window: a block walks the tiles
+// that hold them, then goes on at its window's first tile.
+template <int WAVES, bool SPLIT = false, bool CAP = false, bool EXT = false>
 __global__ void __launch_bounds__(WAVES * QIL_WAVE, WAVES == 4 ? 2 : 1)
 attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_cache,
                    const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int table_stride,
                    const int* __restrict__ cu_seqlens, const int* __restrict__ seq_starts, bf16_t* __restrict__ out,
                    int heads, int kv_heads, int page_size, int window, float scale, int GH, int chunks, int ps_shift,
                    float* __restrict__ part_acc, float* __restrict__ part_m, float* __restrict__ part_l, int P,
-                   int parts, float softcap, const float* __restrict__ sinks) {
+                   int parts, float softcap, const float* __restrict__ sinks, const float* __restrict__ slopes, int keep) {
   const float raw_scale = scale;
-  if (CAP) scale = 1.f;
+  if (CAP || EXT) scale = 1.f;
   constexpr int D = PROMPT_D, BK = PROMPT_BK, THREADS = WAVES * QIL_WAVE;
   constexpr int GW = SPLIT ? WAVES / 2 : WAVES;            // waves that share a tile of keys
   constexpr int WFRAGS = D / 16, WTILES = D / 32;
@@ -119,10 +122,16 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
     if (key_begin >= key_end) return;                                  // no row of the block sees a key of this part
   }
   const int first_tile = key_begin / BK * BK;
+  // EXT: the tiles that hold kept keys come first (those below the window's first tile), and a tile's number counts
+  // without the ones left out between: tile number k0 stands for the keys from k0 + jump on from kept_end on
+  const int kept_end = EXT && keep > 0 ? min((keep + BK - 1) / BK * BK, first_tile) : 0;
+  const int jump = EXT && kept_end > 0 ? first_tile - kept_end : 0;
+  auto tile_key = [&](int k0) __attribute__((always_inline)) { return EXT ? k0 + (k0 >= kept_end ? jump : 0) : k0; };
+  const float slope = (EXT && slopes && wave_active) ? slopes[head] : 0.f;
 
   // Block-table entries of [first_tile, key_end) into LDS, as the page's place in the cache in units of 256 bytes
   // (a page of one kv head is 2 KB or more; 32 bits reach 1 TB).
-  const int first_page = first_tile >> ps_shift, last_page = (key_end - 1) >> ps_shift;
+  const int first_page = (EXT && kept_end > 0 ? 0 : first_tile) >> ps_shift, last_page = (key_end - 1) >> ps_shift;
   {
     const int* table = block_tables + (size_t)seq * table_stride;
     const uint32_t page_units = (uint32_t)kv_heads * page_size * D / 128;
@@ -159,7 +168,7 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
 
   // ---- loads.  Load j = it * GW + wave of a tile: K keys 4 j .. 4 j + 3 (rows prompt_row(4 j) .. + 3, 1 KB), and
   // V^T of the 64 dims 64 (j % 2) .. of the 8 keys from 8 (j / 2) on: both in the page of key 4 j.
-  const int low_page = key_begin >> ps_shift;
+  const int low_page = EXT && keep > 0 ? first_page : key_begin >> ps_shift;     // (kept keys may lie below the window's page)
   const char* k_head = reinterpret_cast<const char*>(k_cache + (size_t)kvh * page_size * D);
   const char* v_head = reinterpret_cast<const char*>(v_cache + ((size_t)kvh * D + (wave & 1) * 64) * page_size);
   // lane = (key lane / 16 of the four, piece lane % 16): it loads the dims that piece lane % 16 of its row holds
@@ -188,25 +197,25 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
                                      (__attribute__((address_space(3))) void*)(to + BK * D * 2 + j * 1024), 16, 0, 0);
   };
   // any k0: the pages are kept inside the needed ones
-  auto load_tile = [&](int k0, unsigned char* to) __attribute__((always_inline)) {
+  auto load_tile = [&](int k0, int k1, unsigned char* to) __attribute__((always_inline)) {
 #pragma unroll
     for (int it = 0; it < LOADS; ++it) {
       load_k(k0 & (page_size - 1), it, to);
       load_v(k0 & (page_size - 1), it, to);
     }
-    held = look_up(k0 + BK);
+    held = look_up(k1);
   };
   // Values of keys outside [key_begin, key_end) of the tile at `tile` become zero (K needs none: the mask).
   auto zero_values = [&](int k0, unsigned char* tile) __attribute__((always_inline)) {
     for (int idx = threadIdx.x % (GW * QIL_WAVE); idx < BK / 8 * D; idx += GW * QIL_WAVE) {
       const int key = k0 + idx / D * 8;
-      if (key >= key_begin && key + 8 <= key_end) continue;
+      if ((key >= key_begin || (EXT && key + 8 <= keep)) && key + 8 <= key_end) continue;
       uint4* cell = reinterpret_cast<uint4*>(tile + BK * D * 2) + idx;
       const uint4 raw = *cell;
       uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
 #pragma unroll
       for (int e = 0; e < 8; ++e)
-        if (!(key + e >= key_begin && key + e < key_end)) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+        if (!((key + e >= key_begin || (EXT && key + e < keep)) && key + e < key_end)) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
       *cell = make_uint4(w[0], w[1], w[2], w[3]);
     }
   };
@@ -215,7 +224,8 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
   const float c = scale * 1.44269504088896f;               // p = exp2((s - m) c): the scale enters in the exponent
   const uint32_t k_read = l32 * (D * 2), k_piece = half ^ (l32 & 15);        // piece 2 ks + half of row l32 is at (2 ks) ^ k_piece
   const uint32_t v_read = (half * D + l32) * 16;
-  auto attend = [&](int k0, const unsigned char* tile, unsigned char* next, bool masked, bool more) __attribute__((always_inline)) {
+  // k0: the tile's first key; k1, k2: those of the two tiles after it (only their pages are asked for).
+  auto attend = [&](int k0, int k1, int k2, const unsigned char* tile, unsigned char* next, bool masked, bool more) __attribute__((always_inline)) {
     const unsigned char* Ks = tile + k_read;
     const unsigned char* Vt = tile + BK * D * 2 + v_read;
     auto k_fragment = [&](int kt, int ks) __attribute__((always_inline)) {
@@ -232,7 +242,7 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
     for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
       for (int i = 0; i < 16; ++i) s[kt][i] = 0.f;
-    const int in_page = (k0 + BK) & (page_size - 1);
+    const int in_page = k1 & (page_size - 1);
     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int ks = 0; ks < WFRAGS; ++ks) {
@@ -246,7 +256,7 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
         else load_k(in_page, ks >> 1, next);
       }
       s[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka[ks][1], qw[ks], s[1], 0, 0, 0);
-      if (ks == 2 * LOADS - 1) held = look_up(k0 + 2 * BK);
+      if (ks == 2 * LOADS - 1) held = look_up(k2);
       __builtin_amdgcn_sched_barrier(0);
     }
     if (CAP) {
@@ -256,13 +266,21 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
 #pragma unroll
         for (int i = 0; i < 16; ++i) s[kt][i] = soft_cap_fast(s[kt][i] * raw_scale, softcap, fast);
     }
+    if (EXT) {
+      const float first = (float)(k0 + 8 * half - my_pos);   // of the lane's first key: key - position
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+          s[kt][i] = fmaf(slope, first + (float)(32 * kt + 16 * (i >> 3) + (i & 7)), s[kt][i] * raw_scale);
+    }
     if (masked) {                                          // keys a row does not see get score -inf (probability 0)
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int key = k0 + 32 * kt + 16 * (i >> 3) + 8 * half + (i & 7);
-          const bool visible = key <= my_pos && (window <= 0 || key > my_pos - window);
+          const bool visible = key <= my_pos && (window <= 0 || key > my_pos - window || (EXT && key < keep));
           s[kt][i] = visible ? s[kt][i] : -INFINITY;
         }
     }
@@ -334,7 +352,7 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
     const int mine = group == 0 ? T / 2 : T - T / 2, steps = T - T / 2;
     int k0 = first_tile + (group == 0 ? 0 : (T / 2) * BK);
     held = look_up(k0);
-    load_tile(k0, tiles);
+    load_tile(k0, k0 + BK, tiles);
     for (int step = 0; step < steps; ++step, k0 += BK) {
       unsigned char* tile = tiles + buffer * PROMPT_TILE_BYTES;
       unsigned char* next = tiles + (buffer ^ 1) * PROMPT_TILE_BYTES;
@@ -346,9 +364,9 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
       }
       if (step < mine && wave_active && k0 <= wave_last_pos) {
         const bool all_visible = k0 + BK - 1 <= start + wave_row0 && wave_row0 + 32 <= n;
-        attend(k0, tile, next, !all_visible, true);
+        attend(k0, k0 + BK, k0 + 2 * BK, tile, next, !all_visible, true);
       } else if (step + 1 < mine) {
-        load_tile(k0 + BK, next);
+        load_tile(k0 + BK, k0 + 2 * BK, next);
       }
       buffer ^= 1;
     }
@@ -377,31 +395,35 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
     row_l = row_l * mine_scale + other_l * other_scale;
     row_m = m;
   } else {
-  held = look_up(first_tile);
-  load_tile(first_tile, tiles);
-  auto tile_step = [&](int k0, auto edge_tag) __attribute__((always_inline)) {
+  // (a tile's number is its first key, but for EXT behind the kept tiles; `last` is one past the last number)
+  const int start_tile = EXT && kept_end > 0 ? 0 : first_tile, last = key_end - jump;
+  held = look_up(tile_key(start_tile));
+  load_tile(tile_key(start_tile), tile_key(start_tile + BK), tiles);
+  auto tile_step = [&](int number, auto edge_tag) __attribute__((always_inline)) {
+    const int k0 = tile_key(number), k1 = tile_key(number + BK), k2 = tile_key(number + 2 * BK);
     unsigned char* tile = lds + buffer * PROMPT_TILE_BYTES;
     unsigned char* next = lds + (buffer ^ 1) * PROMPT_TILE_BYTES;
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");       // this wave's loads of the tile have landed
     __syncthreads();                                       // everyone's have, and everyone is done with the tile before
-    if (decltype(edge_tag)::value && !(k0 >= key_begin && k0 + BK <= key_end)) {
+    if ((EXT || decltype(edge_tag)::value) && !((k0 >= key_begin || (EXT && k0 + BK <= keep)) && k0 + BK <= key_end)) {
       zero_values(k0, tile);
       __syncthreads();
     }
     if (wave_active && k0 <= wave_last_pos) {
       const bool all_visible = k0 + BK - 1 <= start + wave_row0 && wave_row0 + 32 <= n &&
-                               (window <= 0 || k0 > wave_last_pos - window);
-      attend(k0, tile, next, !all_visible, k0 + BK < key_end);
-    } else if (k0 + BK < key_end) {
-      load_tile(k0 + BK, next);
+                               (window <= 0 || k0 > wave_last_pos - window || (EXT && k0 + BK <= keep));
+      attend(k0, k1, k2, tile, next, !all_visible, number + BK < last);
+    } else if (number + BK < last) {
+      load_tile(k1, k2, next);
     }
     buffer ^= 1;
   };
   // only the first and the last tile can hold keys outside [key_begin, key_end): the loop between has no such check
-  int k0 = first_tile;
-  tile_step(k0, std::true_type());
-  for (k0 += BK; k0 + BK < key_end; k0 += BK) tile_step(k0, std::false_type());
-  if (k0 < key_end) tile_step(k0, std::true_type());
+  // (EXT: the last kept tile and the window's first may hold such keys as well, and every tile checks)
+  int number = start_tile;
+  tile_step(number, std::true_type());
+  for (number += BK; number + BK < last; number += BK) tile_step(number, std::false_type());
+  if (number < last) tile_step(number, std::true_type());
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");         // no load into LDS is on its way when the block ends
   }
 
@@ -435,16 +457,16 @@ attn_prompt_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __r
           make_uint2(pack_bf16(ow[t][4 * j] * inv, ow[t][4 * j + 1] * inv), pack_bf16(ow[t][4 * j + 2] * inv, ow[t][4 * j + 3] * inv));
 }
 
-template <int WAVES, bool SPLIT = false, bool CAP = false>
+template <int WAVES, bool SPLIT = false, bool CAP = false, bool EXT = false>
 static int launch_prompt(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                          int table_stride, const int* cu_seqlens, const int* seq_starts, void* out, int n_seqs,
                          int max_query, int heads, int kv_heads, int page_size, int window, float scale, hipStream_t s,
                          float* workspace, int total_rows, int P, int parts, float softcap = 0.f,
-                         const float* sinks = nullptr) {
+                         const float* sinks = nullptr, const float* slopes = nullptr, int keep = 0) {
   const int g = heads / kv_heads;
   const int GH = g >= 3 ? 4 : g, chunks = (g + GH - 1) / GH, RT = (SPLIT ? WAVES / 2 : WAVES) / GH;
   const size_t lds = (SPLIT ? 4 : 2) * (size_t)PROMPT_TILE_BYTES + (size_t)table_stride * sizeof(int);
-  auto kernel = attn_prompt_kernel<WAVES, SPLIT, CAP>;
+  auto kernel = attn_prompt_kernel<WAVES, SPLIT, CAP, EXT>;
   static size_t granted = 0;                     // per instantiation
   if (lds > granted) {
     hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -460,7 +482,7 @@ static int launch_prompt(const void* q, int q_stride, const void* k_cache, const
   hipLaunchKernelGGL(kernel, grid, dim3(WAVES * QIL_WAVE), lds, s, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
                      (const bf16_t*)v_cache, block_tables, table_stride, cu_seqlens, seq_starts, (bf16_t*)out, heads,
                      kv_heads, page_size, window, scale, GH, chunks, ps_shift, workspace, part_m, part_l, P, parts,
-                     softcap, sinks);
+                     softcap, sinks, slopes, keep);
   return (int)hipGetLastError();
 }
 
@@ -520,4 +542,20 @@ extern "C" int qil_attn_prompt_sinks(const void* q, int q_stride, const void* k_
     return -1;
   return launch_prompt<4>(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out, n_seqs,
                           max_query, heads, kv_heads, page_size, window, scale, s, nullptr, 0, 0, 1, 0.f, sinks);
+}
+
+// The same with a bias by distance (slopes float32 [heads], or null) and the first `keep` keys visible behind a window
+// (keep > 0 needs one); sinks as above or null.  Keys in one part, blocks of 4 waves.
+extern "C" int qil_attn_prompt_extended(const void* q, int q_stride, const void* k_cache, const void* v_cache,
+                                        const int* block_tables, int table_stride, const int* cu_seqlens,
+                                        const int* seq_starts, void* out, int n_seqs, int max_query, int heads, int kv_heads,
+                                        int page_size, int window, float scale, const float* sinks, const float* slopes,
+                                        int keep, hipStream_t s) {
+  if (n_seqs == 0 || max_query < 2) return 0;
+  if (!qil_attn_prompt_takes(PROMPT_D, page_size, table_stride) || heads % kv_heads || n_seqs > 65535 ||
+      (long)kv_heads * 2 > 65535 || !out || keep < 0 || (keep > 0 && window <= 0))
+    return -1;
+  return launch_prompt<4, false, false, true>(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens,
+                                              seq_starts, out, n_seqs, max_query, heads, kv_heads, page_size, window, scale,
+                                              s, nullptr, 0, 0, 1, 0.f, sinks, slopes, keep);
 }

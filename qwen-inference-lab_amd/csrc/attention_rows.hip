@@ -13,6 +13,8 @@
 // float32 (qil/paged_attention.py:27-41).  A block whose range is empty returns without writing,
 // and the merge skips the same parts (qil/paged_attention.py:33-34 handles it with a safe maximum).
 // With a single part the normalised result is written directly.
+// keep > 0: the first `keep` keys stay visible behind a window, and the parts count places (key_span.h).  slopes:
+// slopes[h] * (position - key) is taken off head h's scaled score.
 //
 // Merge kernel: grid (rows, heads): out = sum_p acc_p exp(m_p - m) / sum_p l_p exp(m_p - m)
 // (qil/paged_attention.py:44-58).
@@ -20,6 +22,7 @@
 // Lanes: a token's d elements are spread over TG = next_pow2(ceil(d / 8)) lanes, eight elements a
 // lane; a wave handles 64 / TG tokens at a time.
 #include "common.h"
+#include "key_span.h"
 
 #define ATT_THREADS 256
 #define ATT_WAVES (ATT_THREADS / QIL_WAVE)
@@ -54,14 +57,14 @@ attn_rows_partial_kernel(const T* __restrict__ q, int q_stride, const T* __restr
                          const int* __restrict__ row_index, float* __restrict__ part_acc,
                          float* __restrict__ part_m, float* __restrict__ part_l,
                          T* __restrict__ out, int heads, int kv_heads, int d, int page_size, int window,
-                         float scale, float softcap, int P, int parts, int tg_log2, const float* __restrict__ sinks) {
+                         float scale, float softcap, int P, int parts, int tg_log2, const float* __restrict__ sinks,
+                         const float* __restrict__ slopes, int keep) {
   extern __shared__ float lds[];
   const int slot_row = blockIdx.x, kvh = blockIdx.y, part = blockIdx.z;   // slot_row indexes the workspace
   const int row = row_index ? row_index[slot_row] : slot_row;             // row of the step's batch
   const int g = heads / kv_heads;
-  const int ctx = positions[row] + 1;
-  const int lo = window > 0 ? max(0, ctx - window) : 0;
-  const int begin = max(part * P, lo), end = min((part + 1) * P, ctx);
+  const KeySpan span(positions[row], window, keep);
+  const int begin = max(part * P, span.first_place()), end = min((part + 1) * P, span.places());
   if (begin >= end) return;
   const int count = end - begin;
 
@@ -94,7 +97,7 @@ attn_rows_partial_kernel(const T* __restrict__ q, int q_stride, const T* __restr
       float kv[4][8];
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
-        const int j = begin + min(t0 + u * stride, count - 1);
+        const int j = span.key(begin + min(t0 + u * stride, count - 1));
         const size_t page = table[j / page_size];
         const size_t base = ((page * kv_heads + kvh) * page_size + (j % page_size)) * (size_t)d + e0;
         if (live) ld8(k_cache + base, kv[u]);
@@ -111,7 +114,15 @@ attn_rows_partial_kernel(const T* __restrict__ q, int q_stride, const T* __restr
 #pragma unroll
           for (int e = 0; e < 8; ++e) dot += qv[h][e] * kv[u][e];
           dot = group_sum(dot, tg_log2);
-          if (sub == 0 && t < count) scores[h * P + t] = soft_cap(dot * scale, softcap);
+          if (sub == 0 && t < count) {
+            float score = soft_cap(dot * scale, softcap);
+            if (slopes || keep > 0) {
+              const int j = span.key(begin + t);
+              if (slopes && h0 + h < g) score -= slopes[kvh * g + h0 + h] * (float)(span.ctx - 1 - j);
+              if (!span.visible(j)) score = -INFINITY;
+            }
+            scores[h * P + t] = score;
+          }
         }
       }
     }
@@ -170,11 +181,12 @@ attn_rows_partial_kernel(const T* __restrict__ q, int q_stride, const T* __restr
         float vv[2][8];
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
-          const int j = begin + min(t0 + u * V_STRIDE, count - 1);
+          const int j = span.key(begin + min(t0 + u * V_STRIDE, count - 1));
           const size_t page = table[j / page_size];
           const T* column = v_cache + ((page * kv_heads + kvh) * (size_t)d + ve) * page_size + (j % page_size);
+          const bool seen = v_live && span.visible(j);         // what a hidden key's page holds may be anything
 #pragma unroll
-          for (int e = 0; e < 8; ++e) vv[u][e] = v_live ? ld(column + (size_t)e * page_size) : 0.f;
+          for (int e = 0; e < 8; ++e) vv[u][e] = seen ? ld(column + (size_t)e * page_size) : 0.f;
         }
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
@@ -233,14 +245,13 @@ __global__ void __launch_bounds__(QIL_WAVE)
 attn_rows_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_m,
                        const float* __restrict__ part_l, const int* __restrict__ positions,
                        const int* __restrict__ row_index, T* __restrict__ out, int heads, int d,
-                       int window, int P, int parts, int tg, const float* __restrict__ sinks) {
+                       int window, int P, int parts, int tg, const float* __restrict__ sinks, int keep) {
   const int slot_row = blockIdx.x;
   const int head = blockIdx.y * (QIL_WAVE / tg) + threadIdx.x / tg, e = (threadIdx.x % tg) * 4;
   const bool head_there = head < heads;                    // the same for the tg lanes of a head; all of them take part in the maximum
   const int row = row_index ? row_index[slot_row] : slot_row;
-  const int ctx = positions[row] + 1;
-  const int lo = window > 0 ? max(0, ctx - window) : 0;
-  const int first = lo / P, last = (ctx - 1) / P;
+  const KeySpan span(positions[row], window, keep);
+  const int first = span.first_place() / P, last = (span.places() - 1) / P;
   const size_t cell0 = ((size_t)slot_row * heads + head) * parts;
   // the largest exponent: a head's lanes take a part each, then the largest among them (one round trip to memory for
   // up to tg parts, not one for every four)
@@ -306,7 +317,7 @@ static int launch_rows(const void* q, int q_stride, const void* k_cache, const v
                        float* part_acc, float* part_m,
                        float* part_l, void* out, int rows, int heads, int kv_heads, int d, int page_size, int window,
                        float scale, float softcap, int P, int parts, hipStream_t s, bool merge = true,
-                       const float* sinks = nullptr) {
+                       const float* sinks = nullptr, const float* slopes = nullptr, int keep = 0) {
   const int g = heads / kv_heads;
   const int gt = g >= 8 ? 8 : g > 2 ? 4 : g;            // head tile: 1, 2, 4 or 8
   const int tg_log2 = next_pow2_log2((d + 7) / 8);
@@ -316,7 +327,7 @@ static int launch_rows(const void* q, int q_stride, const void* k_cache, const v
   hipLaunchKernelGGL((attn_rows_partial_kernel<T, GT>), grid, dim3(ATT_THREADS), lds, s, (const T*)q, q_stride,    \
                      (const T*)k_cache, (const T*)v_cache, block_tables, table_stride, row_seq, positions,         \
                      row_index, part_acc, part_m, part_l, (T*)out, heads, kv_heads, d, page_size, window, scale, softcap, P, parts,    \
-                     tg_log2, sinks)
+                     tg_log2, sinks, slopes, keep)
   switch (gt) {
     case 1: QIL_ROWS_CASE(1); break;
     case 2: QIL_ROWS_CASE(2); break;
@@ -330,7 +341,7 @@ static int launch_rows(const void* q, int q_stride, const void* k_cache, const v
   dim3 merge_grid;
   merge_shape(rows, heads, d, &tg, &merge_grid);
   hipLaunchKernelGGL(attn_rows_merge_kernel<T>, merge_grid, dim3(QIL_WAVE), 0, s, part_acc, part_m, part_l, positions,
-                     row_index, (T*)out, heads, d, window, P, parts, tg, sinks);
+                     row_index, (T*)out, heads, d, window, P, parts, tg, sinks, keep);
   return (int)hipGetLastError();
 }
 
@@ -344,14 +355,16 @@ size_t qil_attn_rows_workspace(int rows, int heads, int d, int parts) {
 // q: rows of stride q_stride elements, head h at offset h * d.  out: [all rows, heads * d].
 // row_index: null (the kernel's rows are the batch's rows 0 .. rows-1) or the batch rows to serve.
 // workspace: qil_attn_rows_workspace bytes.  P: keys per part, parts = ceil(max context / P).
-// sinks: null, or float32 [heads] (a term exp(sink) more in every head's divisor).
+// sinks: null, or float32 [heads] (a term exp(sink) more in every head's divisor).  slopes: null, or float32 [heads].
+// keep > 0 (with a window): P is a multiple of 32 and parts = ceil(most places / P).
 // Requires d % 8 == 0, d <= 256, P <= 1024.  Returns -1 on a size it does not take.
 int qil_attn_rows(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                   int table_stride, const int* row_seq, const int* positions, const int* row_index, void* workspace,
                   void* out, int rows,
                   int heads, int kv_heads, int d, int page_size, int window, float scale, float softcap, int P, int parts, int dtype,
-                  const float* sinks, hipStream_t s) {
+                  const float* sinks, const float* slopes, int keep, hipStream_t s) {
   if (rows == 0) return 0;
+  if (keep < 0 || (keep > 0 && (window <= 0 || P % 32))) return -1;
   if (d % 8 || d > 256 || d < 8 || heads % kv_heads || P < 1 || P > 1024 || parts < 1 || parts > 65535 ||
       kv_heads > 65535) return -1;
   const int g = heads / kv_heads;
@@ -362,9 +375,11 @@ int qil_attn_rows(const void* q, int q_stride, const void* k_cache, const void* 
   float* l = m ? m + (size_t)rows * heads * parts : nullptr;
   if (dtype == QIL_F32)
     return launch_rows<float>(q, q_stride, k_cache, v_cache, block_tables, table_stride, row_seq, positions, row_index,
-                              acc, m, l, out, rows, heads, kv_heads, d, page_size, window, scale, softcap, P, parts, s, true, sinks);
+                              acc, m, l, out, rows, heads, kv_heads, d, page_size, window, scale, softcap, P, parts, s, true, sinks,
+                              slopes, keep);
   return launch_rows<bf16_t>(q, q_stride, k_cache, v_cache, block_tables, table_stride, row_seq, positions, row_index,
-                             acc, m, l, out, rows, heads, kv_heads, d, page_size, window, scale, softcap, P, parts, s, true, sinks);
+                             acc, m, l, out, rows, heads, kv_heads, d, page_size, window, scale, softcap, P, parts, s, true, sinks,
+                              slopes, keep);
 }
 
 // The same without the merge: the parts' results stay in the workspace for a consumer that merges them itself
@@ -390,9 +405,9 @@ int qil_attn_rows_unmerged(const void* q, int q_stride, const void* k_cache, con
 }
 
 // Merge of partial results written by a partial kernel (this file's or the matrix-core decode kernel's).
-// sinks: null, or float32 [heads]: exp(sink) joins every head's divisor once.
+// sinks: null, or float32 [heads]: exp(sink) joins every head's divisor once.  keep: the kept first keys (key_span.h).
 int qil_attn_merge(const void* workspace, const int* positions, const int* row_index, void* out, int rows, int heads,
-                   int d, int window, int P, int parts, int dtype, const float* sinks, hipStream_t s) {
+                   int d, int window, int P, int parts, int dtype, const float* sinks, int keep, hipStream_t s) {
   if (rows == 0 || parts <= 1) return 0;
   const float* acc = (const float*)workspace;
   const float* m = acc + (size_t)rows * heads * parts * d;
@@ -404,10 +419,10 @@ int qil_attn_merge(const void* workspace, const int* positions, const int* row_i
   const dim3 block(QIL_WAVE);
   if (dtype == QIL_F32)
     hipLaunchKernelGGL(attn_rows_merge_kernel<float>, grid, block, 0, s, acc, m, l, positions, row_index, (float*)out,
-                       heads, d, window, P, parts, tg, sinks);
+                       heads, d, window, P, parts, tg, sinks, keep);
   else
     hipLaunchKernelGGL(attn_rows_merge_kernel<bf16_t>, grid, block, 0, s, acc, m, l, positions, row_index, (bf16_t*)out,
-                       heads, d, window, P, parts, tg, sinks);
+                       heads, d, window, P, parts, tg, sinks, keep);
   QIL_RETURN_LAUNCH_STATUS();
 }
 

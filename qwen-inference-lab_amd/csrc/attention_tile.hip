@@ -12,6 +12,9 @@
 // (qil/model.py:62-64).  Keys at or beyond the block's last position + 1 are never loaded: they
 // are not written yet or belong to nobody; their LDS slots are zero so that 0 * garbage cannot
 // make a NaN.  A wave skips key sub-tiles that lie wholly in the future of all its rows.
+// keep > 0 (with a window, keys in one part): the first `keep` keys stay visible; a block walks the tiles that hold
+// them, then goes on at its window's first tile.  slopes: slopes[h] * (position - key) is taken off head h's scaled
+// score.
 //
 // Matrix-core formulation (wave64, 16x16 tiles).  Scores are computed transposed,
 //   S^T[key, row] = sum_dim K[key, dim] Q[row, dim]        A = K tile (LDS), B = Q (registers)
@@ -64,10 +67,10 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
                  const int* __restrict__ seq_starts, T* __restrict__ out, int heads, int kv_heads, int d,
                  int page_size, int window, float scale, int GH, int chunks, int ps_shift,
                  float* __restrict__ part_acc, float* __restrict__ part_m, float* __restrict__ part_l, int P, int parts,
-                 float softcap, const float* __restrict__ sinks) {
-  // with a soft cap the scores are scaled and capped as they are made, and nothing is left for the exponent to scale
+                 float softcap, const float* __restrict__ sinks, const float* __restrict__ slopes, int keep) {
+  // with a soft cap or a bias by distance the scores are scaled as they are made, and nothing is left for the exponent
   const float raw_scale = scale;
-  if (softcap > 0.f) scale = 1.f;
+  if (softcap > 0.f || slopes) scale = 1.f;
   using TT = TileTraits<T>;
   constexpr int BK = TT::BK, KSTEP = TT::KSTEP, PAD = TT::PAD;
   constexpr bool BF16 = sizeof(T) == 2;
@@ -196,22 +199,27 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
   // Addresses of places that are not needed are clamped onto needed ones.
   const bool fast = BF16 && fast_v;
   const int first_tile = key_begin / BK * BK;
+  // the tiles that hold kept keys come first (those that lie below the window's first tile)
+  const int kept_end = keep > 0 ? min((keep + BK - 1) / BK * BK, first_tile) : 0;
+  const int low_key = keep > 0 ? 0 : key_begin;            // the first key whose page the block's table is asked for
+  const float slope = (slopes && wave_active) ? slopes[head] : 0.f;
+  auto needed = [&](int key) { return key < key_end && (key >= key_begin || key < keep); };
 
-  for (int k0 = first_tile; k0 < key_end; k0 += BK) {
+  for (int k0 = kept_end > 0 ? 0 : first_tile; k0 < key_end; k0 = k0 + BK == kept_end ? first_tile : k0 + BK) {
     __syncthreads();                                   // the previous tile is consumed
     if (fast) {
       if constexpr (BF16) {
-        const bool inside = k0 >= key_begin && k0 + BK <= key_end;          // no key of the tile needs zeroing
+        const bool inside = (k0 >= key_begin || k0 + BK <= keep) && k0 + BK <= key_end;     // no key of the tile needs zeroing
         size_t k_page[K_ITERS], v_page[V_ITERS];
         int k_off[K_ITERS], v_off[V_ITERS];
 #pragma unroll
         for (int it = 0; it < K_ITERS; ++it) {
-          const int key = min(max(k0 + max(k_kl[it], 0), key_begin), key_end - 1);
+          const int key = min(max(k0 + max(k_kl[it], 0), low_key), key_end - 1);
           k_page[it] = page_of(key, k_off[it]);
         }
 #pragma unroll
         for (int it = 0; it < V_ITERS; ++it) {
-          const int key = min(max(k0 + max(v_grp[it], 0) * 8, key_begin & ~7), (key_end - 1) & ~7);
+          const int key = min(max(k0 + max(v_grp[it], 0) * 8, low_key & ~7), (key_end - 1) & ~7);
           v_page[it] = page_of(key, v_off[it]);
         }
         uint4 k_reg[K_ITERS], v_reg[V_ITERS];
@@ -227,7 +235,7 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
         for (int it = 0; it < K_ITERS; ++it) {
           if (k_kl[it] < 0) continue;
           const int key = k0 + k_kl[it];
-          const bool valid = key >= key_begin && key < key_end && k_dv[it] < d;
+          const bool valid = needed(key) && k_dv[it] < d;
           *reinterpret_cast<uint4*>(Ks + k_kl[it] * k_row + k_dv[it]) = valid ? k_reg[it] : make_uint4(0, 0, 0, 0);
         }
 #pragma unroll
@@ -239,7 +247,7 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
             uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
 #pragma unroll
             for (int e = 0; e < 8; ++e)
-              if (!(key + e >= key_begin && key + e < key_end)) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+              if (!needed(key + e)) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
             raw = make_uint4(w[0], w[1], w[2], w[3]);
           }
           *reinterpret_cast<uint4*>(Vt + v_dim[it] * v_row + v_grp[it] * 8) = raw;
@@ -251,7 +259,7 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
     for (int it = 0; it < K_ITERS; ++it) {
       if (k_kl[it] < 0) continue;
       const int kl = k_kl[it], dv = k_dv[it], key = k0 + kl;
-      const bool valid = key >= key_begin && key < key_end && dv < d;
+      const bool valid = needed(key) && dv < d;
       T* kdst = Ks + kl * k_row + dv;
       size_t page = 0;
       int offset = 0;
@@ -286,7 +294,7 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
         if (v_grp[it] < 0) continue;
         const int grp = v_grp[it], dim = v_dim[it], key = k0 + grp * 8;
         T* dst = Vt + dim * v_row + grp * 8;
-        const bool any = key + 7 >= key_begin && key < key_end && dim < d;
+        const bool any = (key + 7 >= key_begin || key < keep) && key < key_end && dim < d;
         float vals[8];
         if (any) {
           int offset;
@@ -294,7 +302,7 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
           ld8(v_cache + ((page * kv_heads + kvh) * (size_t)d + dim) * page_size + offset, vals);
         }
 #pragma unroll
-        for (int e = 0; e < 8; ++e) dst[e] = (any && key + e >= key_begin && key + e < key_end) ? vals[e] : 0.f;
+        for (int e = 0; e < 8; ++e) dst[e] = (any && needed(key + e)) ? vals[e] : 0.f;
       }
     }
     }
@@ -351,12 +359,22 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
           for (int i = 0; i < 4; ++i)
             s[b][jt][i] = BF16 ? soft_cap_fast(s[b][jt][i] * raw_scale, softcap, fast) : soft_cap(s[b][jt][i] * raw_scale, softcap);
     }
+    if (slopes) {
+      const float rest = softcap > 0.f ? 1.f : raw_scale;
+#pragma unroll
+      for (int b = 0; b < RB; ++b)
+#pragma unroll
+        for (int jt = 0; jt < SUB; ++jt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            s[b][jt][i] = fmaf(slope, (float)(k0 + jt * 16 + 4 * kb + i - my_pos[b]), s[b][jt][i] * rest);
+    }
     // ---- mask and online softmax (per-lane row statistics).  m holds the running maximum of the RAW
     // scores; the scale (> 0) enters once, in the exponent: p = exp(scale * (s - m)).
     // every key of the tile is visible to every row of the wave unless the tile touches the wave's
     // first row's future, the window's edge or the rows beyond the sequence
     const bool all_visible = k0 + BK - 1 <= start + wave_row0 && wave_row0 + 16 * RB <= n &&
-                             (window <= 0 || k0 > wave_last_pos - window);
+                             (window <= 0 || k0 > wave_last_pos - window || k0 + BK <= keep);
 #pragma unroll
     for (int b = 0; b < RB; ++b) {
       float mx = -INFINITY;
@@ -371,7 +389,8 @@ attn_tile_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ k_
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int key = k0 + jt * 16 + 4 * kb + i;
-            const bool visible = row_valid[b] && key <= my_pos[b] && (window <= 0 || key > my_pos[b] - window);
+            const bool visible = row_valid[b] && key <= my_pos[b] &&
+                                 (window <= 0 || key > my_pos[b] - window || key < keep);
             const float v = visible ? s[b][jt][i] : -INFINITY;
             s[b][jt][i] = v;
             mx = fmaxf(mx, v);
@@ -498,7 +517,7 @@ static int launch_tile(const void* q, int q_stride, const void* k_cache, const v
                        int table_stride, const int* cu_seqlens, const int* seq_starts, void* out, int n_seqs,
                        int max_query, int heads, int kv_heads, int d, int page_size, int window, float scale,
                        hipStream_t s, float* workspace = nullptr, int total_rows = 0, int P = 0, int parts = 1,
-                       float softcap = 0.f, const float* sinks = nullptr) {
+                       float softcap = 0.f, const float* sinks = nullptr, const float* slopes = nullptr, int keep = 0) {
   using TT = TileTraits<T>;
   const int g = heads / kv_heads;
   const int GH = g >= 3 ? 4 : g, chunks = (g + GH - 1) / GH, RT = 4 / GH;
@@ -522,7 +541,8 @@ static int launch_tile(const void* q, int q_stride, const void* k_cache, const v
     if (page_size == (1 << b)) ps_shift = b;
   hipLaunchKernelGGL(kernel, grid, dim3(TILE_THREADS), lds, s, (const T*)q, q_stride, (const T*)k_cache,
                      (const T*)v_cache, block_tables, table_stride, cu_seqlens, seq_starts, (T*)out, heads, kv_heads, d,
-                     page_size, window, scale, GH, chunks, ps_shift, workspace, part_m, part_l, P, parts, softcap, sinks);
+                     page_size, window, scale, GH, chunks, ps_shift, workspace, part_m, part_l, P, parts, softcap, sinks, slopes,
+                     keep);
   return (int)hipGetLastError();
 }
 
@@ -569,6 +589,11 @@ extern "C" int qil_attn_prompt_sinks(const void* q, int q_stride, const void* k_
                                      const int* block_tables, int table_stride, const int* cu_seqlens,
                                      const int* seq_starts, void* out, int n_seqs, int max_query, int heads, int kv_heads,
                                      int page_size, int window, float scale, const float* sinks, hipStream_t s);
+extern "C" int qil_attn_prompt_extended(const void* q, int q_stride, const void* k_cache, const void* v_cache,
+                                        const int* block_tables, int table_stride, const int* cu_seqlens,
+                                        const int* seq_starts, void* out, int n_seqs, int max_query, int heads, int kv_heads,
+                                        int page_size, int window, float scale, const float* sinks, const float* slopes,
+                                        int keep, hipStream_t s);
 // parts > 1: the keys in `parts` parts of P keys (P a multiple of 64) on this file's kernel; every row of a sequence
 // of two or more rows gets float32 partial results in `workspace` (qil_attn_rows_workspace bytes for all `total_rows`
 // rows of the step, indexed by the step's row) for qil_attn_merge, and `out` is not written.
@@ -576,24 +601,30 @@ static int tile_dispatch(const void* q, int q_stride, const void* k_cache, const
                          const int* block_tables, int table_stride, const int* cu_seqlens, const int* seq_starts,
                          void* out, int n_seqs, int max_query, int heads, int kv_heads, int d, int page_size,
                          int window, float scale, int dtype, hipStream_t s, float* workspace, int total_rows, int P,
-                         int parts, float softcap, const float* sinks = nullptr) {
+                         int parts, float softcap, const float* sinks = nullptr, const float* slopes = nullptr, int keep = 0) {
   if (n_seqs == 0 || max_query < 2) return 0;
+  if (keep < 0 || (keep > 0 && (window <= 0 || parts > 1))) return -1;
+  const bool extended = slopes || keep > 0;
+  // a bias by distance or kept first keys on bfloat16 heads of 128, keys in one part: the prompt kernel's extended form
+  if (extended && parts == 1 && softcap <= 0.f && dtype == QIL_BF16 && qil_attn_prompt_takes(d, page_size, table_stride))
+    return qil_attn_prompt_extended(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out,
+                                    n_seqs, max_query, heads, kv_heads, page_size, window, scale, sinks, slopes, keep, s);
   if (d % 8 || d < 8 || d > 256 || heads % kv_heads || n_seqs > 65535 || kv_heads * 2 > 65535) return -1;
   // capped scores of bfloat16 heads of 128: the prompt kernel's capped form (keys in one part or in parts of whole tiles)
-  if (softcap > 0.f && !sinks && dtype == QIL_BF16 && qil_attn_prompt_takes(d, page_size, table_stride) && (parts == 1 || P % 64 == 0))
+  if (softcap > 0.f && !sinks && !extended && dtype == QIL_BF16 && qil_attn_prompt_takes(d, page_size, table_stride) && (parts == 1 || P % 64 == 0))
     return qil_attn_prompt_capped(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out,
                                   n_seqs, max_query, heads, kv_heads, page_size, window, scale, softcap, workspace,
                                   total_rows, P, parts, s);
   // sinks on bfloat16 heads of 128, keys in one part: the prompt kernel's form with sinks
-  if (sinks && parts == 1 && softcap <= 0.f && dtype == QIL_BF16 && qil_attn_prompt_takes(d, page_size, table_stride))
+  if (sinks && !extended && parts == 1 && softcap <= 0.f && dtype == QIL_BF16 && qil_attn_prompt_takes(d, page_size, table_stride))
     return qil_attn_prompt_sinks(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out,
                                  n_seqs, max_query, heads, kv_heads, page_size, window, scale, sinks, s);
-  if (parts == 1 && softcap <= 0.f && !sinks && dtype == QIL_BF16 && qil_attn_tile_bf16_takes(d, page_size, table_stride))
+  if (parts == 1 && softcap <= 0.f && !sinks && !extended && dtype == QIL_BF16 && qil_attn_tile_bf16_takes(d, page_size, table_stride))
     return qil_attn_tile_bf16(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out,
                               n_seqs, max_query, heads, kv_heads, d, page_size, window, scale, s);
 #define QIL_TILE_CASE(T, DMAX)                                                                                      \
   return launch_tile<T, DMAX, (sizeof(T) == 2 && DMAX <= 128) ? 2 : 1>(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out, \
-                              n_seqs, max_query, heads, kv_heads, d, page_size, window, scale, s, workspace, total_rows, P, parts, softcap, sinks)
+                              n_seqs, max_query, heads, kv_heads, d, page_size, window, scale, s, workspace, total_rows, P, parts, softcap, sinks, slopes, keep)
   if (dtype == QIL_F32) {
     if (d <= 64) QIL_TILE_CASE(float, 64);
     if (d <= 128) QIL_TILE_CASE(float, 128);
@@ -608,19 +639,20 @@ static int tile_dispatch(const void* q, int q_stride, const void* k_cache, const
 extern "C" int qil_attn_tile(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                              const int* block_tables, int table_stride, const int* cu_seqlens, const int* seq_starts,
                              void* out, int n_seqs, int max_query, int heads, int kv_heads, int d, int page_size,
-                             int window, float scale, float softcap, int dtype, const float* sinks, hipStream_t s) {
+                             int window, float scale, float softcap, int dtype, const float* sinks, const float* slopes,
+                             int keep, hipStream_t s) {
   return tile_dispatch(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, out, n_seqs,
-                       max_query, heads, kv_heads, d, page_size, window, scale, dtype, s, nullptr, 0, 0, 1, softcap, sinks);
+                       max_query, heads, kv_heads, d, page_size, window, scale, dtype, s, nullptr, 0, 0, 1, softcap, sinks, slopes, keep);
 }
 
 extern "C" int qil_attn_tile_in_parts(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                       const int* block_tables, int table_stride, const int* cu_seqlens,
                                       const int* seq_starts, void* workspace, int total_rows, int n_seqs, int max_query,
                                       int heads, int kv_heads, int d, int page_size, int window, float scale,
-                                      float softcap, int P, int parts, int dtype, hipStream_t s) {
+                                      float softcap, int P, int parts, int dtype, const float* slopes, hipStream_t s) {
   if (n_seqs == 0 || max_query < 2) return 0;
   if (parts < 2 || P < 64 || P % 64 || !workspace || total_rows < 1) return -1;
   return tile_dispatch(q, q_stride, k_cache, v_cache, block_tables, table_stride, cu_seqlens, seq_starts, nullptr, n_seqs,
                        max_query, heads, kv_heads, d, page_size, window, scale, dtype, s, (float*)workspace, total_rows,
-                       P, parts, softcap);
+                       P, parts, softcap, nullptr, slopes);
 }

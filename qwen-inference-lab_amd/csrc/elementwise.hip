@@ -29,6 +29,26 @@ __global__ void embed_bf16x8_kernel(const int* __restrict__ tokens, const bf16_t
   }
 }
 
+// stream[n, :] = table[token[n], :] * scale + pairs[row, :] with row = (previous[n] * mul_prev + token[n] * mul_cur) mod
+// buckets, or `buckets` (the table's last row) where previous[n] < 0 (a sequence's first token).  `copy`: null, or a
+// second place for the result.
+template <typename T>
+__global__ void embed_pairs_kernel(const int* __restrict__ tokens, const int* __restrict__ previous,
+                                   const T* __restrict__ table, const T* __restrict__ pairs, float* __restrict__ stream,
+                                   float* __restrict__ copy, int width, float scale, int buckets, long long mul_prev,
+                                   long long mul_cur) {
+  const int n = blockIdx.x, token = tokens[n], before = previous[n];
+  const size_t row = before < 0 ? (size_t)buckets : (size_t)((before * mul_prev + token * mul_cur) % buckets);
+  const T* a = table + (size_t)token * width;
+  const T* b = pairs + row * width;
+  const size_t at = (size_t)n * width;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float v = ld(a + i) * scale + ld(b + i);
+    stream[at + i] = v;
+    if (copy) copy[at + i] = v;
+  }
+}
+
 __device__ __forceinline__ float4 load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 __device__ __forceinline__ float4 load4(const bf16_t* p) {
   const uint2 raw = *reinterpret_cast<const uint2*>(p);
@@ -221,6 +241,22 @@ int qil_embed(const int* tokens, const void* table, float* stream, int n, int wi
   else
     hipLaunchKernelGGL(embed_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, tokens, (const bf16_t*)table, stream, width,
                        scale);
+  QIL_RETURN_LAUNCH_STATUS();
+}
+
+// pairs: [buckets + 1, width]; mul_prev, mul_cur >= 0.
+int qil_embed_pairs(const int* tokens, const int* previous, const void* table, const void* pairs, float* stream, float* copy,
+                    int n, int width, float scale, int buckets, long long mul_prev, long long mul_cur, int dtype,
+                    hipStream_t s) {
+  if (n == 0) return 0;
+  if (buckets < 1 || mul_prev < 0 || mul_cur < 0 || !previous || !pairs) return -1;
+  const int threads = width >= 1024 ? 256 : 64;
+  if (dtype == QIL_F32)
+    hipLaunchKernelGGL(embed_pairs_kernel<float>, dim3(n), dim3(threads), 0, s, tokens, previous, (const float*)table,
+                       (const float*)pairs, stream, copy, width, scale, buckets, mul_prev, mul_cur);
+  else
+    hipLaunchKernelGGL(embed_pairs_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, tokens, previous, (const bf16_t*)table,
+                       (const bf16_t*)pairs, stream, copy, width, scale, buckets, mul_prev, mul_cur);
   QIL_RETURN_LAUNCH_STATUS();
 }
 

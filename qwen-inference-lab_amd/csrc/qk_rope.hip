@@ -39,10 +39,11 @@ __global__ void qk_norm_rope_store_kernel(
     const float* __restrict__ cos_table, const float* __restrict__ sin_table, const int* __restrict__ positions,
     const int* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache,
     int heads, int kv_heads, int d, int rot, int page_size, float eps, int norm_dim, int rotate_first, int row_elems,
-    float temp_coef, int temp_every, const float* __restrict__ bias) {
+    float temp_coef, int temp_every, const float* __restrict__ bias, int v_head) {
   __shared__ float vec[QIL_MAX_HEAD_DIM];
   const int n = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
-  const size_t src = (size_t)n * row_elems + (size_t)head * d;    // index into qkv
+  const int piece = head < heads + kv_heads ? head : head - heads - kv_heads + v_head;     // head-sized piece of the row
+  const size_t src = (size_t)n * row_elems + (size_t)piece * d;   // index into qkv
   const bool is_q = head < heads, is_k = !is_q && head < heads + kv_heads;
   if (!is_q && slots == nullptr) return;                 // a reader of another entry's cache writes no k/v
 
@@ -56,14 +57,14 @@ __global__ void qk_norm_rope_store_kernel(
     } else {                                             // v: copy, transposed within the page
       T* column = v_cache + (page * kv_heads + kvh) * (size_t)d * page_size + offset;
       for (int i = lane; i < d; i += QIL_WAVE)
-        st(column + (size_t)i * page_size, load_sum(qkv, src + i, splits, split_stride) + (bias ? bias[head * d + i] : 0.f));
+        st(column + (size_t)i * page_size, load_sum(qkv, src + i, splits, split_stride) + (bias ? bias[piece * d + i] : 0.f));
       return;
     }
   }
 
   const float* weight = is_q ? q_weight : k_weight;
   for (int i = lane; i < d; i += QIL_WAVE)
-    vec[i] = load_sum(qkv, src + i, splits, split_stride) + (bias ? bias[head * d + i] : 0.f);
+    vec[i] = load_sum(qkv, src + i, splits, split_stride) + (bias ? bias[piece * d + i] : 0.f);
   __syncthreads();
   const int half = rot / 2;
   const int position = positions[n];
@@ -119,7 +120,7 @@ qk_norm_rope_store_vec_kernel(
     const float* __restrict__ sin_table, const int* __restrict__ positions, const int* __restrict__ slots,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int n, int heads, int kv_heads, int d, int rot, int page_size,
     float eps, int tg_log2, unsigned v_first_block, int norm_dim, int rotate_first, int row_elems, float temp_coef,
-    int temp_every, const float* __restrict__ bias) {
+    int temp_every, const float* __restrict__ bias, int v_head) {
   const int total_heads = heads + 2 * kv_heads;
   const int TG = 1 << tg_log2;
   if (blockIdx.x >= v_first_block) {
@@ -135,8 +136,8 @@ qk_norm_rope_store_vec_kernel(
     const int chunk = quad * 4 + (lane & 3);
     if (token >= (size_t)n) return;
     float x[8];
-    load8_sum(qkv, token * row_elems + (size_t)(heads + kv_heads + kvh) * d + chunk * 8, splits, split_stride, x);
-    add_bias8(x, bias, (heads + kv_heads + kvh) * d + chunk * 8);
+    load8_sum(qkv, token * row_elems + (size_t)(v_head + kvh) * d + chunk * 8, splits, split_stride, x);
+    add_bias8(x, bias, (v_head + kvh) * d + chunk * 8);
     const int slot = slots[token];
     const size_t page = slot / page_size, offset = slot % page_size;
     T* column = v_cache + ((page * kv_heads + kvh) * (size_t)d + chunk * 8) * page_size + offset;
@@ -152,8 +153,9 @@ qk_norm_rope_store_vec_kernel(
   const bool is_q = head < heads, is_k = !is_q && head < heads + kv_heads;
   if (!is_q && slots == nullptr) return;
   float x[8];
-  load8_sum(qkv, (size_t)token * row_elems + (size_t)head * d + chunk * 8, splits, split_stride, x);
-  add_bias8(x, bias, head * d + chunk * 8);
+  const int piece = is_q || is_k ? head : head - heads - kv_heads + v_head;
+  load8_sum(qkv, (size_t)token * row_elems + (size_t)piece * d + chunk * 8, splits, split_stride, x);
+  add_bias8(x, bias, piece * d + chunk * 8);
 
   if (!is_q && !is_k) {                                 // v: copy, transposed within the page
     const int kvh = head - heads - kv_heads, slot = slots[token];
@@ -188,15 +190,17 @@ qk_norm_rope_store_vec_kernel(
 // product); they are skipped.  kv_heads 0: the rows hold queries only (a reader of another entry's cache).
 // bias: null, or float32 [(heads + 2 kv_heads) d]: the projection's bias, added to the sums as they are loaded (the
 // product before this kernel then needs none, and may leave partial sums).
+// shared_kv: the rows hold no values of their own; a value is its key as projected, before norm and rotation.
 // temp_every > 0: the query at position p is multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) last.
 extern "C" int qil_qk_norm_rope_store(
     const void* qkv, int in_dtype, int splits, void* q_out, const float* q_weight, const float* k_weight,
     const float* cos_table, const float* sin_table, const int* positions, const int* slots, void* k_cache,
     void* v_cache, int n, int heads, int kv_heads, int d, int rot, int page_size, float eps, int norm_dim, int rotate_first,
-    int extra_columns, float temp_coef, int temp_every, const float* bias, int dtype, hipStream_t s) {
+    int extra_columns, float temp_coef, int temp_every, const float* bias, int shared_kv, int dtype, hipStream_t s) {
   if (n == 0) return 0;
   if (extra_columns < 0 || temp_every < 0 || kv_heads < 0 || (kv_heads == 0 && slots)) return -1;
-  const int row_elems = (heads + 2 * kv_heads) * d + extra_columns;
+  const int row_elems = (heads + (shared_kv ? 1 : 2) * kv_heads) * d + extra_columns;
+  const int v_head = shared_kv ? heads : heads + kv_heads;
   if (norm_dim == 0) norm_dim = d;
   if (norm_dim < 1 || norm_dim > d) return -1;
   if (d > QIL_MAX_HEAD_DIM || rot > d || (rot & 1) || splits < 1 || (in_dtype == QIL_BF16 && splits != 1)) return -1;
@@ -224,7 +228,7 @@ extern "C" int qil_qk_norm_rope_store(
   hipLaunchKernelGGL((qk_norm_rope_store_vec_kernel<TD, T>), dim3(blocks), dim3(256), 0, s, (const TD*)qkv, splits,    \
                      stride, (T*)q_out, q_weight, k_weight, cos_table, sin_table, positions, slots, (T*)k_cache,       \
                      (T*)v_cache, n, heads, kv_heads, d, rot, page_size, eps, tg_log2, v_first_block, norm_dim, rotate_first,       \
-                     row_elems, temp_coef, temp_every, bias)
+                     row_elems, temp_coef, temp_every, bias, v_head)
     if (dtype == QIL_F32) QIL_QKV_CASE(float, float);
     else if (in_dtype == QIL_F32) QIL_QKV_CASE(float, bf16_t);
     else QIL_QKV_CASE(bf16_t, bf16_t);
@@ -234,10 +238,125 @@ extern "C" int qil_qk_norm_rope_store(
 #define QIL_QK_CASE(TD, T)                                                                                            \
   hipLaunchKernelGGL((qk_norm_rope_store_kernel<TD, T>), grid, dim3(QIL_WAVE), 0, s, (const TD*)qkv, splits, stride,   \
                      (T*)q_out, q_weight, k_weight, cos_table, sin_table, positions, slots, (T*)k_cache, (T*)v_cache,  \
-                     heads, kv_heads, d, rot, page_size, eps, norm_dim, rotate_first, row_elems, temp_coef, temp_every, bias)
+                     heads, kv_heads, d, rot, page_size, eps, norm_dim, rotate_first, row_elems, temp_coef, temp_every, bias, \
+                     v_head)
   if (dtype == QIL_F32) QIL_QK_CASE(float, float);
   else if (in_dtype == QIL_F32) QIL_QK_CASE(float, bf16_t);
   else QIL_QK_CASE(bf16_t, bf16_t);
 #undef QIL_QK_CASE
+  QIL_RETURN_LAUNCH_STATUS();
+}
+
+// The same task with ONE norm over all query heads of a row and one over all its key heads (a norm of the whole
+// projection, before it is split into heads): x / sqrt(sum(x^2) / norm_elems + eps) * weight[column], then the rotation, in
+// float32 and rounded once.  Blocks 0 .. 2 n - 1 take a row's queries (even) or keys (odd), the row waiting in LDS
+// between the statistics and the result; the blocks behind them take the values, a wave 16 tokens x 4 chunks of 8
+// elements of one head, as in the vector kernel above.
+template <typename TD, typename T>
+__global__ void __launch_bounds__(256)
+qk_row_norm_store_kernel(const TD* __restrict__ qkv, int splits, size_t split_stride, T* __restrict__ q_out,
+                         const float* __restrict__ q_weight, const float* __restrict__ k_weight,
+                         const float* __restrict__ cos_table, const float* __restrict__ sin_table,
+                         const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ k_cache,
+                         T* __restrict__ v_cache, int n, int heads, int kv_heads, int d, int rot, int page_size, float eps,
+                         float q_elems, float k_elems, int row_elems, int v_head) {
+  extern __shared__ __align__(16) float row[];
+  __shared__ float scratch[16];
+  const int chunks = d / 8;
+  if ((int)blockIdx.x >= 2 * n) {                        // values: copied, transposed within the page
+    const int lane = threadIdx.x & (QIL_WAVE - 1), quads = (chunks + 3) / 4;
+    const size_t wave = (size_t)(blockIdx.x - 2 * n) * (blockDim.x / QIL_WAVE) + threadIdx.x / QIL_WAVE;
+    const int quad = (int)(wave % quads), kvh = (int)(wave / quads % kv_heads);
+    const size_t token = wave / quads / kv_heads * 16 + (lane >> 2);
+    const int chunk = quad * 4 + (lane & 3);
+    if (token >= (size_t)n || chunk >= chunks) return;
+    float x[8];
+    load8_sum(qkv, token * row_elems + (size_t)(v_head + kvh) * d + chunk * 8, splits, split_stride, x);
+    const int slot = slots[token];
+    const size_t page = slot / page_size, offset = slot % page_size;
+    T* column = v_cache + ((page * kv_heads + kvh) * (size_t)d + chunk * 8) * page_size + offset;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) st(column + (size_t)e * page_size, x[e]);
+    return;
+  }
+  const int token = blockIdx.x >> 1;
+  const bool is_k = blockIdx.x & 1;
+  if (is_k && slots == nullptr) return;                  // a reader of another entry's cache (the whole block)
+  const int count = (is_k ? kv_heads : heads) * chunks;
+  const size_t src = (size_t)token * row_elems + (is_k ? (size_t)heads * d : 0);
+  float sum = 0.f;
+  for (int c = threadIdx.x; c < count; c += blockDim.x) {
+    float x[8];
+    load8_sum(qkv, src + (size_t)c * 8, splits, split_stride, x);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum += x[e] * x[e];
+    store8(row + c * 8, x);
+  }
+  sum = block_sum(sum, scratch);                         // (its barriers also make the row whole)
+  const float rstd = 1.f / sqrtf(sum / (is_k ? k_elems : q_elems) + eps);
+  const float* weight = is_k ? k_weight : q_weight;
+  const int half = rot / 2, position = positions[token];
+  const bool rotates = cos_table && rot > 0;
+  size_t page = 0, offset = 0;
+  if (is_k) { page = slots[token] / page_size; offset = slots[token] % page_size; }
+  for (int c = threadIdx.x; c < count; c += blockDim.x) {
+    const int head = c / chunks, e0 = (c - head * chunks) * 8, base = head * d;
+    float y[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int i = e0 + e;
+      y[e] = row[base + i] * rstd * weight[base + i];
+      if (rotates && i < rot) {
+        const int f = i < half ? i : i - half, other = base + (i < half ? i + half : i - half);
+        float sn, cs;
+        if (sin_table) { cs = cos_table[(size_t)position * half + f]; sn = sin_table[(size_t)position * half + f]; }
+        else sincosf((float)position * cos_table[f], &sn, &cs);
+        const float z = row[other] * rstd * weight[other];
+        y[e] = i < half ? y[e] * cs - z * sn : z * sn + y[e] * cs;
+      }
+    }
+    T* dst = is_k ? k_cache + ((page * kv_heads + head) * page_size + offset) * (size_t)d + e0
+                  : q_out + ((size_t)token * heads + head) * d + e0;
+    store8(dst, y);
+  }
+}
+
+// qkv, caches, slots, rotation, shared_kv, extra_columns: as in qil_qk_norm_rope_store (no bias, no temperature).
+// q_weight float32 [heads * d], k_weight float32 [kv_heads * d]; q_elems, k_elems: the numbers of elements the two means
+// run over (fewer than heads * d where the heads are padded with zeros).  d % 8 == 0 and 16-byte aligned rows.
+extern "C" int qil_qk_row_norm_store(
+    const void* qkv, int in_dtype, int splits, void* q_out, const float* q_weight, const float* k_weight,
+    const float* cos_table, const float* sin_table, const int* positions, const int* slots, void* k_cache,
+    void* v_cache, int n, int heads, int kv_heads, int d, int rot, int page_size, float eps, int q_elems, int k_elems,
+    int extra_columns, int shared_kv, int dtype, hipStream_t s) {
+  if (n == 0) return 0;
+  if (heads < 1 || kv_heads < 1 || d < 8 || d % 8 || rot > d || (rot & 1) || splits < 1 || extra_columns < 0 ||
+      extra_columns % 8 || (in_dtype == QIL_BF16 && splits != 1) || (dtype == QIL_F32 && in_dtype != QIL_F32) ||
+      q_elems < 1 || q_elems > heads * d || k_elems < 1 || k_elems > kv_heads * d || !q_weight || !k_weight)
+    return -1;
+  const int row_elems = (heads + (shared_kv ? 1 : 2) * kv_heads) * d + extra_columns;
+  const int v_head = shared_kv ? heads : heads + kv_heads;
+  if (((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)q_weight | (uintptr_t)k_weight) % 16) return -1;
+  const size_t lds = (size_t)(heads > kv_heads ? heads : kv_heads) * d * sizeof(float);
+  if (lds > 128 * 1024) return -1;
+  const size_t v_waves = slots ? (size_t)((n + 15) / 16) * kv_heads * ((d / 8 + 3) / 4) : 0;
+  const dim3 grid((unsigned)(2 * (size_t)n + (v_waves + 3) / 4));
+  const size_t stride = (size_t)n * row_elems;
+#define QIL_ROW_NORM(TD, T)                                                                                           \
+  do {                                                                                                                \
+    if (lds > 60 * 1024) {                                                                                            \
+      hipError_t e = hipFuncSetAttribute((const void*)qk_row_norm_store_kernel<TD, T>,                                \
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);                       \
+      if (e != hipSuccess) return (int)e;                                                                             \
+    }                                                                                                                 \
+    hipLaunchKernelGGL((qk_row_norm_store_kernel<TD, T>), grid, dim3(256), lds, s, (const TD*)qkv, splits, stride,     \
+                       (T*)q_out, q_weight, k_weight, cos_table, sin_table, positions, slots, (T*)k_cache,            \
+                       (T*)v_cache, n, heads, kv_heads, d, rot, page_size, eps, (float)q_elems, (float)k_elems,        \
+                       row_elems, v_head);                                                                            \
+  } while (0)
+  if (dtype == QIL_F32) QIL_ROW_NORM(float, float);
+  else if (in_dtype == QIL_F32) QIL_ROW_NORM(float, bf16_t);
+  else QIL_ROW_NORM(bf16_t, bf16_t);
+#undef QIL_ROW_NORM
   QIL_RETURN_LAUNCH_STATUS();
 }

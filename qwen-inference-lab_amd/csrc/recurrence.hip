@@ -10,6 +10,9 @@
 //   QIL_SCAN_CHANNEL a decay of its own for every row of S (key channel i of head h) and token:
 //                   a_t[i] = sigmoid(z_t[h, i])^(1 / tau) = exp(logsigmoid(z_t[h, i]) / tau), b_t = 1, with z float32
 //                   [n, heads * dim] in the place of the gates and tau in the place of the cap; o_t as above.
+//   QIL_SCAN_STEP   a step size per head and token, d_t = softplus(raw_t[h] + bias[h]): a_t = exp(rate_h d_t), b_t = d_t
+//                   (rate_h in the place of the decay); o_t as above.  Queries and keys are shared by groups of heads:
+//                   head h reads those of group h / (heads / groups).  raw is an operand of its own (operand.h).
 // Queries and keys may be rotated by position first (the leading rot elements of a head, element i with i + rot / 2,
 // angle position * freq[i]) and are then scaled (q_scale, k_scale).  Gates, rotation, state and sums are float32.
 //
@@ -26,14 +29,17 @@
 // undivided, and the head-norm kernel divides.  The state slot of a sequence is read unless the sequence starts at
 // position 0, and written back at the end.
 #include "common.h"
+#include "operand.h"
 
-enum { QIL_SCAN_DECAY = 0, QIL_SCAN_MLSTM = 1, QIL_SCAN_CHANNEL = 2 };
+enum { QIL_SCAN_DECAY = 0, QIL_SCAN_MLSTM = 1, QIL_SCAN_CHANNEL = 2, QIL_SCAN_STEP = 3 };
 #define SCAN_CHUNK 16
 #define SCAN_COLUMNS 16                                          // state columns a block (one wave) owns
 
 __device__ __forceinline__ float log_sigmoid(float z) {         // -softplus(-z), stable on both sides
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
+
+__device__ __forceinline__ float scan_softplus(float v) { return v > 20.f ? v : log1pf(expf(v)); }
 
 // State of one slot: [heads][dim * vdim] matrices, then (MLSTM) [heads][dim] normalisers and [heads][tiles + 1] maxima,
 // tiles = ceil(vdim / 16): every block along z reads and writes only its own copy of the maximum, so no block sees
@@ -45,7 +51,7 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
                   const float* __restrict__ decay, const float* __restrict__ freq, int rot, float q_scale, float k_scale,
                   float* __restrict__ state, size_t slot_stride, const int* __restrict__ cu_seqlens,
                   const int* __restrict__ seq_starts, const int* __restrict__ seq_slots, float* __restrict__ out,
-                  float* __restrict__ below, int heads, int dim, int vdim) {
+                  float* __restrict__ below, int heads, int dim, int vdim, Operand raw, int raw_row, int groups) {
   constexpr int CH = DMAX > 128 ? SCAN_CHUNK / 2 : SCAN_CHUNK;  // tokens a chunk
   constexpr int PER = CH * DMAX / 64;                           // elements of q (and of k) a lane fetches a chunk
   __shared__ __align__(16) float qs[CH][DMAX];
@@ -80,7 +86,8 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
   float top = 0.f;
   if (MODE == QIL_SCAN_MLSTM && !fresh) top = *s_top;
   const int half = rot / 2;
-  const float fixed = MODE == QIL_SCAN_DECAY ? decay[h] : 0.f;
+  const float fixed = (MODE == QIL_SCAN_DECAY || MODE == QIL_SCAN_STEP) ? decay[h] : 0.f;
+  const int hq = MODE == QIL_SCAN_STEP ? h / (heads / groups) : h;             // whose queries and keys
 
   // What a lane fetches of a chunk, all requests sent before any is used: elements lane + 64 u of the chunk's
   // [CH][DMAX] queries and keys, its own column of every token's values, and one token's gate inputs.
@@ -91,7 +98,7 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
     for (int u = 0; u < PER; ++u) {
       const int idx = lane + 64 * u, t = idx / DMAX, i = idx % DMAX;
       const bool live = t < cn && i < dim;
-      const T* x = proj + (size_t)(c0 + (live ? t : 0)) * proj_row + h * dim + (live ? i : 0);
+      const T* x = proj + (size_t)(c0 + (live ? t : 0)) * proj_row + hq * dim + (live ? i : 0);
       rq[u] = live ? ld(x + q_off) : 0.f;
       rk[u] = live ? ld(x + k_off) : 0.f;
       if (MODE == QIL_SCAN_CHANNEL) rz[u] = live ? gates[(size_t)(c0 + t) * heads * dim + h * dim + i] : 0.f;
@@ -103,6 +110,7 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
       rgi = gates[(size_t)(c0 + lane) * 2 * heads + h];
       rgk = gates[(size_t)(c0 + lane) * 2 * heads + heads + h];
     }
+    if (MODE == QIL_SCAN_STEP && lane < cn) rgi = operand_at(raw, (size_t)(c0 + lane) * raw_row + h);
   };
   fetch(row0);
 
@@ -123,6 +131,11 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
     if (MODE == QIL_SCAN_MLSTM && lane < cn) {
       gi[lane] = cap * tanhf((rgi + gate_bias[h]) / cap);
       gk[lane] = log_sigmoid(cap * tanhf((rgk + gate_bias[heads + h]) / cap));
+    }
+    if (MODE == QIL_SCAN_STEP && lane < cn) {
+      const float step = scan_softplus(rgi + gate_bias[h]);
+      fa[lane] = expf(fixed * step);
+      fb[lane] = step;
     }
     __syncthreads();
     if (c0 + CH < row1) fetch(c0 + CH);                          // on its way while this chunk is walked
@@ -156,7 +169,8 @@ state_scan_kernel(const T* __restrict__ proj, int proj_row, int q_off, int k_off
     __syncthreads();
     if (!keeper) {
       for (int t = 0; t < cn; ++t) {
-        const float a = MODE == QIL_SCAN_MLSTM ? fa[t] : fixed, b = MODE == QIL_SCAN_MLSTM ? fb[t] : 1.f;
+        constexpr bool VARIES = MODE == QIL_SCAN_MLSTM || MODE == QIL_SCAN_STEP;
+        const float a = VARIES ? fa[t] : fixed, b = VARIES ? fb[t] : 1.f;
         const float bv = b * vs[t][jj];
         float o = 0.f;
 #pragma unroll
@@ -249,15 +263,21 @@ int qil_state_scan_takes(int dim, int vdim, int rot) {
 
 // proj [n, proj_row] (dtype): a row holds the heads' queries from q_off, keys from k_off (heads x dim each) and
 // values from v_off (heads x vdim).  gates [n, 2 heads] float32 (inputs first, then keeps), gate_bias [2 heads]: MLSTM.
+// STEP: raw (raw_code, raw_splits: an operand of rows of raw_row elements, split stride n * raw_row; row t's step size of
+// head h at t * raw_row + h), gate_bias [heads], decay [heads] = the rates; groups of queries and keys (1 .. heads).
 // CHANNEL: gates [n, heads * dim] float32 (z, one per row of every head's state) and cap = tau.
 // decay [heads]: DECAY.  freq [rot / 2] or rot == 0.  out [n, heads * vdim] float32; MLSTM: undivided, with every
 // token's denominator in below [n, heads].
 int qil_state_scan(const void* proj, int dtype, int proj_row, int q_off, int k_off, int v_off, const float* gates,
                    const float* gate_bias, float cap, const float* decay, const float* freq, int rot, float q_scale,
                    float k_scale, float* state, const int* cu_seqlens, const int* seq_starts, const int* seq_slots,
-                   float* out, float* below, int n_seqs, int heads, int dim, int vdim, int mode, hipStream_t s) {
+                   float* out, float* below, int n_seqs, int heads, int dim, int vdim, int mode, const void* raw,
+                   int raw_code, int raw_splits, int raw_row, int n, int groups, hipStream_t s) {
   if (n_seqs == 0) return 0;
-  if (!qil_state_scan_takes(dim, vdim, rot) || mode < QIL_SCAN_DECAY || mode > QIL_SCAN_CHANNEL) return -1;
+  if (!qil_state_scan_takes(dim, vdim, rot) || mode < QIL_SCAN_DECAY || mode > QIL_SCAN_STEP) return -1;
+  if (mode == QIL_SCAN_STEP && (!raw || !gate_bias || !decay || groups < 1 || heads % groups || rot || raw_splits < 1 ||
+                                (raw_code == QIL_BF16 && raw_splits != 1) || raw_row < heads)) return -1;
+  const Operand step_raw{raw, raw_code, raw_splits, (size_t)n * raw_row};
   if ((mode == QIL_SCAN_MLSTM && (!gates || !gate_bias || !below)) || (mode == QIL_SCAN_DECAY && !decay) ||
       (mode == QIL_SCAN_CHANNEL && (!gates || !(cap > 0.f))) || (rot && !freq)) return -1;
   const size_t slot_stride = qil_state_scan_slot(heads, dim, vdim, mode);
@@ -265,7 +285,7 @@ int qil_state_scan(const void* proj, int dtype, int proj_row, int q_off, int k_o
 #define QIL_SCAN(T, DMAX, MODE)                                                                                      \
   hipLaunchKernelGGL((state_scan_kernel<T, DMAX, MODE>), grid, dim3(64), 0, s, (const T*)proj, proj_row, q_off, k_off, \
                      v_off, gates, gate_bias, cap, decay, freq, rot, q_scale, k_scale, state, slot_stride, cu_seqlens, \
-                     seq_starts, seq_slots, out, below, heads, dim, vdim)
+                     seq_starts, seq_slots, out, below, heads, dim, vdim, step_raw, raw_row, groups)
 #define QIL_SCAN_DIM(T, MODE)                                                                                        \
   do {                                                                                                               \
     if (dim <= 32) QIL_SCAN(T, 32, MODE);                                                                            \
@@ -276,10 +296,12 @@ int qil_state_scan(const void* proj, int dtype, int proj_row, int q_off, int k_o
   if (dtype == QIL_F32) {
     if (mode == QIL_SCAN_MLSTM) QIL_SCAN_DIM(float, QIL_SCAN_MLSTM);
     else if (mode == QIL_SCAN_CHANNEL) QIL_SCAN_DIM(float, QIL_SCAN_CHANNEL);
+    else if (mode == QIL_SCAN_STEP) QIL_SCAN_DIM(float, QIL_SCAN_STEP);
     else QIL_SCAN_DIM(float, QIL_SCAN_DECAY);
   } else {
     if (mode == QIL_SCAN_MLSTM) QIL_SCAN_DIM(bf16_t, QIL_SCAN_MLSTM);
     else if (mode == QIL_SCAN_CHANNEL) QIL_SCAN_DIM(bf16_t, QIL_SCAN_CHANNEL);
+    else if (mode == QIL_SCAN_STEP) QIL_SCAN_DIM(bf16_t, QIL_SCAN_STEP);
     else QIL_SCAN_DIM(bf16_t, QIL_SCAN_DECAY);
   }
 #undef QIL_SCAN_DIM
@@ -302,3 +324,82 @@ int qil_head_norm_gate(const float* o, const float* below, const void* g, int g_
 }
 
 }  // extern "C"
+
+// y[n, j] = o[n, j] + skip[head of j] * u[n, j], times silu(z[n, j]); then every one of the row's `groups` equal parts is
+// divided by its root mean square (eps inside the root) and multiplied by weight[j].  float32 until the one rounding.
+// One block per (row, part); V neighbouring columns a thread.
+template <typename T, int V>
+__global__ void gated_group_norm_kernel(const float* __restrict__ o, const T* __restrict__ u, int u_row,
+                                        const float* __restrict__ skip, Operand z, int z_row, const float* __restrict__ weight,
+                                        T* __restrict__ y, int y_row, int vdim, int size, float eps, float scale) {
+  extern __shared__ __align__(16) float held[];
+  __shared__ float scratch[16];
+  const int n = blockIdx.x, first = blockIdx.y * size;
+  float squares = 0.f;
+  for (int i = threadIdx.x * V; i < size; i += blockDim.x * V) {
+    const int j = first + i;
+    float a[V], b[V], g[V];
+    const size_t at = (size_t)n * gridDim.y * size + j;
+    if constexpr (V == 4) {
+      const float4 a4 = ld4(o + at), b4 = ld4(u + (size_t)n * u_row + j), g4 = operand_at4(z, (size_t)n * z_row + j);
+      a[0] = a4.x; a[1] = a4.y; a[2] = a4.z; a[3] = a4.w;
+      b[0] = b4.x; b[1] = b4.y; b[2] = b4.z; b[3] = b4.w;
+      g[0] = g4.x; g[1] = g4.y; g[2] = g4.z; g[3] = g4.w;
+    } else {
+      a[0] = o[at]; b[0] = ld(u + (size_t)n * u_row + j); g[0] = operand_at(z, (size_t)n * z_row + j);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const float v = (a[e] + skip[(j + e) / vdim] * b[e]) * (g[e] / (1.f + expf(-g[e])));
+      held[i + e] = v;
+      squares += v * v;
+    }
+  }
+  squares = block_sum(squares, scratch);
+  const float unit = scale / sqrtf(squares / (float)size + eps);
+  for (int i = threadIdx.x * V; i < size; i += blockDim.x * V) {       // (a thread meets its own elements again)
+    const int j = first + i;
+    T* to = y + (size_t)n * y_row + j;
+    if constexpr (V == 4) {
+      const float4 w = ld4(weight + j);
+      st4(to, make_float4(held[i] * unit * w.x, held[i + 1] * unit * w.y, held[i + 2] * unit * w.z, held[i + 3] * unit * w.w));
+    } else {
+      st(to, held[i] * unit * weight[j]);
+    }
+  }
+}
+
+// o float32 [n, inner]; u [n, u_row] of dtype (its first inner columns); skip float32 [inner / vdim]; z an operand of rows
+// of z_row elements (split stride n * z_row) whose first inner columns are read; weight float32 [inner]; y rows of y_row
+// elements of dtype; inner = groups * size.  scale: a factor on the result.
+extern "C" int qil_gated_group_norm(const float* o, const void* u, int u_row, const float* skip, const void* z, int z_code,
+                                    int z_splits, int z_row, const float* weight, void* y, int y_row, int n, int inner,
+                                    int vdim, int groups, float eps, float scale, int dtype, hipStream_t s) {
+  if (n == 0) return 0;
+  if (inner < 1 || groups < 1 || inner % groups || vdim < 1 || inner % vdim || u_row < inner || z_row < inner ||
+      y_row < inner || z_splits < 1 || (z_code == QIL_BF16 && z_splits != 1) || groups > 65535 || !skip || !weight)
+    return -1;
+  const int size = inner / groups;
+  const size_t lds = (size_t)size * sizeof(float);
+  if (lds > 128 * 1024) return -1;
+  const Operand gate{z, z_code, z_splits, (size_t)n * z_row};
+  const bool vec = size % 4 == 0 && u_row % 4 == 0 && z_row % 4 == 0 && y_row % 4 == 0 &&
+                   (((uintptr_t)o | (uintptr_t)u | (uintptr_t)z | (uintptr_t)weight | (uintptr_t)y) % 16) == 0;
+  const int lanes = vec ? size / 4 : size;
+  const int threads = lanes >= 512 ? 512 : (lanes + 63) / 64 * 64;
+  const dim3 grid(n, groups);
+#define QIL_GROUP_NORM(T, V)                                                                                          \
+  do {                                                                                                                \
+    if (lds > 60 * 1024) {                                                                                            \
+      hipError_t e = hipFuncSetAttribute((const void*)gated_group_norm_kernel<T, V>,                                  \
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);                       \
+      if (e != hipSuccess) return (int)e;                                                                             \
+    }                                                                                                                 \
+    hipLaunchKernelGGL((gated_group_norm_kernel<T, V>), grid, dim3(threads), lds, s, o, (const T*)u, u_row, skip, gate, \
+                       z_row, weight, (T*)y, y_row, vdim, size, eps, scale);                                          \
+  } while (0)
+  if (dtype == QIL_F32) { if (vec) QIL_GROUP_NORM(float, 4); else QIL_GROUP_NORM(float, 1); }
+  else { if (vec) QIL_GROUP_NORM(bf16_t, 4); else QIL_GROUP_NORM(bf16_t, 1); }
+#undef QIL_GROUP_NORM
+  QIL_RETURN_LAUNCH_STATUS();
+}

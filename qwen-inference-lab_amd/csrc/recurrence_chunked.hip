@@ -23,9 +23,14 @@
 //     o_t = S_in^T (q_t * 2^G_t) + sum_(s <= t) (sum_i q_t[i] k_s[i] 2^(G_t[i] - G_s[i])) v_s
 // so `sums` weighs row i of k_s by 2^(G_end[i] - G_s[i]), `carry` keeps row i by 2^G_end[i], and `outputs` makes the
 // scores inside the block with the weight inside the sum over i (every exponent <= 0: nothing is divided by a decay).
+//
+// QIL_SCAN_STEP (a step size d_t per head and token, a_t = exp(rate d_t), b_t = d_t): with F_t the block's sum of rate d,
+//     S_t = exp(F_t) S_in + sum_(s <= t) exp(F_t - F_s) d_s k_s v_s^T
+// every exponent <= 0 again.  Queries and keys are shared by groups of heads and read where they lie: nothing to rotate.
 #include "common.h"
+#include "operand.h"
 
-enum { QIL_SCAN_DECAY = 0, QIL_SCAN_MLSTM = 1, QIL_SCAN_CHANNEL = 2 };
+enum { QIL_SCAN_DECAY = 0, QIL_SCAN_MLSTM = 1, QIL_SCAN_CHANNEL = 2, QIL_SCAN_STEP = 3 };
 #define SCAN_BLOCK 64
 #define SCAN_TOP_TILE 16                                         // recurrence.hip keeps one maximum per 16 state columns
 
@@ -50,6 +55,25 @@ __device__ __forceinline__ GateLane gate_lane(const float* __restrict__ gates, c
   g.sum = sum;
   g.lead = live ? (double)in - sum : -INFINITY;
   return g;
+}
+
+// STEP, lane t: F_t and the step size d_t of token t (0 past the block's end).
+struct StepInput { Operand raw; int row, q_off, k_off, groups; };
+struct StepLane { double sum; float step; };
+__device__ __forceinline__ StepLane step_lane(const StepInput& in, const float* __restrict__ bias, float rate, int row, int h,
+                                              bool live, int lane) {
+  float step = 0.f;
+  if (live) {
+    const float v = operand_at(in.raw, (size_t)row * in.row + h) + bias[h];
+    step = v > 20.f ? v : log1pf(expf(v));
+  }
+  double sum = (double)(rate * step);
+#pragma unroll
+  for (int d = 1; d < QIL_WAVE; d <<= 1) {
+    const double up = __shfl_up(sum, d, QIL_WAVE);
+    if (lane >= d) sum += up;
+  }
+  return {sum, step};
 }
 
 // Where block c of sequence seq keeps its sums: sequences before it took at most row0 / SCAN_BLOCK + seq places.
@@ -110,7 +134,7 @@ scan_sums_kernel(const T* __restrict__ proj, int proj_row, int v_off, const floa
                  const int* __restrict__ cu_seqlens, const int* __restrict__ seq_starts, const int* __restrict__ seq_slots,
                  float* __restrict__ sums, float* __restrict__ norm_sums, double* __restrict__ info,
                  float* __restrict__ carried, int heads, int dim, int vdim, int dim_tiles,
-                 const float* __restrict__ gsum) {
+                 const float* __restrict__ gsum, StepInput steps) {
   __shared__ __align__(16) float kw[SCAN_BLOCK][64];
   __shared__ __align__(16) float vs[SCAN_BLOCK][64];
   __shared__ float w[SCAN_BLOCK];
@@ -140,6 +164,11 @@ scan_sums_kernel(const T* __restrict__ proj, int proj_row, int v_off, const floa
           carried[at] = seq_starts[seq] == 0 ? 0.f : *s_top;
         }
       }
+    } else if (MODE == QIL_SCAN_STEP) {
+      const StepLane g = step_lane(steps, gate_bias, decay[h], r0 + (live ? tid : 0), h, live, tid);
+      const double total = __shfl(g.sum, lc - 1, QIL_WAVE);
+      weight = live ? expf((float)(total - g.sum)) * g.step : 0.f;
+      if (blockIdx.z == 0 && tid == 0) info[at * 2] = total;
     } else if (MODE == QIL_SCAN_CHANNEL) {
       weight = live ? 1.f : 0.f;                                 // (the rows' own weights follow below)
     } else {
@@ -149,13 +178,17 @@ scan_sums_kernel(const T* __restrict__ proj, int proj_row, int v_off, const floa
   }
   __syncthreads();
   const size_t hd = (size_t)heads * dim;
+  const int group = MODE == QIL_SCAN_STEP ? h / (heads / steps.groups) : h;
   for (int idx = tid; idx < SCAN_BLOCK * 64; idx += 256) {
     const int s = idx / 64, x = idx % 64, i = it * 64 + x, j = jt * 64 + x;
     float weight = w[s];
     if (MODE == QIL_SCAN_CHANNEL && s < lc && i < dim)
       weight = __builtin_amdgcn_exp2f(gsum[(size_t)(r0 + lc - 1) * hd + (size_t)h * dim + i] -
                                       gsum[(size_t)(r0 + s) * hd + (size_t)h * dim + i]);
-    kw[s][x] = (s < lc && i < dim) ? weight * qk[(size_t)(r0 + s) * 2 * hd + hd + (size_t)h * dim + i] : 0.f;
+    if (MODE == QIL_SCAN_STEP)
+      kw[s][x] = (s < lc && i < dim) ? weight * ld(proj + (size_t)(r0 + s) * proj_row + steps.k_off + group * dim + i) : 0.f;
+    else
+      kw[s][x] = (s < lc && i < dim) ? weight * qk[(size_t)(r0 + s) * 2 * hd + hd + (size_t)h * dim + i] : 0.f;
     vs[s][x] = (s < lc && j < vdim) ? ld(proj + (size_t)(r0 + s) * proj_row + v_off + h * vdim + j) : 0.f;
   }
   __syncthreads();
@@ -217,6 +250,8 @@ scan_carry_kernel(float* __restrict__ sums, float* __restrict__ norm_sums, const
       take = expf((float)(local - end));
       if (e == 0) carried[at] = top;
       top = (float)(info[at * 2 + 1] + end);
+    } else if (MODE == QIL_SCAN_STEP) {
+      keep = expf((float)info[at * 2]);
     } else if (MODE == QIL_SCAN_CHANNEL) {
       const int last = row0 + min((c + 1) * SCAN_BLOCK, len) - 1;       // the block's last token
       keep = __builtin_amdgcn_exp2f(gsum[(size_t)last * heads * dim + (size_t)h * dim + e / vdim]);
@@ -241,7 +276,8 @@ scan_outputs_kernel(const T* __restrict__ proj, int proj_row, int v_off, const f
                     const float* __restrict__ gates, const float* __restrict__ gate_bias, float cap,
                     const float* __restrict__ decay, const float* __restrict__ before, const float* __restrict__ norm_before,
                     const float* __restrict__ carried, const int* __restrict__ cu_seqlens, float* __restrict__ out,
-                    float* __restrict__ below, int heads, int dim, int vdim, const float* __restrict__ gsum) {
+                    float* __restrict__ below, int heads, int dim, int vdim, const float* __restrict__ gsum,
+                    StepInput steps) {
   // first the slabs [q^T | k^T | S_in rows] (CHANNEL: and [G^T | (q 2^G)^T]), then [weighted scores^T | v]
   constexpr bool CHANNEL = MODE == QIL_SCAN_CHANNEL;
   __shared__ __align__(16) float stage[SCAN_BLOCK * OUT_PAD + SCAN_BLOCK * 64 + (CHANNEL ? 2 * OUT_SLAB * OUT_PAD : 0)];
@@ -275,6 +311,12 @@ scan_outputs_kernel(const T* __restrict__ proj, int proj_row, int v_off, const f
       tops[tid] = top;
       cw[tid] = expf((float)(brought - top));
       em[tid] = expf(-(float)(g.sum + top));
+    } else if (MODE == QIL_SCAN_STEP) {
+      const bool live = tid < lc;
+      const StepLane g = step_lane(steps, gate_bias, decay[h], r0 + (live ? tid : 0), h, live, tid);
+      tops[tid] = g.sum;
+      cw[tid] = expf((float)g.sum);
+      em[tid] = g.step;
     } else if (!CHANNEL) {
       pw[tid] = (float)pow((double)decay[h], (double)tid);
       if (tid == 0) pw[SCAN_BLOCK] = (float)pow((double)decay[h], (double)SCAN_BLOCK);
@@ -282,6 +324,7 @@ scan_outputs_kernel(const T* __restrict__ proj, int proj_row, int v_off, const f
   }
   const int ti = tid / 16, tj = tid % 16;
   const size_t hd = (size_t)heads * dim;
+  const int group = MODE == QIL_SCAN_STEP ? h / (heads / steps.groups) : h;
   const float* s_in = before + at * dim * vdim;
   float p[4][4] = {}, o[4][4] = {}, nq[4] = {};
   for (int i0 = 0; i0 < dim; i0 += OUT_SLAB) {
@@ -289,6 +332,12 @@ scan_outputs_kernel(const T* __restrict__ proj, int proj_row, int v_off, const f
     for (int idx = tid; idx < SCAN_BLOCK * OUT_SLAB; idx += 256) {
       const int t = idx / OUT_SLAB, x = idx % OUT_SLAB, i = i0 + x;
       const bool ok = t < lc && i < dim;
+      if (MODE == QIL_SCAN_STEP) {
+        const T* row = proj + (size_t)(r0 + (ok ? t : 0)) * proj_row + group * dim + (ok ? i : 0);
+        qT[x * OUT_PAD + t] = ok ? ld(row + steps.q_off) : 0.f;
+        kT[x * OUT_PAD + t] = ok ? ld(row + steps.k_off) : 0.f;
+        continue;
+      }
       const float* src = qk + (size_t)(r0 + (ok ? t : 0)) * 2 * hd + (size_t)h * dim + (ok ? i : 0);
       qT[x * OUT_PAD + t] = ok ? src[0] : 0.f;
       kT[x * OUT_PAD + t] = ok ? src[hd] : 0.f;
@@ -345,13 +394,16 @@ scan_outputs_kernel(const T* __restrict__ proj, int proj_row, int v_off, const f
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int t = ti * 4 + r;
-    const float brought = MODE == QIL_SCAN_MLSTM ? cw[t] : CHANNEL ? 1.f : pw[t + 1];
+    const float brought = (MODE == QIL_SCAN_MLSTM || MODE == QIL_SCAN_STEP) ? cw[t] : CHANNEL ? 1.f : pw[t + 1];
     float row_sum = 0.f;
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int s = tj * 4 + u;
       float weight = 0.f;
-      if (s <= t && t < lc) weight = MODE == QIL_SCAN_MLSTM ? expf((float)(lead[s] - tops[t])) : CHANNEL ? 1.f : pw[t - s];
+      if (s <= t && t < lc)
+        weight = MODE == QIL_SCAN_MLSTM ? expf((float)(lead[s] - tops[t]))
+                 : MODE == QIL_SCAN_STEP ? expf((float)(tops[t] - tops[s])) * em[s]
+                 : CHANNEL ? 1.f : pw[t - s];
       p[r][u] *= weight;
       row_sum += p[r][u];
       o[r][u] *= brought;
@@ -402,7 +454,8 @@ extern "C" {
 // Floats of the scratch memory of a step of n rows in n_seqs sequences.
 size_t qil_state_scan_chunked_workspace(int n, int n_seqs, int heads, int dim, int vdim, int mode) {
   const size_t places = chunked_places(n, n_seqs);
-  size_t floats = places * heads * 4 + (places * heads + 3) / 4 * 4 + (size_t)n * 2 * heads * dim + places * heads * dim * vdim;
+  size_t floats = places * heads * 4 + (places * heads + 3) / 4 * 4 + places * heads * dim * vdim;
+  if (mode != QIL_SCAN_STEP) floats += (size_t)n * 2 * heads * dim;
   if (mode == QIL_SCAN_MLSTM) floats += places * heads * dim;
   if (mode == QIL_SCAN_CHANNEL) floats += (size_t)n * heads * dim;
   return floats;
@@ -413,18 +466,22 @@ int qil_state_scan_chunked(const void* proj, int dtype, int proj_row, int q_off,
                            const float* gate_bias, float cap, const float* decay, const float* freq, int rot, float q_scale,
                            float k_scale, float* state, size_t slot_stride, const int* cu_seqlens, const int* seq_starts,
                            const int* seq_slots, float* out, float* below, float* workspace, int n, int n_seqs,
-                           int max_query, int heads, int dim, int vdim, int mode, hipStream_t s) {
+                           int max_query, int heads, int dim, int vdim, int mode, const void* raw, int raw_code,
+                           int raw_splits, int raw_row, int groups, hipStream_t s) {
   if (n_seqs == 0 || n == 0) return 0;
   if (dim < 1 || vdim < 1 || rot < 0 || rot % 2 || rot > dim || max_query < 1 ||
-      mode < QIL_SCAN_DECAY || mode > QIL_SCAN_CHANNEL || !workspace || (size_t)n_seqs * heads > 65535)
+      mode < QIL_SCAN_DECAY || mode > QIL_SCAN_STEP || !workspace || (size_t)n_seqs * heads > 65535)
     return -1;
   if ((mode == QIL_SCAN_MLSTM && (!gates || !gate_bias || !below)) || (mode == QIL_SCAN_DECAY && !decay) ||
       (mode == QIL_SCAN_CHANNEL && (!gates || !(cap > 0.f) || n_seqs > 65535)) || (rot && !freq)) return -1;
+  if (mode == QIL_SCAN_STEP && (!raw || !gate_bias || !decay || groups < 1 || heads % groups || rot || raw_splits < 1 ||
+                                (raw_code == QIL_BF16 && raw_splits != 1) || raw_row < heads)) return -1;
+  const StepInput steps{{raw, raw_code, raw_splits, (size_t)n * raw_row}, raw_row, q_off, k_off, groups};
   const size_t places = chunked_places(n, n_seqs);
   double* info = reinterpret_cast<double*>(workspace);
   float* carried = workspace + places * heads * 4;
   float* qk = carried + (places * heads + 3) / 4 * 4;
-  float* sums = qk + (size_t)n * 2 * heads * dim;
+  float* sums = qk + (mode == QIL_SCAN_STEP ? 0 : (size_t)n * 2 * heads * dim);
   float* norm_sums = sums + places * heads * dim * vdim;
   float* gsum = norm_sums;                                       // CHANNEL has no normaliser: its place holds the decays' sums
   const int blocks = (max_query + SCAN_BLOCK - 1) / SCAN_BLOCK;
@@ -437,24 +494,27 @@ int qil_state_scan_chunked(const void* proj, int dtype, int proj_row, int q_off,
     if (MODE == QIL_SCAN_CHANNEL)                                                                                     \
       hipLaunchKernelGGL(scan_decays_kernel, dim3(blocks, n_seqs, (heads * dim + 255) / 256), dim3(256), 0, s, gates,  \
                          cap, cu_seqlens, gsum, heads * dim);                                                          \
+    if (MODE != QIL_SCAN_STEP)                                                                                        \
     hipLaunchKernelGGL(scan_rotate_kernel<T>, dim3(n), dim3(256), 0, s, (const T*)proj, proj_row, q_off, k_off, freq,  \
                        rot, q_scale, k_scale, cu_seqlens, seq_starts, n_seqs, qk, heads, dim);                         \
     hipLaunchKernelGGL((scan_sums_kernel<T, MODE>), g_sums, dim3(256), 0, s, (const T*)proj, proj_row, v_off, qk,      \
                        gates, gate_bias, cap, decay, state, slot_stride, cu_seqlens, seq_starts, seq_slots, sums,      \
-                       norm_sums, info, carried, heads, dim, vdim, dim_tiles, gsum);                                   \
+                       norm_sums, info, carried, heads, dim, vdim, dim_tiles, gsum, steps);                            \
     hipLaunchKernelGGL(scan_carry_kernel<MODE>, g_carry, dim3(256), 0, s, sums, norm_sums, info, carried, decay,       \
                        state, slot_stride, cu_seqlens, seq_starts, seq_slots, heads, dim, vdim, gsum);                 \
     hipLaunchKernelGGL((scan_outputs_kernel<T, MODE>), g_out, dim3(256), 0, s, (const T*)proj, proj_row, v_off, qk,    \
                        gates, gate_bias, cap, decay, sums, norm_sums, carried, cu_seqlens, out, below, heads, dim,     \
-                       vdim, gsum);                                                                                    \
+                       vdim, gsum, steps);                                                                             \
   } while (0)
   if (dtype == QIL_F32) {
     if (mode == QIL_SCAN_MLSTM) QIL_CHUNKED(float, QIL_SCAN_MLSTM);
     else if (mode == QIL_SCAN_CHANNEL) QIL_CHUNKED(float, QIL_SCAN_CHANNEL);
+    else if (mode == QIL_SCAN_STEP) QIL_CHUNKED(float, QIL_SCAN_STEP);
     else QIL_CHUNKED(float, QIL_SCAN_DECAY);
   } else {
     if (mode == QIL_SCAN_MLSTM) QIL_CHUNKED(bf16_t, QIL_SCAN_MLSTM);
     else if (mode == QIL_SCAN_CHANNEL) QIL_CHUNKED(bf16_t, QIL_SCAN_CHANNEL);
+    else if (mode == QIL_SCAN_STEP) QIL_CHUNKED(bf16_t, QIL_SCAN_STEP);
     else QIL_CHUNKED(bf16_t, QIL_SCAN_DECAY);
   }
 #undef QIL_CHUNKED

@@ -39,13 +39,15 @@ class StepContext:
     host_starts: list = field(default_factory=list)
     host_slots: list = field(default_factory=list)
     requests: list = field(default_factory=list)
+    previous_tokens: torch.Tensor = None   # [N] the token before each row's in its sequence (-1: none), for embeddings
+                                           # that ask for it (``needs_previous_tokens``)
     tile_seqs: int = None          # sequences 0 .. tile_seqs - 1 are those of two or more rows; None: any may be
 
 
 class StepPieces:
     """The integer arrays that describe a step, by name, and where each lies once they are laid end to end into
     the one int32 array that goes to the device.  Names: ``tokens``, ``positions``, ``row_seq``, ``cu_seqlens``,
-    ``starts``, ``slots``, ``logit_rows``, ``single_rows``, and per page group g ``tables<g>`` (the block tables,
+    ``starts``, ``slots``, ``logit_rows``, ``single_rows``, ``previous`` (if the embedding asks for it), and per page group g ``tables<g>`` (the block tables,
     row-major) and ``token_slots<g>`` (the cache slot of every new token)."""
 
     def __init__(self):

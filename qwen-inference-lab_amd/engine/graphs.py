@@ -132,6 +132,9 @@ class _Graph:
         put('tokens', [e.tokens[0] for e in entries], 0)
         put('positions', starts, 0)
         put('starts', starts, 0)                            # where the requests' rows begin
+        if runner.previous_tokens:
+            last = [cache.last_tokens[e.request] for e in entries]
+            put('previous', [-1 if token is None else token for token in last], -1)
         put('slots', [cache.slots[e.request] for e in entries], spare_slot)
         for group, width in enumerate(self.widths):
             tables_at, slots_at, written = spans[f'tables{group}'][0], spans[f'token_slots{group}'][0], self.written[group]

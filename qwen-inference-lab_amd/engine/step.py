@@ -28,6 +28,7 @@ class ModelRunner:
                                   max_requests=max_requests, dtype=model.dtype, device=model.device,
                                   max_step_tokens=max_step_tokens)
         self.views = self.cache.views()
+        self.previous_tokens = bool(getattr(model.embedding, 'needs_previous_tokens', False))
         self.steps = 0
         self.graphs = DecodeGraphs(self) if graphs and self.model.device.type == 'cuda' else None
 
@@ -107,6 +108,11 @@ class ModelRunner:
         for name, array in (('tokens', tokens), ('positions', positions), ('row_seq', row_seq), ('cu_seqlens', cu),
                             ('starts', starts), ('slots', slots), ('logit_rows', logit_rows), ('single_rows', single)):
             pieces.add(name, array)
+        if self.previous_tokens:
+            previous = np.concatenate(([-1], tokens[:-1])) if n else tokens
+            last = [cache.last_tokens[e.request] for e in entries] + [None] * pad_rows
+            previous[cu[:-1]] = [-1 if token is None else token for token in last]
+            pieces.add('previous', previous)
         widths = []
         for index, group in enumerate(cache.kv_groups):
             tables = [cache.table(index, e.request) for e in entries] + [[cache.spare_page(index)]] * pad_rows
@@ -142,6 +148,8 @@ class ModelRunner:
                 values = np.zeros_like(values)
             elif name == 'positions':
                 values = positions
+            elif name == 'previous':
+                values = np.full_like(values, -1)
             elif name == 'slots':
                 values = np.full_like(values, cache.spare_slot)
             elif name.startswith('tables'):
@@ -162,7 +170,8 @@ class ModelRunner:
             seq_slots=part('slots'), logit_rows=part('logit_rows'),
             single_rows=part('single_rows') if max(counts) > 1 else None, max_query=max(counts),
             max_context=max_context or facts['max_context'], host_cu_seqlens=facts['cu'], host_starts=facts['starts'],
-            host_slots=facts['slots'], requests=[e.request for e in entries], tile_seqs=facts['tile_seqs'])
+            host_slots=facts['slots'], requests=[e.request for e in entries], tile_seqs=facts['tile_seqs'],
+            previous_tokens=part('previous') if self.previous_tokens else None)
         for view in (one for view in self.views for one in (view if isinstance(view, tuple) else (view,))):
             if view is not None and hasattr(view, 'block_tables'):
                 view.block_tables = part(f'tables{view.group}').view(s, facts['widths'][view.group])
@@ -184,7 +193,7 @@ class ModelRunner:
         replayed = self.graphs.step(entries) if self.graphs is not None and self.graphs.takes(entries) else None
         logits, entries, starts = replayed if replayed is not None else self._forward(entries)
         for entry, start in zip(entries, starts):
-            self.cache.advance(entry.request, start + len(entry.tokens))
+            self.cache.advance(entry.request, start + len(entry.tokens), entry.tokens[-1])
         self.steps += 1
         return logits
 
@@ -217,6 +226,6 @@ class ModelRunner:
                 sampler.draw(logits, torch.from_numpy(packed).to(logits.device), out)
                 drawn = out.tolist()
         for entry, start in zip(entries, starts):
-            self.cache.advance(entry.request, start + len(entry.tokens))
+            self.cache.advance(entry.request, start + len(entry.tokens), entry.tokens[-1])
         self.steps += 1
         return sampler.unpack(drawn) if drawn is not None else []

@@ -4,3 +4,4 @@ from . import fubapel  # noqa: F401
 from . import gerivik  # noqa: F401
 from . import zinesun  # noqa: F401
 from . import dogozen  # noqa: F401
+from . import tinuzen  # noqa: F401

@@ -99,6 +99,75 @@ class Partials:
         return self.tensor.sum(dim=0)
 
 
+class Columns:
+    """Neighbouring columns of a stacked product: ``source`` is the product ([N, R] tensor of the model's type, or
+    ``Partials`` of it), the columns from ``offset`` on are meant.  Consumers that read rows of a larger array take it
+    where they take a tensor or ``Partials``."""
+
+    def __init__(self, source, offset, columns):
+        if isinstance(source, Columns):
+            source, offset = source.source, source.offset + offset
+        n, row = source.shape
+        if offset < 0 or columns < 1 or offset + columns > row:
+            raise ValueError(f'columns {offset} .. {offset + columns} do not lie inside a row of {row}')
+        self.source, self.offset, self.row, self.shape = source, int(offset), int(row), (n, int(columns))
+        self.device = source.device
+
+
+def columns(value, offset, count):
+    """The columns [offset, offset + count) of a tensor, ``Partials`` or ``Columns``."""
+    return Columns(value, offset, count)
+
+
+class SharedInput:
+    """The input ``x`` of several matrices that one product serves: ``stack`` [R, K] holds their rows one behind
+    another and ``places`` maps id(matrix) to its first row there.  ``linear`` of a matrix that is in the stack is the
+    ``Columns`` of the product with the whole stack, which is made once, when it is first asked for."""
+
+    def __init__(self, x, stack, places):
+        self.x, self.stack, self.places, self._product = x, stack, places, None
+        self.shape, self.dtype, self.device = tuple(x.shape), x.dtype, x.device
+
+    def product(self):
+        if self._product is None:
+            self._product = linear(self.x, self.stack, None, partials=True)
+        return self._product
+
+
+class Weighted:
+    """left_scale * left + right_scale * right, not summed yet (each a tensor of the model's type or ``Partials``)."""
+
+    def __init__(self, left, right, left_scale, right_scale):
+        self.left, self.right, self.left_scale, self.right_scale = left, right, float(left_scale), float(right_scale)
+        self.shape, self.device = tuple(left.shape), left.device
+
+    def materialize(self):
+        return scaled_sum(self.left, self.right, self.left_scale, self.right_scale)
+
+
+class Joined:
+    """What a layer with gated branches side by side leaves for the stream, not added yet:
+
+        stream += sigmoid(gates[:, :H] + bias[:H]) * mixed + sigmoid(gates[:, H:] + bias[H:]) * ffn + plus + step
+
+    ``mixed``: a tensor of the model's type, ``Partials`` or ``Weighted``; ``ffn`` the same or None; ``gates``
+    (tensor, ``Partials`` or ``Columns``, the logits) None: the factors are 1; ``plus`` float32 [N, H] and ``step``
+    float32 [H]: what the start of a pass over the layers adds (``joined_with_pass``).  Without anything it is a
+    complete stream.  ``residual_join`` makes the sum and the norm that follows in one kernel."""
+
+    def __init__(self, mixed=None, ffn=None, gates=None, bias=None, plus=None, step=None):
+        self.mixed, self.ffn, self.gates, self.bias, self.plus, self.step = mixed, ffn, gates, bias, plus, step
+
+
+def joined_with_pass(pending, plus, step):
+    """A pending output together with what a pass adds before its first layer."""
+    if pending is None or (isinstance(pending, Added) and not isinstance(pending, Averaged)):
+        pending = Joined()
+    if not isinstance(pending, Joined):
+        raise TypeError(f'a pass cannot begin behind a pending {type(pending).__name__}')
+    return Joined(pending.mixed, pending.ffn, pending.gates, pending.bias, plus, step)
+
+
 class Unmerged:
     """Attention of single rows left as the float32 partial results of the context's parts (rows 0 .. N-1
     of the step, all alone in their sequences).  ``merge()`` gives the [N, heads * d] tensor; ``linear``
@@ -112,7 +181,7 @@ class Unmerged:
     def merge(self):
         _check(library.load().qil_attn_merge(_ptr(self.workspace), _ptr(self.positions), None, _ptr(self.out),
                                              self.shape[0], self.heads, self.head_dim, self.window, self.part,
-                                             self.parts, _code(self.dtype), None, _stream()), 'attn_merge')
+                                             self.parts, _code(self.dtype), None, 0, _stream()), 'attn_merge')
         return self.out
 
 
@@ -245,6 +314,21 @@ def _operand(value, name, model_dtype, shape):
     return value.data_ptr(), _code(model_dtype), 1
 
 
+def _row_operand(value, name, n, width, dtypes=None):
+    """(pointer, dtype code, splits, elements of a row) of rows of ``width`` columns: a tensor, Partials or Columns."""
+    source, offset = (value.source, value.offset) if isinstance(value, Columns) else (value, 0)
+    if tuple(value.shape) != (n, width):
+        raise ValueError(f'{name} must have shape {(n, width)}, has {tuple(value.shape)}')
+    row = source.shape[1]
+    if isinstance(source, Partials):
+        _require(source.tensor, name, torch.float32, (source.splits, n, row))
+        return source.tensor.data_ptr() + 4 * offset, 0, source.splits, row
+    _require(source, name, None, (n, row))
+    if dtypes is not None and source.dtype not in dtypes:
+        raise ValueError(f'{name} must be one of {dtypes}, is {source.dtype}')
+    return source.data_ptr() + source.element_size() * offset, _code(source.dtype), 1, row
+
+
 _CODES = {torch.float32: 0, torch.bfloat16: 1}
 
 
@@ -320,6 +404,59 @@ def embed(token_ids, table, scale=1.0):
     return stream
 
 
+def embed_pairs(token_ids, previous, table, pairs, *, scale, buckets, mul_prev, mul_cur, keep=False):
+    """int32 [N] tokens and the tokens before them (negative: a sequence's first) -> float32 stream [N, H] =
+    table[token] * scale + pairs[(previous * mul_prev + token * mul_cur) mod buckets] (``pairs`` [buckets + 1, H]; its last
+    row for a first token).  ``keep``: (stream, a copy of it in memory of its own)."""
+    library.check_device()
+    n, width = token_ids.shape[0], table.shape[1]
+    _require(token_ids, 'token_ids', torch.int32)
+    _require(previous, 'previous', torch.int32, (n,))
+    _require(table, 'table')
+    _require(pairs, 'pairs', table.dtype, (buckets + 1, width))
+    stream = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    copy = torch.empty_like(stream) if keep else None
+    _check(library.load().qil_embed_pairs(_ptr(token_ids), _ptr(previous), _ptr(table), _ptr(pairs), _ptr(stream), _ptr(copy),
+                                          n, width, float(scale), int(buckets), int(mul_prev), int(mul_cur),
+                                          _code(table.dtype), _stream()), 'embed_pairs')
+    return (stream, copy) if keep else stream
+
+
+def residual_join(stream, pending, weight, eps, out_dtype, rows=None):
+    """The sum of a ``Joined`` into the float32 stream [N, H] and the RMS norm of the result, x / sqrt(mean(x^2) + eps) *
+    weight, as ``out_dtype``: for all rows (the stream is updated in place), or for the selected ``rows`` (the stream is
+    left as it is).  float32 until the one rounding of the result."""
+    n, width = stream.shape
+    _require(stream, 'stream', torch.float32)
+    _require(weight, 'weight', torch.float32, (width,))
+    mixed = pending.mixed
+    left, right, left_scale, right_scale = mixed, None, 1.0, 1.0
+    if isinstance(mixed, Weighted):
+        left, right, left_scale, right_scale = mixed.left, mixed.right, mixed.left_scale, mixed.right_scale
+    none = (None, 0, 1, width)
+    a = _row_operand(left, 'mixed', n, width) if left is not None else none
+    b = _row_operand(right, 'mixed', n, width) if right is not None else none
+    f = _row_operand(pending.ffn, 'ffn', n, width) if pending.ffn is not None else none
+    g = none
+    if pending.gates is not None:
+        both = (2 if pending.ffn is not None else 1) * width
+        g = _row_operand(pending.gates, 'gates', n, both)
+        _require(pending.bias, 'bias', torch.float32, (both,))
+    if pending.plus is not None:
+        _require(pending.plus, 'plus', torch.float32, (n, width))
+    if pending.step is not None:
+        _require(pending.step, 'step', torch.float32, (width,))
+    if rows is not None:
+        _require(rows, 'rows', torch.int32)
+    count = n if rows is None else rows.shape[0]
+    out = torch.empty((count, width), dtype=out_dtype, device=stream.device)
+    _check(library.load().qil_residual_join(
+        _ptr(stream), *a, left_scale, *b, right_scale, *f, *g, _ptr(pending.bias) if pending.gates is not None else None,
+        _ptr(pending.plus), _ptr(pending.step), _ptr(rows), _ptr(weight), _ptr(out), count, n, width, float(eps),
+        int(rows is None), _code(out_dtype), _stream()), 'residual_join')
+    return out
+
+
 def add_rmsnorm(stream, delta, weight, eps, out_dtype):
     """stream += delta (in place, float32 sum; skipped if delta is None); returns norm(stream) as out_dtype.
 
@@ -362,6 +499,11 @@ def linear(x, weight, bias=None, out_dtype=None, partials=False, add_to=None):
     ``x`` may be ``Unmerged`` attention results, or a ``Normed`` residual stream.
     ``add_to``: the float32 residual stream [N, O]; if the kernel for these sizes can add its result into it
     (every element complete before it is added), it does and an ``Added`` is returned instead of the result."""
+    if isinstance(x, SharedInput):
+        at = x.places.get(id(weight))
+        if at is not None and bias is None and add_to is None and out_dtype in (None, x.dtype):
+            return Columns(x.product(), at, weight.shape[0])
+        x = x.x
     if isinstance(x, Gated):
         lib = library.load()
         n, k = x.shape
@@ -506,6 +648,11 @@ def gated_linear(x, weight, out_dtype=None, interleaved=False, lazy=False, activ
     ``lazy``: a few float32 rows may come back as ``Gated`` (the product's partial sums) for ``linear`` to finish."""
     if isinstance(x, Normed):
         x = x.materialize()
+    if isinstance(x, SharedInput):
+        if id(weight) in x.places:                  # the stack's product, then the activation kernel
+            return gated_act(linear(x, weight, None, partials=True), out_dtype or x.dtype, activation=activation, limit=limit,
+                             alpha=alpha, interleaved=interleaved)
+        x = x.x
     _require(x, 'x')
     _require(weight, 'weight', x.dtype)
     n, k = x.shape
@@ -581,7 +728,7 @@ def _rotation_arguments(rotation, head_dim):
 
 def qk_norm_rope_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps, rotation, positions, slots,
                        k_cache, v_cache, page_size, dtype, norm_dim=None, rotate_first=False, extra_columns=0,
-                       q_temperature=None, bias=None):
+                       q_temperature=None, bias=None, values_are_keys=False):
     """Per-head RMSNorm of q and k (if weights are given), rotation by position (if given).  ``norm_dim``: the
     number of elements the norm's mean runs over when the heads are padded with zeros (default: head_dim).
     ``rotate_first``: the rotation comes before the norm.  A rotation that carries ``frequencies`` is applied from
@@ -591,15 +738,18 @@ def qk_norm_rope_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, ep
     product); they are skipped.  ``kv_heads`` 0: the rows hold queries only.  ``q_temperature`` (coef, every): the
     query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) last, in float32.  ``bias``
     float32 [(heads + 2 kv_heads) d]: the projection's bias, added here (the product before then has none and may
-    stay partial sums).
+    stay partial sums).  ``values_are_keys``: the rows hold no values; a value is its key as projected, before norm and
+    rotation (the row is then (heads + kv_heads) d + extra_columns long).
 
-    ``qkv`` [N, (heads + 2 kv_heads) d + extra_columns]: tensor of type ``dtype`` or Partials.  Returns q as ``dtype``
+    ``qkv`` [N, (heads + 2 kv_heads) d + extra_columns]: tensor of type ``dtype``, Partials or Columns.  Returns q as ``dtype``
     [N, heads * d]; k and v go into the caches at ``slots`` (None: not stored)."""
     n = qkv.shape[0]
-    pointer, code, splits = _operand(qkv, 'qkv', dtype, (n, (heads + 2 * kv_heads) * head_dim + extra_columns))
+    own = (heads + (1 if values_are_keys else 2) * kv_heads) * head_dim
+    pointer, code, splits, row = _row_operand(qkv, 'qkv', n, own + extra_columns, (dtype,))
+    extra_columns = row - own
     coef, every = q_temperature if q_temperature is not None else (0.0, 0)
     if bias is not None:
-        _require(bias, 'bias', torch.float32, ((heads + 2 * kv_heads) * head_dim,))
+        _require(bias, 'bias', torch.float32, (own,))
     _require(positions, 'positions', torch.int32, (n,))
     for w, name in ((q_weight, 'q_weight'), (k_weight, 'k_weight')):
         if w is not None:
@@ -614,10 +764,42 @@ def qk_norm_rope_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, ep
     _check(library.load().qil_qk_norm_rope_store(
         pointer, code, splits, _ptr(q), _ptr(q_weight), _ptr(k_weight), _ptr(cos), _ptr(sin), _ptr(positions),
         _ptr(slots), _ptr(k_cache), _ptr(v_cache), n, heads, kv_heads, head_dim, rot, page_size, float(eps),
-        int(norm_dim or 0), int(bool(rotate_first)), int(extra_columns), float(coef), int(every), _ptr(bias), _code(dtype),
-        _stream()),
+        int(norm_dim or 0), int(bool(rotate_first)), int(extra_columns), float(coef), int(every), _ptr(bias),
+        int(bool(values_are_keys)), _code(dtype), _stream()),
         'qk_norm_rope_store')
     return q
+
+
+def qk_row_norm_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps, rotation, positions, slots, k_cache,
+                      v_cache, page_size, dtype, q_elems, k_elems, extra_columns=0, values_are_keys=False):
+    """``qk_norm_rope_store`` with one RMS norm over all query heads of a row and one over all its key heads, before
+    they are split into heads (``q_weight`` float32 [heads * d], ``k_weight`` [kv_heads * d]; ``q_elems`` / ``k_elems``:
+    how many elements the means run over, fewer than that when the heads are padded with zeros), then the rotation;
+    float32 and one rounding."""
+    n = qkv.shape[0]
+    own = (heads + (1 if values_are_keys else 2) * kv_heads) * head_dim
+    pointer, code, splits, row = _row_operand(qkv, 'qkv', n, own + extra_columns, (dtype,))
+    _require(positions, 'positions', torch.int32, (n,))
+    _require(q_weight, 'q_weight', torch.float32, (heads * head_dim,))
+    _require(k_weight, 'k_weight', torch.float32, (kv_heads * head_dim,))
+    cos, sin, rot = _rotation_arguments(rotation, head_dim)
+    if slots is not None:
+        _require(slots, 'slots', torch.int32, (n,))
+        _check_caches(k_cache, v_cache, dtype, kv_heads, page_size, head_dim)
+    q = torch.empty((n, heads * head_dim), dtype=dtype, device=qkv.device)
+    _check(library.load().qil_qk_row_norm_store(
+        pointer, code, splits, _ptr(q), _ptr(q_weight), _ptr(k_weight), _ptr(cos), _ptr(sin), _ptr(positions), _ptr(slots),
+        _ptr(k_cache), _ptr(v_cache), n, heads, kv_heads, head_dim, rot, page_size, float(eps), int(q_elems), int(k_elems),
+        row - own, int(bool(values_are_keys)), _code(dtype), _stream()), 'qk_row_norm_store')
+    return q
+
+
+def _places(max_context, window, keep_first):
+    """Most places (``csrc/key_span.h``) a row's visible keys take: all keys of the context, or, with kept first keys in
+    front of a window, the two ranges in whole steps of 32."""
+    if not keep_first or not window:
+        return max_context
+    return min(max_context, -(-keep_first // 32) * 32 + window + 31)
 
 
 def _rows_part(rows, kv_heads, max_context):
@@ -664,28 +846,37 @@ def decode_attention_takes(qkv, *, heads, kv_heads, head_dim, page_size, rotatio
     """Whether ``decode_attention`` takes the step: a float32 ``Partials`` q/k/v product, bfloat16 caches, sizes of
     the fused kernel."""
     rot = rotation.rot_dim if rotation is not None else 0
-    return isinstance(qkv, Partials) and qkv.shape[0] <= FUSED_DECODE_MOST_ROWS and dtype == torch.bfloat16 and \
+    source = qkv.source if isinstance(qkv, Columns) else qkv
+    if isinstance(qkv, Columns) and (qkv.offset % 8 or qkv.row % 8):
+        return False
+    return isinstance(source, Partials) and qkv.shape[0] <= FUSED_DECODE_MOST_ROWS and dtype == torch.bfloat16 and \
         bool(library.load().qil_attn_decode_fused_takes(heads, kv_heads, head_dim, page_size, rot))
 
 
 def decode_attention(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps, rotation, positions, writes, k_cache,
                      v_cache, page_size, block_tables, row_seq, max_context, scale, window, unmerged=False,
-                     rotate_first=False, softcap=None, has_kv=True, extra_columns=0, bias=None, q_temperature=None, sinks=None):
+                     rotate_first=False, softcap=None, has_kv=True, extra_columns=0, bias=None, q_temperature=None, sinks=None,
+                     values_are_keys=False, slopes=None, keep_first=0):
     """``qk_norm_rope_store`` and ``paged_attention`` in one kernel for a step whose rows are all alone in their
     sequences: queries, the new key and the new value are made from the partial sums ``qkv`` inside the
     attention kernel (bit for bit what the two kernels make), the new key and value are written into the
     pages (``writes``) and used from registers.  ``rotate_first`` and ``softcap`` as in ``qk_norm_rope_store`` and
     ``paged_attention``.  ``has_kv=False`` (with ``writes`` False): the rows of ``qkv`` hold queries only;
     ``extra_columns``, ``bias``, ``q_temperature`` as in ``qk_norm_rope_store``, ``sinks`` as in ``paged_attention``
-    (a step with sinks comes back merged).  Returns what ``paged_attention`` returns."""
+    (a step with sinks comes back merged); ``values_are_keys`` as in ``qk_norm_rope_store``, ``slopes`` and
+    ``keep_first`` as in ``paged_attention``.  Returns what ``paged_attention`` returns."""
     n = qkv.shape[0]
     dtype = torch.bfloat16
     stored = kv_heads if has_kv else 0
+    own = (heads + (1 if values_are_keys else 2) * stored) * head_dim
     if writes and not has_kv:
         raise ValueError('decode_attention: a step that writes keys and values needs them in qkv')
-    _require(qkv.tensor, 'qkv', torch.float32, (qkv.splits, n, (heads + 2 * stored) * head_dim + extra_columns))
+    pointer, _, splits, row = _row_operand(qkv, 'qkv', n, own + extra_columns, ())
+    if slopes is not None:
+        _require(slopes, 'slopes', torch.float32, (heads,))
+    keep = int(keep_first) if window else 0
     if bias is not None:
-        _require(bias, 'bias', torch.float32, ((heads + 2 * stored) * head_dim,))
+        _require(bias, 'bias', torch.float32, (own,))
     if sinks is not None:
         _require(sinks, 'sinks', torch.float32, (heads,))
         unmerged = False
@@ -703,20 +894,21 @@ def decode_attention(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps,
     lib = library.load()
     out = torch.empty((n, heads * head_dim), dtype=dtype, device=k_cache.device)
     window_arg = int(window or 0)
-    part, parts = _decode_parts(n, kv_heads, max_context)
+    part, parts = _decode_parts(n, kv_heads, _places(max_context, window, keep))
     nbytes = lib.qil_attn_rows_workspace(n, heads, head_dim, parts)
     workspace = torch.empty(nbytes // 4, dtype=torch.float32, device=out.device) if nbytes else None
-    _check(lib.qil_attn_decode_fused(_ptr(qkv.tensor), qkv.splits, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos),
+    _check(lib.qil_attn_decode_fused(pointer, splits, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos),
                                      _ptr(sin), rot, int(bool(writes)), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                      block_tables.shape[1], _ptr(row_seq), _ptr(positions), _ptr(workspace), _ptr(out),
                                      n, heads, kv_heads, head_dim, page_size, window_arg, float(scale), part, parts,
                                      DECODE_WAVES, int(n * kv_heads * parts <= DECODE_PAIRS_BLOCKS and head_dim <= FUSED_PAIRS_MOST_DIM),
-                                     int(bool(rotate_first)), float(softcap or 0.0), int(bool(has_kv)), int(extra_columns),
-                                     _ptr(bias), float(coef), int(every), _ptr(sinks), _stream()), 'attn_decode_fused')
+                                     int(bool(rotate_first)), float(softcap or 0.0), int(bool(has_kv)), row - own,
+                                     _ptr(bias), float(coef), int(every), _ptr(sinks), int(bool(values_are_keys)),
+                                     _ptr(slopes), keep, _stream()), 'attn_decode_fused')
     if parts > 1:
-        if sinks is not None:                           # the merge adds the sinks' term
+        if sinks is not None or keep:                   # the merge adds the sinks' term; its parts count places
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), None, _ptr(out), n, heads, head_dim, window_arg,
-                                      part, parts, _code(dtype), _ptr(sinks), _stream()), 'attn_merge')
+                                      part, parts, _code(dtype), _ptr(sinks), keep, _stream()), 'attn_merge')
             return out
         result = Unmerged(workspace, positions, out, heads=heads, head_dim=head_dim, window=window_arg, part=part,
                           parts=parts)
@@ -751,7 +943,7 @@ def tile_key_parts(lib, dtype, n_seqs, max_query, heads, kv_heads, head_dim, pag
 
 def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size, block_tables, row_seq, positions,
                     cu_seqlens, seq_starts, single_rows, n_seqs, max_query, max_context, scale, window,
-                    unmerged=False, tile_seqs=None, softcap=None, sinks=None):
+                    unmerged=False, tile_seqs=None, softcap=None, sinks=None, slopes=None, keep_first=0):
     """Attention of every row of the step over its request's cached keys.
 
     ``q`` [N, heads * head_dim] (head h at columns [h d, (h + 1) d)).  Row n belongs to sequence ``row_seq[n]`` (a row of ``block_tables``) and sees keys j with
@@ -769,11 +961,22 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
     scaled).  It enters where a row's result is normalised: in the kernel when the keys are in one piece, in the merge
     of the parts otherwise.  The general tile kernel, the bfloat16 prompt kernel for heads of 128, the matrix-core
     decode kernel and the row kernel take it; steps with sinks run on those and come back merged.
+    ``slopes`` float32 [heads]: slopes[h] * (position - key) is taken off head h's score after the scale (and the cap).
+    ``keep_first``: with a window, the first so many keys stay visible: row n sees j <= positions[n] with
+    j > positions[n] - window or j < keep_first.  Both run on the kernels that take sinks; with kept keys the parts of a
+    row's keys leave out the whole steps between the two ranges, and a portion's keys stay in one part.
     """
     cap = float(softcap or 0.0)
     if sinks is not None:
         _require(sinks, 'sinks', torch.float32, (heads,))
         unmerged = False
+    keep = int(keep_first) if window else 0
+    if keep < 0:
+        raise ValueError('keep_first must not be negative')
+    if keep:
+        unmerged = False
+    if slopes is not None:
+        _require(slopes, 'slopes', torch.float32, (heads,))
     if cap < 0:
         raise ValueError('softcap must be positive')
     n = q.shape[0]
@@ -803,7 +1006,9 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
                 raise ValueError('tile_seqs must count the sequences of two or more rows')
             n_seqs = tile_seqs
         part, parts = tile_key_parts(lib, qkv.dtype, several, max_query, heads, kv_heads,
-                                     head_dim, page_size, block_tables.shape[1], max_context, general=cap > 0)
+                                     head_dim, page_size, block_tables.shape[1], max_context, general=cap > 0 or slopes is not None)
+        if keep:
+            part, parts = 0, 1
         if parts > 1:
             # few row tiles deep in a long context: the keys in parts, one block each, merged afterwards (over all
             # rows of the step: what the merge leaves in rows that are alone is overwritten below)
@@ -811,7 +1016,7 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
             merged = n if tile_seqs is None else n - single_rows.shape[0]
             workspace = torch.empty(lib.qil_attn_rows_workspace(merged, heads, head_dim, parts) // 4, dtype=torch.float32,
                                     device=qkv.device)
-            if cap == 0 and qkv.dtype == torch.bfloat16 and head_dim in (64, 128) and \
+            if cap == 0 and slopes is None and qkv.dtype == torch.bfloat16 and head_dim in (64, 128) and \
                     lib.qil_attn_tile_bf16_takes(head_dim, page_size, block_tables.shape[1]):
                 _check(lib.qil_attn_tile_bf16_parts(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache),
                                                     _ptr(block_tables), block_tables.shape[1], _ptr(cu_seqlens),
@@ -823,22 +1028,25 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
                                                   _ptr(block_tables), block_tables.shape[1], _ptr(cu_seqlens),
                                                   _ptr(seq_starts), _ptr(workspace), merged, n_seqs, max_query, heads,
                                                   kv_heads, head_dim, page_size, int(window or 0), float(scale), cap,
-                                                  part, parts, _code(qkv.dtype), _stream()), 'attn_tile_in_parts')
+                                                  part, parts, _code(qkv.dtype), _ptr(slopes), _stream()),
+                       'attn_tile_in_parts')
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), None, _ptr(out), merged, heads, head_dim,
-                                      int(window or 0), part, parts, _code(qkv.dtype), _ptr(sinks), _stream()), 'attn_merge')
+                                      int(window or 0), part, parts, _code(qkv.dtype), _ptr(sinks), 0, _stream()),
+                   'attn_merge')
         else:
             _check(lib.qil_attn_tile(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                      block_tables.shape[1], _ptr(cu_seqlens), _ptr(seq_starts), _ptr(out), n_seqs,
                                      max_query, heads, kv_heads, head_dim, page_size, int(window or 0), float(scale),
-                                     cap, _code(qkv.dtype), _ptr(sinks), _stream()), 'attn_tile')
+                                     cap, _code(qkv.dtype), _ptr(sinks), _ptr(slopes), keep, _stream()), 'attn_tile')
         rows = single_rows.shape[0]
     else:
         single_rows, rows = None, n
     if rows:
         window_arg = int(window or 0)
+        places = _places(max_context, window, keep)
         if qkv.dtype == torch.bfloat16 and lib.qil_attn_decode_takes(heads, kv_heads, head_dim, page_size):
             # matrix-core kernel; split the context until the chip has about four blocks per CU
-            part, parts = _decode_parts(rows, kv_heads, max_context)
+            part, parts = _decode_parts(rows, kv_heads, places)
             nbytes = lib.qil_attn_rows_workspace(rows, heads, head_dim, parts)
             workspace = torch.empty(nbytes // 4, dtype=torch.float32, device=qkv.device) if nbytes else None
             _check(lib.qil_attn_decode(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
@@ -846,18 +1054,19 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
                                        _ptr(workspace), _ptr(out), rows, heads, kv_heads, head_dim, page_size,
                                        window_arg, float(scale), part, parts, DECODE_WAVES,
                                        int(rows * kv_heads * parts <= DECODE_PAIRS_BLOCKS and head_dim <= 128), cap,
-                                       _ptr(sinks), _stream()), 'attn_decode')
+                                       _ptr(sinks), _ptr(slopes), keep, _stream()), 'attn_decode')
             if unmerged and parts > 1 and single_rows is None:
                 return Unmerged(workspace, positions, out, heads=heads, head_dim=head_dim, window=window_arg,
                                 part=part, parts=parts)
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), _ptr(single_rows), _ptr(out), rows, heads,
-                                      head_dim, window_arg, part, parts, _code(qkv.dtype), _ptr(sinks), _stream()), 'attn_merge')
+                                      head_dim, window_arg, part, parts, _code(qkv.dtype), _ptr(sinks), keep, _stream()),
+                   'attn_merge')
         else:
-            part = _rows_part(rows, kv_heads, max_context)
-            parts = max(1, -(-max_context // part))
+            part = _rows_part(rows, kv_heads, places)
+            parts = max(1, -(-places // part))
             nbytes = lib.qil_attn_rows_workspace(rows, heads, head_dim, parts)
             workspace = torch.empty(nbytes // 4, dtype=torch.float32, device=qkv.device) if nbytes else None
-            if unmerged and parts > 1 and single_rows is None and rows <= UNMERGED_ROWS_MOST:
+            if unmerged and slopes is None and parts > 1 and single_rows is None and rows <= UNMERGED_ROWS_MOST:
                 _check(lib.qil_attn_rows_unmerged(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache),
                                                   _ptr(block_tables), block_tables.shape[1], _ptr(row_seq),
                                                   _ptr(positions), _ptr(workspace), rows, heads, kv_heads, head_dim,
@@ -868,8 +1077,8 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
             _check(lib.qil_attn_rows(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                      block_tables.shape[1], _ptr(row_seq), _ptr(positions), _ptr(single_rows),
                                      _ptr(workspace), _ptr(out), rows, heads, kv_heads, head_dim, page_size,
-                                     window_arg, float(scale), cap, part, parts, _code(qkv.dtype), _ptr(sinks), _stream()),
-                   'attn_rows')
+                                     window_arg, float(scale), cap, part, parts, _code(qkv.dtype), _ptr(sinks), _ptr(slopes), keep,
+                                     _stream()), 'attn_rows')
     return out
 
 
@@ -934,18 +1143,19 @@ def rows_norm(stream, delta, rows, weight, eps, out_dtype, *, centre, delta_scal
 
 # Gate functions of gated feed-forwards: name -> code of the kernels.  'silu': silu(g) * u.  'clamped_swish' (with a
 # limit L and a slope a): g' = min(g, L), u' = clamp(u, -L, L), g' * sigmoid(a g') * (u' + 1).
-GATE_FUNCTIONS = {'silu': 0, 'clamped_swish': 1}
+# 'relu': max(g, 0) * u.
+GATE_FUNCTIONS = {'silu': 0, 'clamped_swish': 1, 'relu': 2}
 
 
 def gated_act(gate_up, out_dtype, *, activation, limit=0.0, alpha=1.0, interleaved=False):
-    """[N, 2 I] (tensor of the model's type or Partials) -> act(gate, up), [N, I], for any gate function of
+    """[N, 2 I] (tensor of the model's type, Partials or Columns) -> act(gate, up), [N, I], for any gate function of
     ``GATE_FUNCTIONS``.  The gate columns come first, or (``interleaved``) gate and up columns come in turns of 16."""
     n, both = gate_up.shape
     if both % 2 or (interleaved and both % 32):
         raise ValueError('gated_act: needs an even number of columns (a multiple of 32 when they are interleaved)')
-    pointer, code, splits = _operand(gate_up, 'gate_up', out_dtype, (n, both))
+    pointer, code, splits, row = _row_operand(gate_up, 'gate_up', n, both, (out_dtype,))
     out = torch.empty((n, both // 2), dtype=out_dtype, device=gate_up.device)
-    _check(library.load().qil_gated_act(pointer, code, splits, _ptr(out), n, both // 2, _code(out_dtype), int(interleaved),
+    _check(library.load().qil_gated_act(pointer, code, splits, row, _ptr(out), n, both // 2, _code(out_dtype), int(interleaved),
                                         GATE_FUNCTIONS[activation], float(limit), float(alpha), _stream()), 'gated_act')
     return out
 
@@ -1182,7 +1392,7 @@ def latent_attention(q, *, latent, rope, page_size, block_tables, row_seq, posit
 
 # ---------------------------------------------------------------------------------------------------------------
 # Recurrences with a matrix state
-SCAN_MODES = {'decay': 0, 'mlstm': 1, 'channel': 2}
+SCAN_MODES = {'decay': 0, 'mlstm': 1, 'channel': 2, 'step': 3}
 SCAN_BLOCKS_FROM = 32           # rows of one sequence from which a step's recurrence runs in blocks side by side
 
 
@@ -1196,7 +1406,7 @@ def state_scan_slot(*, heads, dim, vdim, mode):
 
 def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, state, cu_seqlens, seq_starts, seq_slots,
                n_seqs, gates=None, gate_bias=None, cap=0.0, decay=None, frequencies=None, rot=0, q_scale=1.0, k_scale=1.0,
-               max_query=None):
+               max_query=None, groups=None):
     """S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t per head over every sequence's rows of the step, from the
     sequence's state slot (empty where the sequence starts at position 0) and back into it.
 
@@ -1205,6 +1415,9 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
     gates from ``gates`` float32 [N, 2 heads] (+ ``gate_bias`` [2 heads]; input gates first) soft-capped at ``cap``,
     with a running maximum and a normaliser.  Mode 'channel': every row i of a head's S keeps a_t[i] =
     sigmoid(z)^(1 / tau) of itself, with z = ``gates`` float32 [N, heads * dim] and tau = ``cap``; b_t = 1.
+    Mode 'step': a step size per head and token, d_t = softplus(gates[t, h] + gate_bias[h]) (``gates`` [N, heads]: a
+    tensor, Partials or Columns; ``gate_bias`` [heads]), a_t = exp(decay[h] * d_t), b_t = d_t; queries and keys are those of
+    ``groups`` groups (groups * dim columns each), head h reads group h // (heads / groups)'s; nothing is rotated.
     Queries and keys are rotated by position on their leading ``rot``
     elements (``frequencies`` [rot / 2]) and then scaled.  ``max_query``: the most rows of one sequence, if the caller
     knows it; from ``SCAN_BLOCKS_FROM`` rows on the step is worked in blocks of 64 tokens side by side (the sums of the
@@ -1218,7 +1431,10 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
     if not lib.qil_state_scan_takes(dim, vdim, rot):
         raise UnsupportedShape(f'state_scan: dim {dim} (up to 256), vdim {vdim}, {rot} rotated elements')
     width = proj.shape[1]
-    if min(q_offset, k_offset, v_offset) < 0 or max(q_offset, k_offset) + heads * dim > width or v_offset + heads * vdim > width:
+    if mode == 'step' and (groups is None or groups < 1 or heads % groups or rot):
+        raise ValueError("state_scan: mode 'step' takes groups that divide the heads and no rotation")
+    shared = groups if mode == 'step' else heads
+    if min(q_offset, k_offset, v_offset) < 0 or max(q_offset, k_offset) + shared * dim > width or v_offset + heads * vdim > width:
         raise ValueError('state_scan: offsets do not fit the rows')
     slot = state_scan_slot(heads=heads, dim=dim, vdim=vdim, mode=mode)
     if slot != lib.qil_state_scan_slot(heads, dim, vdim, SCAN_MODES[mode]):
@@ -1229,7 +1445,13 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
     _require(cu_seqlens, 'cu_seqlens', torch.int32, (n_seqs + 1,))
     _require(seq_starts, 'seq_starts', torch.int32, (n_seqs,))
     _require(seq_slots, 'seq_slots', torch.int32, (n_seqs,))
-    if mode == 'mlstm':
+    raw = (None, 0, 1, 0)
+    if mode == 'step':
+        raw = _row_operand(gates, 'gates', n, heads)
+        gates = None
+        _require(gate_bias, 'gate_bias', torch.float32, (heads,))
+        _require(decay, 'decay', torch.float32, (heads,))
+    elif mode == 'mlstm':
         _require(gates, 'gates', torch.float32, (n, 2 * heads))
         _require(gate_bias, 'gate_bias', torch.float32, (2 * heads,))
     elif mode == 'channel':
@@ -1249,14 +1471,34 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
                                           _ptr(gate_bias), float(cap), _ptr(decay), _ptr(frequencies) if rot else None,
                                           rot, float(q_scale), float(k_scale), _ptr(state), slot, _ptr(cu_seqlens),
                                           _ptr(seq_starts), _ptr(seq_slots), _ptr(out), _ptr(below), _ptr(workspace), n,
-                                          n_seqs, int(max_query), heads, dim, vdim, SCAN_MODES[mode], _stream()),
-               'state_scan_chunked')
+                                          n_seqs, int(max_query), heads, dim, vdim, SCAN_MODES[mode], *raw, int(shared),
+                                          _stream()), 'state_scan_chunked')
         return out, below
     _check(lib.qil_state_scan(_ptr(proj), code, width, q_offset, k_offset, v_offset, _ptr(gates), _ptr(gate_bias),
                               float(cap), _ptr(decay), _ptr(frequencies) if rot else None, rot, float(q_scale),
                               float(k_scale), _ptr(state), _ptr(cu_seqlens), _ptr(seq_starts), _ptr(seq_slots), _ptr(out),
-                              _ptr(below), n_seqs, heads, dim, vdim, SCAN_MODES[mode], _stream()), 'state_scan')
+                              _ptr(below), n_seqs, heads, dim, vdim, SCAN_MODES[mode], *raw, n, int(shared), _stream()), 'state_scan')
     return out, below
+
+
+def gated_group_norm(o, u, *, skip, z, weight, vdim, groups, eps, out_dtype):
+    """y = o + skip[head] * u (heads of ``vdim`` columns), times silu(z); then each of the row's ``groups`` equal parts over
+    its root mean square (eps inside the root), times ``weight``.  ``o`` float32 [N, inner]; ``u`` [N, >= inner] of
+    ``out_dtype`` (its first inner columns); ``z`` [N, inner]: tensor, Partials or Columns; ``skip`` float32
+    [inner / vdim]; ``weight`` float32 [inner].  float32 and one rounding.  -> [N, inner] of ``out_dtype``."""
+    n, inner = o.shape
+    _require(o, 'o', torch.float32)
+    _require(u, 'u', out_dtype)
+    if u.shape[0] != n or u.shape[1] < inner or inner % groups or inner % vdim:
+        raise ValueError('gated_group_norm: sizes do not fit')
+    _require(skip, 'skip', torch.float32, (inner // vdim,))
+    _require(weight, 'weight', torch.float32, (inner,))
+    z_pointer, z_code, z_splits, z_row = _row_operand(z, 'z', n, inner)
+    y = torch.empty((n, inner), dtype=out_dtype, device=o.device)
+    _check(library.load().qil_gated_group_norm(_ptr(o), _ptr(u), u.shape[1], _ptr(skip), z_pointer, z_code, z_splits, z_row,
+                                               _ptr(weight), _ptr(y), inner, n, inner, int(vdim), int(groups), float(eps),
+                                               1.0, _code(out_dtype), _stream()), 'gated_group_norm')
+    return y
 
 
 def head_norm_gate(o, gate_source, *, gate_offset, heads, vdim, weight, eps, gate, out_dtype, denominators=None):
@@ -1380,7 +1622,9 @@ def sigmoid_gate(x, source, *, offset):
     width = source.shape[1]
     if source.shape[0] != n or offset < 0 or offset + columns > width:
         raise ValueError('sigmoid_gate: the gate columns do not lie inside the source')
-    pointer, code, splits = _any_operand(source, 'source', (n, width))
+    pointer, code, splits, row = _row_operand(source, 'source', n, width)
+    if isinstance(source, Columns):                     # (the kernel checks the columns against the whole row)
+        pointer, offset, width = pointer - source.offset * (4 if code == 0 else 2), offset + source.offset, row
     out = torch.empty_like(x)
     _check(library.load().qil_sigmoid_gate(_ptr(x), pointer, code, splits, width, int(offset), _ptr(out), n, columns,
                                            _code(x.dtype), _stream()), 'sigmoid_gate')
@@ -1406,7 +1650,7 @@ CONV_ACTIVATIONS = {None: 0, 'silu': 1}
 def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq_slots, row_seq, n_seqs, activation,
                  out_dtype):
     """act(bias + causal convolution over time) on the first ``columns`` columns of ``x`` [N, W] (tensor of the
-    model's type or Partials): out[t, c] = act(bias[c] + sum_j weight[j, c] * x[t - taps + 1 + j, c]) over the rows of
+    model's type, Partials or Columns): out[t, c] = act(bias[c] + sum_j weight[j, c] * x[t - taps + 1 + j, c]) over the rows of
     every sequence of the step and the taps - 1 inputs before them, which are the sequence's state (``state`` float32
     [slots, taps - 1, columns]: read unless the sequence starts at position 0, and left holding the sequence's last
     taps - 1 inputs).  ``weight`` float32 [taps, columns], ``bias`` float32 [columns] or None.  -> [N, columns] of
@@ -1424,7 +1668,7 @@ def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq
     _require(seq_starts, 'seq_starts', torch.int32, (n_seqs,))
     _require(seq_slots, 'seq_slots', torch.int32, (n_seqs,))
     _require(row_seq, 'row_seq', torch.int32, (n,))
-    pointer, code, splits = _any_operand(x, 'x', (n, width))
+    pointer, code, splits, width = _row_operand(x, 'x', n, width)
     out = torch.empty((n, columns), dtype=out_dtype, device=weight.device)
     _check(library.load().qil_channel_conv(pointer, code, splits, width, _ptr(weight), _ptr(bias),
                                            _ptr(state) if taps > 1 else None, _ptr(cu_seqlens), _ptr(seq_starts),

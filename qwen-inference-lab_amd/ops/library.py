@@ -212,18 +212,19 @@ def _declare(lib):
     lib.qil_add_rmsnorm.argtypes = [p, p, i, i, i, p, p, p, i, i, f, i, i, p]
     lib.qil_silu_mul.argtypes = [p, i, i, p, i, i, i, i, p]
     lib.qil_add_bias.argtypes = [p, p, i, i, i, p]
-    lib.qil_qk_norm_rope_store.argtypes = [p, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i, f, i, p, i, p]
+    lib.qil_qk_norm_rope_store.argtypes = [p, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i, f, i, p, i, i, p]
+    lib.qil_qk_row_norm_store.argtypes = [p, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, i, p]
     lib.qil_attn_rows_workspace.argtypes = [i, i, i, i]
     lib.qil_attn_rows_workspace.restype = z
-    lib.qil_attn_rows.argtypes = [p, i, p, p, p, i, p, p, p, p, p, i, i, i, i, i, i, f, f, i, i, i, p, p]
-    lib.qil_attn_merge.argtypes = [p, p, p, p, i, i, i, i, i, i, i, p, p]
+    lib.qil_attn_rows.argtypes = [p, i, p, p, p, i, p, p, p, p, p, i, i, i, i, i, i, f, f, i, i, i, p, p, i, p]
+    lib.qil_attn_merge.argtypes = [p, p, p, p, i, i, i, i, i, i, i, p, i, p]
     lib.qil_attn_decode_fused_takes.argtypes = [i, i, i, i, i]
     lib.qil_attn_decode_fused_takes.restype = i
-    lib.qil_attn_decode_fused.argtypes = [p, i, p, p, f, p, p, i, i, p, p, p, i, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, i, f, i, i, p, f, i, p, p]
+    lib.qil_attn_decode_fused.argtypes = [p, i, p, p, f, p, p, i, i, p, p, p, i, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, i, f, i, i, p, f, i, p, i, p, i, p]
     lib.qil_attn_decode_takes.argtypes = [i, i, i, i]
     lib.qil_attn_decode_takes.restype = i
-    lib.qil_attn_decode.argtypes = [p, i, p, p, p, i, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, f, p, p]
-    lib.qil_attn_tile.argtypes = [p, i, p, p, p, i, p, p, p, i, i, i, i, i, i, i, f, f, i, p, p]
+    lib.qil_attn_decode.argtypes = [p, i, p, p, p, i, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, f, p, p, i, p]
+    lib.qil_attn_tile.argtypes = [p, i, p, p, p, i, p, p, p, i, i, i, i, i, i, i, f, f, i, p, p, i, p]
     lib.qil_gemm_f32.argtypes = [p, p, p, p, i, i, i, i, p]
     lib.qil_gemm_f32_splits.argtypes = [i, i, i]
     lib.qil_gemm_f32_waves.argtypes = [i, i, i, i]
@@ -255,7 +256,7 @@ def _declare(lib):
     lib.qil_attn_tile_bf16_parts.restype = i
     lib.qil_attn_tile_key_parts.argtypes = [i, i, i, i, i, i, i, ctypes.POINTER(ctypes.c_int)]
     lib.qil_attn_tile_key_parts.restype = i
-    lib.qil_attn_tile_in_parts.argtypes = [p, i, p, p, p, i, p, p, p, i, i, i, i, i, i, i, i, f, f, i, i, i, p]
+    lib.qil_attn_tile_in_parts.argtypes = [p, i, p, p, p, i, p, p, p, i, i, i, i, i, i, i, i, f, f, i, i, i, p, p]
     lib.qil_attn_tile_in_parts.restype = i
     lib.qil_attn_tile_waves.argtypes = [i]
     lib.qil_attn_tile_waves.restype = None
@@ -288,7 +289,7 @@ def _declare(lib):
     lib.qil_gemm_bf16_wide_gated_takes.restype = i
     lib.qil_gemm_bf16_wide_gated.argtypes = [p, p, p, i, i, i, i, p]
     lib.qil_add_norm.argtypes = [p, p, i, i, i, f, p, p, p, p, i, i, f, i, i, i, p]
-    lib.qil_gated_act.argtypes = [p, i, i, p, i, i, i, i, i, f, f, p]
+    lib.qil_gated_act.argtypes = [p, i, i, i, p, i, i, i, i, i, f, f, p]
     lib.qil_latent_prepare.argtypes = [p, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, f, i, p]
     lib.qil_head_product.argtypes = [p, i, i, i, p, i, p, i, i, i, i, i, i, i, p]
     lib.qil_rotate_tail.argtypes = [p, i, i, i, i, p, p, p, i, i, i, i, i, i, p]
@@ -308,11 +309,11 @@ def _declare(lib):
     lib.qil_state_scan_slot.restype = z
     lib.qil_state_scan_takes.argtypes = [i, i, i]
     lib.qil_state_scan_takes.restype = i
-    lib.qil_state_scan.argtypes = [p, i, i, i, i, i, p, p, f, p, p, i, f, f, p, p, p, p, p, p, i, i, i, i, i, p]
+    lib.qil_state_scan.argtypes = [p, i, i, i, i, i, p, p, f, p, p, i, f, f, p, p, p, p, p, p, i, i, i, i, i, p, i, i, i, i, i, p]
     lib.qil_head_norm_gate.argtypes = [p, p, p, i, i, p, p, i, i, i, f, i, i, p]
     lib.qil_state_scan_chunked_workspace.argtypes = [i, i, i, i, i, i]
     lib.qil_state_scan_chunked_workspace.restype = z
-    lib.qil_state_scan_chunked.argtypes = [p, i, i, i, i, i, p, p, f, p, p, i, f, f, p, z, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
+    lib.qil_state_scan_chunked.argtypes = [p, i, i, i, i, i, p, p, f, p, p, i, f, f, p, z, p, p, p, p, p, p, i, i, i, i, i, i, i, p, i, i, i, i, p]
     lib.qil_state_scan_chunked.restype = i
     for name in ('qil_add_norm', 'qil_gated_act', 'qil_latent_prepare', 'qil_head_product', 'qil_rotate_tail',
                  'qil_latent_attention', 'qil_state_scan', 'qil_head_norm_gate'):
@@ -352,6 +353,12 @@ def _declare(lib):
     lib.qil_short_conv.restype = i
     lib.qil_plain_act.argtypes = [p, i, i, p, i, i, i, i, p, p]
     lib.qil_plain_act.restype = i
+    ll = ctypes.c_longlong
+    lib.qil_embed_pairs.argtypes = [p, p, p, p, p, p, i, i, f, i, ll, ll, i, p]
+    lib.qil_gated_group_norm.argtypes = [p, p, i, p, p, i, i, i, p, p, i, i, i, i, i, f, f, i, p]
+    lib.qil_residual_join.argtypes = [p, p, i, i, i, f, p, i, i, i, f, p, i, i, i, p, i, i, i, p, p, p, p, p, p, i, i, i, f, i, i, p]
+    for name in ('qil_embed_pairs', 'qil_gated_group_norm', 'qil_residual_join', 'qil_qk_row_norm_store'):
+        getattr(lib, name).restype = i
     lib.qil_sample.argtypes = [p, p, p, p, p, p, p, i, i, p]
     lib.qil_sample_workspace.argtypes = [i, i]
     lib.qil_sample_workspace.restype = z

@@ -37,6 +37,16 @@ class Attention(Mixer):
     once: it has no key and no value and is not scaled.
     ``gate``: the heads' results are multiplied element by element by sigmoid(W_g h) before the output projection
     (tensor ``g_proj.weight`` [heads * value_dim, width], stacked under q/k/v: one product makes all four).
+    ``values_are_keys``: there is no value projection; a value is its key as projected, before norm and rotation (values
+    and keys have one size then).
+    ``pairing='neighbours'``: the rotation turns elements 2 i and 2 i + 1 together (else i and i + rot / 2).  The rows of
+    the query and key matrices are reordered at ``finalize`` (even elements of the rotated part first, then odd ones), so
+    the kernels see halves; where values are keys the gate's rows and the output matrix's columns follow.
+    ``qk_norm='row'``: one norm over all query heads of a row and one over all key heads, before they are split into heads
+    (weights of the projections' sizes), instead of a norm per head.
+    ``sink_value``: a fixed sink, the same for every head (0: one is added to the softmax's denominator).
+    ``distance_slopes``: a number m_h per query head; m_h * (i - j) is taken off the scaled score of query i and key j.
+    ``keep_first``: behind a window, the first so many keys stay visible (at their true positions).
     ``own_kv=False``: the part has no key and value projections; its schedule entry reads another entry's cache
     (``ScheduleEntry.cache_of``), with its own queries, mask and everything else.
     """
@@ -45,8 +55,26 @@ class Attention(Mixer):
 
     def __init__(self, *, width, heads, kv_heads, head_dim, bias, qk_norm_eps, scale,
                  position=None, window=None, dtype=torch.bfloat16, value_dim=None, softcap=None, qk_norm_weights=True,
-                 norm_after_rotation=False, out_bias=None, q_temperature=None, sink=False, gate=False, own_kv=True):
+                 norm_after_rotation=False, out_bias=None, q_temperature=None, sink=False, gate=False, own_kv=True,
+                 values_are_keys=False, pairing='halves', qk_norm='head', sink_value=None, distance_slopes=None, keep_first=0):
         super().__init__()
+        if pairing not in ('halves', 'neighbours') or qk_norm not in ('head', 'row'):
+            raise ValueError(f'unknown pairing {pairing!r} or norm {qk_norm!r}')
+        if type(keep_first) is not int or keep_first < 0 or (keep_first and window is None):
+            raise ValueError('keep_first is a number of first keys kept behind a window')
+        if distance_slopes is not None and len(distance_slopes) != heads:
+            raise ValueError('one slope per query head')
+        if sink and sink_value is not None:
+            raise ValueError('sinks are stored or fixed, not both')
+        if values_are_keys and (bias or not own_kv or value_dim not in (None, head_dim)):
+            raise ValueError('values that are keys need keys of their own, of the same size, and no bias')
+        if qk_norm == 'row' and (qk_norm_eps is None or not qk_norm_weights or norm_after_rotation or bias or
+                                 q_temperature is not None or not own_kv):
+            raise ValueError('a norm over whole rows has an eps and weights, comes before the rotation, and there are no biases')
+        self.values_are_keys, self.pairing, self.qk_norm = bool(values_are_keys), pairing, qk_norm
+        self.sink_value = None if sink_value is None else float(sink_value)
+        self.distance_slopes = None if distance_slopes is None else [float(m) for m in distance_slopes]
+        self.keep_first = keep_first
         if heads % kv_heads:
             raise ValueError('heads must be a multiple of kv_heads')
         self.width, self.heads, self.kv_heads, self.head_dim = width, heads, kv_heads, head_dim
@@ -79,7 +107,9 @@ class Attention(Mixer):
         v, o = self.kv_heads * self.value_dim, self.heads * self.value_dim
         specs = {'q_proj.weight': ParamSpec((q, self.width)), 'o_proj.weight': ParamSpec((self.width, o))}
         if self.own_kv:
-            specs.update({'k_proj.weight': ParamSpec((kv, self.width)), 'v_proj.weight': ParamSpec((v, self.width))})
+            specs['k_proj.weight'] = ParamSpec((kv, self.width))
+            if not self.values_are_keys:
+                specs['v_proj.weight'] = ParamSpec((v, self.width))
         if self.bias:
             specs['q_proj.bias'] = ParamSpec((q,), 'vector')
             if self.own_kv:
@@ -87,9 +117,10 @@ class Attention(Mixer):
         if self.out_bias:   # o_proj gets a bias too (qil/model.py:35)
             specs['o_proj.bias'] = ParamSpec((self.width,), 'vector')
         if self.qk_norm_eps is not None and self.qk_norm_weights:
-            specs['q_norm.weight'] = ParamSpec((d,), 'vector', 'one_plus_normal')
+            row = self.qk_norm == 'row'
+            specs['q_norm.weight'] = ParamSpec((q if row else d,), 'vector', 'one_plus_normal')
             if self.own_kv:
-                specs['k_norm.weight'] = ParamSpec((d,), 'vector', 'one_plus_normal')
+                specs['k_norm.weight'] = ParamSpec((kv if row else d,), 'vector', 'one_plus_normal')
         if self.gate:
             specs['g_proj.weight'] = ParamSpec((o, self.width))
         if self.sink:
@@ -97,7 +128,7 @@ class Attention(Mixer):
         return specs
 
     def cache_need(self):
-        return KVNeed(self.kv_heads, self.padded_dim, self.window)
+        return KVNeed(self.kv_heads, self.padded_dim, self.window, self.keep_first)
 
     def _pad_heads(self, tensor, axis=0, d=None):
         """``tensor`` with every head's ``d`` (default ``head_dim``) entries along ``axis`` followed by zeros up to
@@ -115,11 +146,26 @@ class Attention(Mixer):
         shape[axis:axis + 2] = [count * dp]
         return out.reshape(shape)
 
+    def _halves(self, tensor, axis=0):
+        """``tensor`` with the rotated part of every head's entries along ``axis`` in the order even, then odd."""
+        rot, d = self.position.rot_dim, self.head_dim
+        order = list(range(0, rot, 2)) + list(range(1, rot, 2)) + list(range(rot, d))
+        index = torch.tensor([base + i for base in range(0, tensor.shape[axis], d) for i in order], device=tensor.device)
+        return tensor.index_select(axis, index).contiguous()
+
     def finalize(self):
         p = self.p
+        if self.pairing == 'neighbours' and self.position is not None:
+            turned = ['q_proj.weight', 'q_proj.bias', 'k_proj.weight', 'k_proj.bias', 'q_norm.weight', 'k_norm.weight']
+            if self.values_are_keys:
+                turned.append('g_proj.weight')
+                p['o_proj.weight'] = self._halves(p['o_proj.weight'], axis=1)
+            for name in turned:
+                if name in p:
+                    p[name] = self._halves(p[name])
         stacked = [('q_proj', self.head_dim)]
         if self.own_kv:
-            stacked += [('k_proj', self.head_dim), ('v_proj', self.value_dim)]
+            stacked += [('k_proj', self.head_dim)] + ([] if self.values_are_keys else [('v_proj', self.value_dim)])
         matrices = [self._pad_heads(p.pop(f'{name}.weight'), d=d) for name, d in stacked]
         biases = [self._pad_heads(p.pop(f'{name}.bias'), d=d) for name, d in stacked] if self.bias else None
         if self.gate:                                    # the gate's rows come last and have no bias
@@ -141,14 +187,31 @@ class Attention(Mixer):
                     p[name] = self._pad_heads(p[name]).contiguous()
         if self.qk_norm_eps is not None and not self.qk_norm_weights:       # a norm that multiplies by nothing
             self._ones = torch.ones(self.padded_dim, dtype=torch.float32, device=self.w_qkv.device)
+        device = self.w_qkv.device
+        if self.sink_value is not None:
+            p['sinks'] = torch.full((self.heads,), self.sink_value, dtype=torch.float32, device=device)
+        self.slopes = None
+        if self.distance_slopes is not None:
+            self.slopes = torch.tensor(self.distance_slopes, dtype=torch.float64).to(torch.float32).to(device)
         if self.position is not None:
             self.position.rotation()                     # device tensors are made here, not in a step that may be captured
+
+    def _is_extended(self):
+        return self.gate or self.sink or self.q_temperature is not None or not self.own_kv or self.values_are_keys or \
+            self.qk_norm == 'row' or self.sink_value is not None or self.distance_slopes is not None or self.keep_first > 0
+
+    def input_matrices(self):
+        return ('qkv_proj.weight',) if self._is_extended() or not self.bias else ()
+
+    def place_matrix(self, name, tensor):
+        super().place_matrix(name, tensor)
+        self.w_qkv = self.p['qkv_proj.weight']
 
     def forward(self, h, ctx, cache):
         p = self.p
         if cache.writes and not self.own_kv:
             raise ValueError('an attention part without keys and values of its own reads another entry\'s cache')
-        extended = self.gate or self.sink or self.q_temperature is not None or not self.own_kv
+        extended = self._is_extended()
         # (the extended step's q/k kernel adds the bias itself: its product may then stay partial sums)
         qkv = ops.linear(h, self.w_qkv, None if extended else self.b_qkv, partials=True)
         rotation = self.position.rotation() if self.position is not None else None
@@ -183,36 +246,41 @@ class Attention(Mixer):
         return ops.linear(attended, p['o_proj.weight'], p.get('o_proj.bias'), partials=True)
 
     def _forward_extended(self, qkv, rotation, norms, sizes, ctx, cache):
-        """The step of a part with a query temperature, sinks, an output gate or another entry's keys and values:
-        the q/k kernel skips the gate's columns of the stacked product (and finds no key and value columns when the
-        part has none), the attention kernels take the sinks, and the gate multiplies what they return."""
+        """The step of a part with a query temperature, sinks, an output gate, values that are keys, a norm over whole rows,
+        slopes, kept keys or another entry's keys and values: the q/k kernel skips the gate's columns of the stacked product
+        (and finds no key and value columns when the part has none), the attention kernels take sinks, slopes and kept
+        keys, and the gate multiplies what they return."""
         p = self.p
         gate_columns = self.heads * self.padded_dim if self.gate else 0
         stored = self.kv_heads if self.own_kv else 0
-        if ctx.max_query == 1 and self.padded_dim == self.head_dim and \
+        own = (self.heads + (1 if self.values_are_keys else 2) * stored) * self.padded_dim
+        masks = dict(scale=self.scale, window=self.window, softcap=self.softcap, sinks=p.get('sinks'), slopes=self.slopes,
+                     keep_first=self.keep_first)
+        rows = self.qk_norm == 'row'
+        if not rows and ctx.max_query == 1 and self.padded_dim == self.head_dim and \
                 ops.decode_attention_takes(qkv, page_size=cache.page_size, rotation=rotation, dtype=self.dtype, **sizes):
             # every row alone in its sequence: bias, norm, rotation, temperature and cache write inside the attention kernel
             attended = ops.decode_attention(
                 qkv, rotation=rotation, positions=ctx.positions, writes=cache.writes, k_cache=cache.k, v_cache=cache.v,
                 page_size=cache.page_size, block_tables=cache.block_tables, row_seq=ctx.row_seq,
-                max_context=ctx.max_context, scale=self.scale, window=self.window, unmerged=False,
-                rotate_first=self.norm_after_rotation, softcap=self.softcap, has_kv=self.own_kv,
-                extra_columns=gate_columns, bias=self.b_qkv_own, q_temperature=self.q_temperature, sinks=p.get('sinks'),
-                **sizes, **norms)
-            if self.gate:
-                attended = ops.sigmoid_gate(attended, qkv, offset=(self.heads + 2 * stored) * self.padded_dim)
-            return ops.linear(attended, p['o_proj.weight'], p.get('o_proj.bias'), partials=True)
-        q = ops.qk_norm_rope_store(
-            qkv, rotation=rotation, positions=ctx.positions, slots=cache.slots if cache.writes else None,
-            k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size, dtype=self.dtype, norm_dim=self.head_dim,
-            rotate_first=self.norm_after_rotation, heads=self.heads, kv_heads=stored, head_dim=self.padded_dim,
-            extra_columns=gate_columns, q_temperature=self.q_temperature, bias=self.b_qkv_own, **norms)
-        attended = ops.paged_attention(
-            q, k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size,
-            block_tables=cache.block_tables, row_seq=ctx.row_seq, positions=ctx.positions,
-            cu_seqlens=ctx.cu_seqlens, seq_starts=ctx.seq_starts, single_rows=ctx.single_rows, n_seqs=ctx.n_seqs,
-            max_query=ctx.max_query, max_context=ctx.max_context, tile_seqs=ctx.tile_seqs,
-            scale=self.scale, window=self.window, unmerged=False, softcap=self.softcap, sinks=p.get('sinks'), **sizes)
+                max_context=ctx.max_context, unmerged=False, rotate_first=self.norm_after_rotation, has_kv=self.own_kv,
+                extra_columns=gate_columns, bias=self.b_qkv_own, q_temperature=self.q_temperature,
+                values_are_keys=self.values_are_keys, **masks, **sizes, **norms)
+        else:
+            store = dict(rotation=rotation, positions=ctx.positions, slots=cache.slots if cache.writes else None,
+                         k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size, dtype=self.dtype, heads=self.heads,
+                         kv_heads=stored, head_dim=self.padded_dim, extra_columns=gate_columns,
+                         values_are_keys=self.values_are_keys, **norms)
+            if rows:
+                q = ops.qk_row_norm_store(qkv, q_elems=self.heads * self.head_dim, k_elems=self.kv_heads * self.head_dim, **store)
+            else:
+                q = ops.qk_norm_rope_store(qkv, norm_dim=self.head_dim, rotate_first=self.norm_after_rotation,
+                                           q_temperature=self.q_temperature, bias=self.b_qkv_own, **store)
+            attended = ops.paged_attention(
+                q, k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size,
+                block_tables=cache.block_tables, row_seq=ctx.row_seq, positions=ctx.positions,
+                cu_seqlens=ctx.cu_seqlens, seq_starts=ctx.seq_starts, single_rows=ctx.single_rows, n_seqs=ctx.n_seqs,
+                max_query=ctx.max_query, max_context=ctx.max_context, tile_seqs=ctx.tile_seqs, unmerged=False, **masks, **sizes)
         if self.gate:
-            attended = ops.sigmoid_gate(attended, qkv, offset=(self.heads + 2 * stored) * self.padded_dim)
+            attended = ops.sigmoid_gate(attended, qkv, offset=own)
         return ops.linear(attended, p['o_proj.weight'], p.get('o_proj.bias'), partials=True)

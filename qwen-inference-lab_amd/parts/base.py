@@ -31,10 +31,12 @@ class ParamSpec:
 
 @dataclass(frozen=True)
 class KVNeed:
-    """Per-token keys and values in pages.  ``window`` None keeps every key."""
+    """Per-token keys and values in pages.  ``window`` None keeps every key; ``keep_first``: behind a window, the first
+    so many tokens are kept for good."""
     kv_heads: int
     head_dim: int
     window: int | None = None
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -83,6 +85,22 @@ class Part:
 
     def finalize(self):
         """Called once after every declared tensor is set."""
+
+    def after_finalize(self):
+        """Called once after ``finalize`` of every part of the model (a block may lay its parts' tensors together)."""
+
+    def input_matrices(self):
+        """Names in ``p`` of the matrices whose products with the part's input the part asks ``ops.linear`` (or
+        ``ops.gated_linear``) for, without a bias: a block whose parts read the same input may lay them one behind
+        another (``ops.SharedInput``).  Empty: the part's input must be a tensor."""
+        return ()
+
+    def matrix(self, name):
+        return self.p[name]
+
+    def place_matrix(self, name, tensor):
+        """``tensor`` holds what ``p[name]`` holds, in memory that other parts' matrices share; use it from now on."""
+        self.p[name] = tensor
 
     def parameter_bytes(self):
         return sum(t.numel() * t.element_size() for t in self.p.values())
@@ -176,6 +194,9 @@ class Block(Part):
     ``ops.Added`` says that the output is in the stream already.
     """
     mixer = None
+    # True if forward takes an ``ops.Joined`` as pending: then a schedule entry of the block may add the embedding's
+    # output or a pass's vector to the stream before the run.
+    takes_pass_start = False
 
     def parts(self):
         """dict local prefix -> Part (for naming tensors)."""

@@ -187,3 +187,78 @@ class PostNormBlock(Block):
             self._join(stream, self.ffn.forward(stream if h is None else h), self.ffn_post_norm, 'ffn_scale', None, history,
                        True)
         return ops.Averaged(history, self.depth) if self.depth is not None else ops.Added(None)
+
+
+class ParallelBlock(Block):
+    """One norm, mixer and feed-forward side by side on its output: h = norm(x), x <- x + g1 * mixer(h) + g2 * ffn(h) (or
+    the mixer alone).  ``gated``: g1, g2 are made per channel from the same input, sigmoid(W h + b) (tensors
+    ``mixer_gate.weight`` [width, width], ``mixer_gate.bias``, and ``ffn_gate.*``); without it they are 1.
+
+    The results leave the block as an ``ops.Joined`` (not yet gated, not yet added), and the norm that follows, the next
+    block's or the model's last, makes the gates, the sum and its own norm in one kernel, all in float32.  All parts read
+    h: on the GPU the matrices of those that say which (``input_matrices``) and the gates' matrices are laid one behind
+    another at ``after_finalize``, every matrix at a multiple of 16 rows, and one product serves them all
+    (``ops.SharedInput``); the parts then read their columns of it."""
+    takes_pass_start = True
+
+    def __init__(self, *, norm, mixer, ffn=None, gated=False, width, dtype, names=None):
+        super().__init__()
+        self.norm, self.mixer, self.ffn, self.gated, self.width, self.dtype = norm, mixer, ffn, bool(gated), int(width), dtype
+        self._names = names or dict(norm='norm', mixer='mixer', ffn='ffn')
+        self.stack, self.places = None, {}
+
+    def parts(self):
+        n = self._names
+        out = {n['norm']: self.norm, n['mixer']: self.mixer}
+        if self.ffn is not None:
+            out[n['ffn']] = self.ffn
+        return out
+
+    def param_specs(self):
+        if not self.gated:
+            return {}
+        specs = {}
+        for name in ('mixer_gate',) + (('ffn_gate',) if self.ffn is not None else ()):
+            specs[f'{name}.weight'] = ParamSpec((self.width, self.width))
+            specs[f'{name}.bias'] = ParamSpec((self.width,), 'vector')
+        return specs
+
+    def finalize(self):
+        if not self.gated:
+            return
+        names = ['mixer_gate'] + (['ffn_gate'] if self.ffn is not None else [])
+        self.p['gates.weight'] = torch.cat([self.p.pop(f'{name}.weight') for name in names]).contiguous()
+        self.p['gates.bias'] = torch.cat([self.p.pop(f'{name}.bias') for name in names]).contiguous()
+
+    def _stacked(self):
+        """(part, name) of every matrix that reads h and may share the product."""
+        out = [(self.mixer, name) for name in self.mixer.input_matrices()]
+        if self.ffn is not None:
+            out += [(self.ffn, name) for name in self.ffn.input_matrices()]
+        return out + ([(self, 'gates.weight')] if self.gated else [])
+
+    def after_finalize(self):
+        members = self._stacked()
+        if len(members) < 2 or not members[0][0].matrix(members[0][1]).is_cuda:
+            return
+        matrices = [part.matrix(name) for part, name in members]
+        rows, at = [], 0
+        for matrix in matrices:
+            rows.append(at)
+            at += -(-matrix.shape[0] // 16) * 16
+        self.stack = matrices[0].new_zeros((at, matrices[0].shape[1]))
+        for (part, name), matrix, first in zip(members, matrices, rows):
+            place = self.stack[first:first + matrix.shape[0]]
+            place.copy_(matrix)
+            part.place_matrix(name, place)
+            self.places[id(place)] = first
+
+    def forward(self, stream, pending, ctx, cache):
+        if pending is None or isinstance(pending, ops.Added):          # the stream is complete
+            pending = ops.Joined()
+        h = self.norm.forward(stream, pending, self.dtype)
+        shared = ops.SharedInput(h, self.stack, self.places) if self.stack is not None else h
+        mixed = self.mixer.forward(shared if self.mixer.input_matrices() else h, ctx, cache)
+        ffn = self.ffn.forward(shared if self.ffn.input_matrices() else h) if self.ffn is not None else None
+        gates = ops.linear(shared, self.p['gates.weight'], None, partials=True) if self.gated else None
+        return ops.Joined(mixed, ffn, gates, self.p.get('gates.bias'))

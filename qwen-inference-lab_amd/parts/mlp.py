@@ -7,8 +7,9 @@ from .. import ops
 
 class GatedMLP(FeedForward):
     """``activation`` names the gate's function (``ops.GATE_FUNCTIONS``): 'silu', silu(g) * u, or 'clamped_swish' with
-    ``limit`` L and ``alpha`` a: g' = min(g, L), u' = clamp(u, -L, L), g' * sigmoid(a g') * (u' + 1).  Gate and up matrices become one [2 * intermediate, width] matrix at
-    ``finalize`` (rows in turns of 16, or gate rows first where the sizes do not allow that): a pure re-layout."""
+    ``limit`` L and ``alpha`` a: g' = min(g, L), u' = clamp(u, -L, L), g' * sigmoid(a g') * (u' + 1), or 'relu', max(g, 0) * u.
+    Gate and up matrices become one [2 * intermediate, width] matrix at ``finalize`` (rows in turns of 16, or gate rows
+    first where the sizes do not allow that): a pure re-layout."""
 
     def __init__(self, *, width, intermediate, activation='silu', limit=None, alpha=1.0, dtype=torch.bfloat16):
         super().__init__()
@@ -33,6 +34,9 @@ class GatedMLP(FeedForward):
         p['gate_up_proj.weight'] = ops.interleave_gate_up(gate, up) if self.interleaved else torch.cat([gate, up]).contiguous()
 
     adds_to_stream = True
+
+    def input_matrices(self):
+        return () if self.activation == 'silu' else ('gate_up_proj.weight',)     # (silu has products with the activation inside)
 
     def forward(self, h, add_to=None):
         hidden = ops.gated_linear(h, self.p['gate_up_proj.weight'], self.dtype, interleaved=self.interleaved, lazy=True,

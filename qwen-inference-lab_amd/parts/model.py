@@ -15,9 +15,14 @@ class ScheduleEntry:
     cache_of  None: the entry owns a cache of its mixer's need; an earlier entry's
               position in the schedule: the entry reads that entry's cache and
               writes nothing
+    add_embedding, add_vector
+              what is added to the stream before the run (the start of a pass of a loop over layers): the
+              embedding's output, and vector number ``add_vector`` of the model's ``pass_vectors``
     """
     block: int
     cache_of: int | None = None
+    add_embedding: bool = False
+    add_vector: int | None = None
 
 
 class CausalLM:
@@ -30,7 +35,8 @@ class CausalLM:
     """
 
     def __init__(self, *, config, embedding, blocks, schedule, final_norm, head, names, tied=None,
-                 dtype=torch.bfloat16, device='cuda', residual_scale=1.0):
+                 dtype=torch.bfloat16, device='cuda', residual_scale=1.0, pass_vectors=None):
+        self.pass_vectors = pass_vectors                # a ``PassVectors`` part, or None
         self.residual_scale = float(residual_scale)     # what the last block's output is multiplied by as it is added
         self.observer = None                            # callable(schedule position, stream, pending, scale) or None
         self.config, self.embedding, self.blocks, self.schedule = config, embedding, list(blocks), list(schedule)
@@ -44,6 +50,12 @@ class CausalLM:
                     raise ValueError(f'schedule entry {position}: cache_of must name an earlier owning entry')
                 if self._need(entry) != self._need(self.schedule[entry.cache_of]):
                     raise ValueError(f'schedule entry {position}: shared cache has another geometry')
+            if entry.add_embedding or entry.add_vector is not None:
+                if not self.blocks[entry.block].takes_pass_start:
+                    raise ValueError(f'schedule entry {position}: its block does not take what a pass adds to the stream')
+                if entry.add_vector is not None and not (pass_vectors is not None and 0 <= entry.add_vector < pass_vectors.passes):
+                    raise ValueError(f'schedule entry {position}: there is no vector {entry.add_vector}')
+        self.keeps_embedding = any(entry.add_embedding for entry in self.schedule)
         declared = {(id(part), local) for part in self.all_parts() for local in part.param_specs()}
         mapped = {(id(part), local) for part, local in self.names.values()}
         if declared != mapped:
@@ -65,6 +77,8 @@ class CausalLM:
             visit(block)
             for part in block.parts().values():
                 visit(part)
+        if self.pass_vectors is not None:
+            visit(self.pass_vectors)
         visit(self.final_norm)
         visit(self.head)
         return out
@@ -81,8 +95,11 @@ class CausalLM:
         return needs
 
     def finalize(self):
-        for part in self.all_parts():
+        parts = self.all_parts()
+        for part in parts:
             part.finalize()
+        for part in parts:
+            part.after_finalize()
         self.loaded = True
 
     def parameter_bytes(self):
@@ -98,9 +115,16 @@ class CausalLM:
         Rows are selected before the final norm; with no wanted row neither the
         norm nor the head runs (qil/model.py:130-134).
         """
-        stream = self.embedding.forward_step(ctx)
+        if self.keeps_embedding:
+            stream, embedded = self.embedding.forward_step_kept(ctx)
+        else:
+            stream, embedded = self.embedding.forward_step(ctx), None
         pending = None
         for position, (entry, cache) in enumerate(zip(self.schedule, caches)):
+            if entry.add_embedding or entry.add_vector is not None:
+                pending = ops.joined_with_pass(
+                    pending, embedded if entry.add_embedding else None,
+                    self.pass_vectors.vectors[entry.add_vector] if entry.add_vector is not None else None)
             pending = self.blocks[entry.block].forward(stream, pending, ctx, cache)
             if self.observer is not None:                       # the stream after this run is stream + scale * pending
                 self.observer(position, stream, pending, self.residual_scale)

@@ -23,6 +23,8 @@ class RMSNorm(Norm):
             self.p['weight'] = (self.p['weight'] + self.offset).contiguous()
 
     def forward(self, stream, delta, out_dtype, delta_scale=1.0):
+        if isinstance(delta, ops.Joined):
+            return ops.residual_join(stream, delta, self.p['weight'], self.eps, out_dtype)
         if delta_scale != 1.0:                      # (the general kernel rounds once, after the weight)
             return ops.add_norm(stream, delta, self.p['weight'], self.eps, out_dtype, centre=False, delta_scale=delta_scale)
         return ops.add_rmsnorm(stream, delta, self.p['weight'], self.eps, out_dtype)
@@ -33,6 +35,8 @@ class RMSNorm(Norm):
         return None
 
     def forward_rows(self, stream, delta, rows, out_dtype, delta_scale=1.0):
+        if isinstance(delta, ops.Joined):
+            return ops.residual_join(stream, delta, self.p['weight'], self.eps, out_dtype, rows=rows)
         if delta_scale != 1.0:
             return ops.rows_norm(stream, delta, rows, self.p['weight'], self.eps, out_dtype, centre=False,
                                  delta_scale=delta_scale)

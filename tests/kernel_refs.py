@@ -9,7 +9,9 @@ import torch
 
 
 def _value(x):
-    """A tensor, or the sum of float32 partial sums."""
+    """A tensor, the sum of float32 partial sums, or columns of either."""
+    if hasattr(x, 'source') and hasattr(x, 'offset'):
+        return _value(x.source)[:, x.offset:x.offset + x.shape[1]]
     return x.sum() if hasattr(x, 'splits') else x
 
 
@@ -64,6 +66,8 @@ def _halves(gate_up, interleaved):
 
 
 def _gate(g, u, activation='silu', limit=0.0, alpha=1.0):
+    if activation == 'relu':
+        return g.clamp(min=0.0) * u
     if activation == 'clamped_swish':
         g, u = g.clamp(max=limit), u.clamp(min=-limit, max=limit)
         return g / (1 + torch.exp(-alpha * g)) * (u + 1)
@@ -84,18 +88,25 @@ def silu_mul(gate_up, out_dtype=None, interleaved=False):
 
 def qk_norm_rope_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps, rotation, positions, slots,
                        k_cache, v_cache, page_size, dtype, norm_dim=None, rotate_first=False, extra_columns=0,
-                       q_temperature=None, bias=None):
+                       q_temperature=None, bias=None, values_are_keys=False, q_elems=None, k_elems=None):
+    """(``q_elems``, ``k_elems``: the norms run over all heads of a row, over so many elements: ``qk_row_norm_store``.)"""
     qkv = _value(qkv)
     n, d = qkv.shape[0], head_dim
-    x = qkv[:, :(heads + 2 * kv_heads) * d]
+    pieces = heads + (1 if values_are_keys else 2) * kv_heads
+    x = qkv[:, :pieces * d]
     if bias is not None:
         x = x.to(torch.float32) + bias
-    x = x.reshape(n, heads + 2 * kv_heads, d)
-    q, k, v = x[:, :heads].to(torch.float32), x[:, heads:heads + kv_heads].to(torch.float32), x[:, heads + kv_heads:]
+    x = x.reshape(n, pieces, d)
+    q, k = x[:, :heads].to(torch.float32), x[:, heads:heads + kv_heads].to(torch.float32)
+    v = x[:, heads:heads + kv_heads] if values_are_keys else x[:, heads + kv_heads:]
 
     def normed(t, weight):
         if weight is None:
             return t
+        if q_elems is not None:
+            flat = t.reshape(n, -1)
+            mean = flat.square().sum(dim=-1, keepdim=True) / (q_elems if t.shape[1] == heads and weight is q_weight else k_elems)
+            return (flat / torch.sqrt(mean + eps) * weight).reshape(t.shape)
         return _round(t * torch.rsqrt(t.square().sum(dim=-1, keepdim=True) / (norm_dim or d) + eps), dtype) * weight
 
     def turned(t):
@@ -127,9 +138,14 @@ def qk_norm_rope_store(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, ep
     return shape(q, q_weight).reshape(n, heads * d)
 
 
+def qk_row_norm_store(qkv, *, q_elems, k_elems, **rest):
+    return qk_norm_rope_store(qkv, q_elems=q_elems, k_elems=k_elems, **rest)
+
+
 def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size, block_tables, row_seq, positions,
                     cu_seqlens, seq_starts, single_rows, n_seqs, max_query, max_context, scale, window,
-                    unmerged=False, tile_seqs=None, softcap=None, sinks=None, accumulate=torch.float32):
+                    unmerged=False, tile_seqs=None, softcap=None, sinks=None, slopes=None, keep_first=0,
+                    accumulate=torch.float32):
     n, d, g = q.shape[0], head_dim, heads // kv_heads
     qkv = q
     q = q.reshape(n, heads, d).to(accumulate)
@@ -138,6 +154,8 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
         ctx = int(positions[row]) + 1
         lo = max(0, ctx - window) if window else 0
         j = torch.arange(lo, ctx, device=qkv.device)
+        if keep_first and lo > 0:
+            j = torch.cat([torch.arange(min(keep_first, lo), device=qkv.device), j])
         pages = block_tables[int(row_seq[row])].long()[j // page_size]
         keys = k_cache[pages, :, j % page_size].to(accumulate)          # [ctx, kv_heads, d]
         values = v_cache[pages, :, :, j % page_size].to(accumulate)     # [ctx, kv_heads, d]
@@ -146,6 +164,8 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
         scores = torch.einsum('hd,jhd->hj', q[row], keys) * scale
         if softcap:
             scores = softcap * torch.tanh(scores / softcap)
+        if slopes is not None:
+            scores = scores - slopes.to(accumulate)[:, None] * (ctx - 1 - j).to(accumulate)[None, :]
         if sinks is not None:                        # one more term in the divisor: no key, no value
             scores = torch.cat([scores, sinks.to(accumulate)[:, None]], dim=-1)
             out[row] = torch.einsum('hj,jhd->hd', torch.softmax(scores, dim=-1)[:, :-1], values)
@@ -323,13 +343,16 @@ def state_scan_slot(*, heads, dim, vdim, mode):
 
 def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, state, cu_seqlens, seq_starts, seq_slots,
                n_seqs, gates=None, gate_bias=None, cap=0.0, decay=None, frequencies=None, rot=0, q_scale=1.0, k_scale=1.0,
-               max_query=None):
+               max_query=None, groups=None):
     """Token by token whatever ``max_query`` says.  -> (o, denominators): for 'mlstm' o is undivided and the denominators are returned beside it.  The state slot's
     layout is the kernel's: matrices, then a normaliser per head, then the maximum tiles + 1 times per head."""
     n, tiles = proj.shape[0], -(-vdim // 16)
     x = proj.to(torch.float32)
-    q = x[:, q_offset:q_offset + heads * dim].reshape(n, heads, dim).clone()
-    k = x[:, k_offset:k_offset + heads * dim].reshape(n, heads, dim).clone()
+    shared = groups if mode == 'step' else heads
+    q = x[:, q_offset:q_offset + shared * dim].reshape(n, shared, dim).repeat_interleave(heads // shared, dim=1)
+    k = x[:, k_offset:k_offset + shared * dim].reshape(n, shared, dim).repeat_interleave(heads // shared, dim=1)
+    if mode == 'step':
+        steps = torch.nn.functional.softplus(_value(gates).to(torch.float32) + gate_bias, threshold=20.0)
     v = x[:, v_offset:v_offset + heads * vdim].reshape(n, heads, vdim)
     out = torch.zeros((n, heads, vdim), dtype=torch.float32)
     below = torch.zeros((n, heads), dtype=torch.float32) if mode == 'mlstm' else None
@@ -362,6 +385,8 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
                 memory = a * memory + ks[t][:, :, None] * v[lo + t][:, None, :]
                 out[lo + t] = torch.einsum('hdv,hd->hv', memory, qs[t])
                 continue
+            elif mode == 'step':
+                a, b = torch.exp(decay * steps[lo + t]), steps[lo + t]
             else:
                 a, b = decay, torch.ones(heads)
             memory = a[:, None, None] * memory + b[:, None, None] * ks[t][:, :, None] * v[lo + t][:, None, :]
@@ -387,6 +412,46 @@ def head_norm_gate(o, gate_source, *, gate_offset, heads, vdim, weight, eps, gat
         unit = unit * weight
     g = gate_source[:, gate_offset:gate_offset + heads * vdim].to(torch.float32)
     return (unit * (torch.sigmoid(g) if gate == 'sigmoid' else g * torch.sigmoid(g))).to(out_dtype)
+
+
+def gated_group_norm(o, u, *, skip, z, weight, vdim, groups, eps, out_dtype):
+    n, inner = o.shape
+    z = _value(z).to(torch.float32)
+    v = (o + skip.repeat_interleave(vdim) * u[:, :inner].to(torch.float32)) * (z * torch.sigmoid(z))
+    v = v.reshape(n, groups, -1)
+    v = (v / torch.sqrt(v.square().mean(dim=-1, keepdim=True) + eps)).reshape(n, inner)
+    return (v * weight).to(out_dtype)
+
+
+def embed_pairs(token_ids, previous, table, pairs, *, scale, buckets, mul_prev, mul_cur, keep=False):
+    before, now = previous.long(), token_ids.long()
+    row = torch.where(before < 0, torch.full_like(now, buckets), (before * mul_prev + now * mul_cur) % buckets)
+    stream = table[now].to(torch.float32) * scale + pairs[row].to(torch.float32)
+    return (stream, stream.clone()) if keep else stream
+
+
+def residual_join(stream, pending, weight, eps, out_dtype, rows=None):
+    x = stream.clone()
+    width = stream.shape[1]
+    if pending.mixed is not None:
+        mixed = pending.mixed
+        if hasattr(mixed, 'left_scale'):
+            mixed = mixed.left_scale * _value(mixed.left).to(torch.float32) + mixed.right_scale * _value(mixed.right).to(torch.float32)
+        else:
+            mixed = _value(mixed).to(torch.float32)
+        gates = torch.sigmoid(_value(pending.gates).to(torch.float32) + pending.bias) if pending.gates is not None else None
+        x += mixed * (gates[:, :width] if gates is not None else 1.0)
+        if pending.ffn is not None:
+            x += _value(pending.ffn).to(torch.float32) * (gates[:, width:] if gates is not None else 1.0)
+    if pending.plus is not None:
+        x += pending.plus
+    if pending.step is not None:
+        x += pending.step
+    if rows is None:
+        stream.copy_(x)
+    else:
+        x = x[rows.long()]
+    return (x / torch.sqrt(x.square().mean(dim=-1, keepdim=True) + eps) * weight).to(out_dtype)
 
 
 def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bias=None, score='softmax',
@@ -497,4 +562,6 @@ ALL = dict(scaled_sum=scaled_sum, sigmoid_gate=sigmoid_gate, soft_cap=soft_cap, 
            qk_norm_rope_store=qk_norm_rope_store, paged_attention=paged_attention, sample=sample,
            add_norm=add_norm, rows_norm=rows_norm, gated_act=gated_act, latent_prepare=latent_prepare, head_product=head_product,
            latent_query=latent_query, latent_attention=latent_attention, state_scan_slot=state_scan_slot, state_scan=state_scan,
-           head_norm_gate=head_norm_gate, plain_act=plain_act, post_norm_scale_add=post_norm_scale_add, short_conv=short_conv)
+           head_norm_gate=head_norm_gate, plain_act=plain_act, post_norm_scale_add=post_norm_scale_add, short_conv=short_conv,
+           qk_row_norm_store=qk_row_norm_store, gated_group_norm=gated_group_norm, embed_pairs=embed_pairs,
+           residual_join=residual_join)
