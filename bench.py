@@ -285,6 +285,30 @@ def dogozen_config(z, layers, vocab, window, kind='turns'):
     return dict(architecture='Dogozen', vocab=vocab, width=z['width'], layers=made, norm=dict(eps=1e-6), logit_softcap=30.0)
 
 
+def tinuzen_config(z, layers, vocab, window, kind='turns'):
+    """`layers` layers of the Tinuzen design, a relu-gated feed-forward beside the mixer of each: attention whose values
+    are its keys beside a state-space recurrence (twice the width in heads of 64 channels, 128 states, 8 groups, four
+    taps), or attention with a bias by distance and a window behind 64 kept first keys, or both in turns ('loop': the turns,
+    half as many layers run twice); every bigram has a row of its own table of 8,191."""
+    kv = max(1, z['heads'] // 4)
+    left = dict(heads=z['heads'], kv_heads=kv, dim=z['dim'], vdim=z['dim'], scale=z['dim'] ** -0.5, rot=dict(base=10000.0, dims=z['rot_dim']))
+    right = dict(heads=2 * z['width'] // 64, vdim=64, state=128, groups=8, conv=4, norm_groups=8)
+    dense = dict(kind='dense', ff=z['ff'])
+    both = dict(type='parallel', mlp=dense, mixer=dict(left=left, right=right, left_scale=0.5, right_scale=0.5))
+    attention = dict(type='attention', mlp=dense,
+                     mixer=dict(heads=z['heads'], kv_heads=kv, dim=z['dim'], vdim=z['dim'], scale=z['dim'] ** -0.5,
+                                mask=dict(size=window, keep_first=64)))
+    small = dict(both, mixer=dict(both['mixer'], right=dict(heads=1, vdim=64, state=16, groups=1, conv=4, norm_groups=1)))
+    kinds = dict(turns=[both, attention], loop=[both, attention], parallel=[both], attention=[attention], left=[small])[kind]
+    out = dict(architecture='Tinuzen', vocab=vocab, width=z['width'], norm=dict(eps=1e-6),
+               embedding=dict(scale=z['width'] ** 0.5, bigram=dict(buckets=8191, mul_prev=31, mul_cur=17)),
+               layers=[kinds[i % len(kinds)] for i in range(layers)])
+    if kind == 'loop':
+        out['layers'] = out['layers'][:max(1, layers // 2)]
+        out['loop'] = dict(start=0, stop=max(1, layers // 2), times=2)
+    return out
+
+
 def designs_phase(args, torch, dtype):
     """Prefill tokens a second and decode milliseconds a step of a design's models whose layers are all of one kind
     (and of its kinds in turns), beside dense Qwen3 of the same width, feed-forward, depth and attention heads."""
@@ -309,6 +333,17 @@ def designs_phase(args, torch, dtype):
                  ('window', f'window {args.design_window} beside a scan of one channel group, dense feed-forwards'))
         models = {f'dogozen ({name})': dogozen_config(z, layers, vocab, args.design_window, kind) for kind, name in names}
         models['gerivik (capped attention only)'] = dict(gerivik_config(z, layers, vocab), layers=[gerivik_config(z, 2, vocab)['layers'][1]] * layers)
+    elif args.design == 'tinuzen':
+        # beside it the closest models of the engine: Dogozen's two kinds of layer with dense feed-forwards (two mixers side
+        # by side, one of them a state-space scan; gated attention) and Fubapel's memory with fixed decays (a matrix
+        # state per head)
+        names = (('turns', f'kinds in turns, window {args.design_window}'), ('loop', 'kinds in turns, half the layers twice'),
+                 ('parallel', 'attention beside a recurrence'), ('attention', f'window {args.design_window} with a bias by distance'),
+                 ('left', 'attention beside a recurrence of one head'))
+        models = {f'tinuzen ({name})': tinuzen_config(z, layers, vocab, args.design_window, kind) for kind, name in names}
+        models['dogozen (window beside a scan)'] = dogozen_config(z, layers, vocab, args.design_window, 'parallel')
+        models['dogozen (gated attention)'] = dogozen_config(z, layers, vocab, args.design_window, 'attention')
+        models['fubapel (decaying memory only)'] = dict(fubapel_config(z, layers, vocab), layers=[fubapel_config(z, 3, vocab)['layers'][2]] * layers)
     elif args.design == 'gerivik':
         mixed = gerivik_config(z, layers, vocab)
         models = {'gerivik (kinds in turns)': mixed}
@@ -390,8 +425,8 @@ def main():
                              'attention kernels alone, at the reference\'s own shapes and at the benchmark\'s.  products: a layer\'s '
                              'matrix products at --prefill-tokens rows alone, GPU BLAS against own kernel.  designs: prefill and decode of the '
                              'design named by --design at --design-sizes beside dense Qwen3 of equal sizes (--layers, default 6)')
-    parser.add_argument('--design', default='fubapel', choices=['fubapel', 'gerivik', 'zinesun', 'dogozen'], help='the design of --phase designs')
-    parser.add_argument('--design-window', type=int, default=512, help='the attention window of --design zinesun and --design dogozen')
+    parser.add_argument('--design', default='fubapel', choices=['fubapel', 'gerivik', 'zinesun', 'dogozen', 'tinuzen'], help='the design of --phase designs')
+    parser.add_argument('--design-window', type=int, default=512, help='the attention window of --design zinesun, dogozen and tinuzen')
     parser.add_argument('--design-only', default=None, help='of the models of --phase designs, only those whose name holds this (for profiling)')
     parser.add_argument('--design-sizes', default='1b', choices=sorted(DESIGN_SIZES), help='layer sizes of --phase designs')
     parser.add_argument('--portion', type=int, default=128, help='tokens of the prompt portion of a mixed step')
