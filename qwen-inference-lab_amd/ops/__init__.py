@@ -1393,6 +1393,7 @@ def latent_attention(q, *, latent, rope, page_size, block_tables, row_seq, posit
 # ---------------------------------------------------------------------------------------------------------------
 # Recurrences with a matrix state
 SCAN_MODES = {'decay': 0, 'mlstm': 1, 'channel': 2, 'step': 3}
+STEP_FORMS = True               # False: mode 'step' runs on the general kernels only (tests)
 SCAN_BLOCKS_FROM = 32           # rows of one sequence from which a step's recurrence runs in blocks side by side
 
 
@@ -1463,6 +1464,21 @@ def state_scan(proj, *, mode, heads, dim, vdim, q_offset, k_offset, v_offset, st
     if rot:
         _require(frequencies, 'frequencies', torch.float32, (rot // 2,))
     out = torch.empty((n, heads * vdim), dtype=torch.float32, device=proj.device)
+    if mode == 'step' and STEP_FORMS and max_query is not None:
+        # kernels of the mode's own: one token a sequence, and many tokens of bfloat16 rows on the matrix cores
+        head = (_ptr(proj), width, q_offset, k_offset, v_offset)
+        if max_query == 1 and n == n_seqs and lib.qil_step_token_takes(dim, vdim):
+            _check(lib.qil_step_token(head[0], code, *head[1:], *raw, _ptr(gate_bias), _ptr(decay), _ptr(state), _ptr(cu_seqlens),
+                                      _ptr(seq_starts), _ptr(seq_slots), _ptr(out), n, n_seqs, heads, shared, dim, vdim,
+                                      _stream()), 'step_token')
+            return out, None
+        if max_query >= SCAN_BLOCKS_FROM and code == 1 and lib.qil_step_scan_takes(width, q_offset, k_offset, v_offset, dim, vdim):
+            floats = lib.qil_step_scan_workspace(n, n_seqs, heads, dim, vdim)
+            workspace = torch.empty(floats, dtype=torch.float32, device=proj.device)
+            _check(lib.qil_step_scan(*head, *raw, _ptr(gate_bias), _ptr(decay), _ptr(state), _ptr(cu_seqlens),
+                                     _ptr(seq_starts), _ptr(seq_slots), _ptr(out), _ptr(workspace), n, n_seqs,
+                                     int(max_query), heads, shared, dim, vdim, _stream()), 'step_scan')
+            return out, None
     below = torch.empty((n, heads), dtype=torch.float32, device=proj.device) if mode == 'mlstm' else None
     if max_query is not None and max_query >= SCAN_BLOCKS_FROM:
         floats = lib.qil_state_scan_chunked_workspace(n, n_seqs, heads, dim, vdim, SCAN_MODES[mode])

@@ -357,7 +357,13 @@ def _declare(lib):
     lib.qil_embed_pairs.argtypes = [p, p, p, p, p, p, i, i, f, i, ll, ll, i, p]
     lib.qil_gated_group_norm.argtypes = [p, p, i, p, p, i, i, i, p, p, i, i, i, i, i, f, f, i, p]
     lib.qil_residual_join.argtypes = [p, p, i, i, i, f, p, i, i, i, f, p, i, i, i, p, i, i, i, p, p, p, p, p, p, i, i, i, f, i, i, p]
-    for name in ('qil_embed_pairs', 'qil_gated_group_norm', 'qil_residual_join', 'qil_qk_row_norm_store'):
+    lib.qil_step_scan_takes.argtypes = [i, i, i, i, i, i]
+    lib.qil_step_token_takes.argtypes = [i, i]
+    lib.qil_step_scan_workspace.argtypes = [i, i, i, i, i]
+    lib.qil_step_scan_workspace.restype = z
+    lib.qil_step_scan.argtypes = [p, i, i, i, i, p, i, i, i, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
+    lib.qil_step_token.argtypes = [p, i, i, i, i, i, p, i, i, i, p, p, p, p, p, p, p, i, i, i, i, i, i, p]
+    for name in ('qil_step_scan_takes', 'qil_step_token_takes', 'qil_step_scan', 'qil_step_token', 'qil_embed_pairs', 'qil_gated_group_norm', 'qil_residual_join', 'qil_qk_row_norm_store'):
         getattr(lib, name).restype = i
     lib.qil_sample.argtypes = [p, p, p, p, p, p, p, i, i, p]
     lib.qil_sample_workspace.argtypes = [i, i]

@@ -186,8 +186,9 @@ def test_decoding_with_queries_made_inside_is_the_two_kernels(lengths, page_size
 # ------------------------------------------------------------------------------------------------ the recurrence
 @pytest.mark.parametrize('dtype', DTYPES)
 @pytest.mark.parametrize('heads,dim,vdim,groups,splits', [(4, 128, 64, 2, 3), (6, 33, 7, 3, 0), (1, 1, 1, 1, 1), (3, 200, 70, 1, 2),
-                                                          (8, 64, 128, 8, 0), (5, 16, 130, 5, 4), (16, 128, 64, 1, 0)])
-def test_recurrence_with_step_sizes(dtype, heads, dim, vdim, groups, splits):
+                                                          (8, 64, 128, 8, 0), (5, 16, 130, 5, 4), (16, 128, 64, 1, 0), (2, 256, 72, 2, 2),
+                                                          (4, 40, 8, 2, 1)])
+def test_recurrence_with_step_sizes(dtype, heads, dim, vdim, groups, splits, monkeypatch):
     """Three sequences of unequal lengths with states of their own (one begins, whatever its slot holds), in blocks side by
     side and token by token; then the second part of each from what the first left."""
     if dtype == torch.float32 and splits == 0:
@@ -209,7 +210,8 @@ def test_recurrence_with_step_sizes(dtype, heads, dim, vdim, groups, splits):
     want, _ = refs.state_scan(u, gates=ops.columns(raw, 5, heads), gate_bias=bias, decay=rates, state=want_state,
                               cu_seqlens=cu, seq_starts=ints(starts), seq_slots=ints(slots), n_seqs=3, **columns)
     scale = max(1.0, want.abs().max().item())
-    for longest in (150, None):
+    for longest, forms in ((150, True), (150, False), (None, True)):   # the matrix cores where they take the sizes; the general kernels
+        monkeypatch.setattr(ops, 'STEP_FORMS', forms)
         got_state = state.cuda()
         got, _ = ops.state_scan(u.cuda(), gates=ops.columns(moved(raw), 5, heads), gate_bias=bias.cuda(), decay=rates.cuda(),
                                 state=got_state, cu_seqlens=cu.cuda(), seq_starts=ints(starts).cuda(), seq_slots=ints(slots).cuda(),
@@ -218,6 +220,54 @@ def test_recurrence_with_step_sizes(dtype, heads, dim, vdim, groups, splits):
         live = [2, 0, 3]
         torch.testing.assert_close(got_state.cpu()[live], want_state[live], atol=2e-5 * scale, rtol=2e-5)
         assert torch.equal(got_state.cpu()[[1, 4]], state[[1, 4]]), 'a slot that belongs to nobody was written'
+
+
+@pytest.mark.parametrize('dtype', DTYPES)
+def test_recurrence_in_long_blocks(dtype):
+    """Many blocks a sequence, the second half from the state the first left; decays from a token's to thousands of tokens'."""
+    g = torch.Generator().manual_seed(5)
+    heads, dim, vdim, groups, n = 4, 128, 64, 2, 900
+    inner, shared = heads * vdim, groups * dim
+    u = (torch.randn(n, inner + 2 * shared, generator=g) / 3).to(dtype)
+    raw, bias = torch.randn(n, heads, generator=g).to(dtype), torch.tensor([3.0, 0.0, -4.0, 25.0])
+    rates = torch.tensor([-20.0, -1e-4, -1.0, -1e-5])
+    columns = dict(mode='step', heads=heads, dim=dim, vdim=vdim, groups=groups, v_offset=0, k_offset=inner, q_offset=inner + shared)
+    want_state = torch.zeros(1, heads * dim * vdim)
+    want, _ = refs.state_scan(u, gates=raw, gate_bias=bias, decay=rates, state=want_state, cu_seqlens=ints([0, n]),
+                              seq_starts=ints([0]), seq_slots=ints([0]), n_seqs=1, **columns)
+    state, rows, at = torch.full((1, heads * dim * vdim), float('nan')).cuda(), [], 0
+    for size in (513, 1, 386):
+        part, _ = ops.state_scan(u[at:at + size].cuda(), gates=raw[at:at + size].cuda(), gate_bias=bias.cuda(), decay=rates.cuda(),
+                                 state=state, cu_seqlens=ints([0, size]).cuda(), seq_starts=ints([at]).cuda(),
+                                 seq_slots=ints([0]).cuda(), n_seqs=1, max_query=size, **columns)
+        rows.append(part)
+        at += size
+    got = torch.cat(rows).cpu().view(n, heads, vdim)
+    for h in range(heads):                             # (a head that sums everything is thousands of times larger than one that forgets)
+        expected = want.view(n, heads, vdim)[:, h]
+        torch.testing.assert_close(got[:, h], expected, atol=1e-5 * expected.abs().max().item(), rtol=1e-4)
+    torch.testing.assert_close(state.cpu(), want_state, atol=1e-5 * want_state.abs().max().item(), rtol=1e-4)
+
+
+@pytest.mark.parametrize('dtype', DTYPES)
+@pytest.mark.parametrize('lengths', [1, 5])
+@pytest.mark.parametrize('heads,dim,vdim,groups', [(64, 128, 64, 8), (3, 256, 256, 1), (2, 5, 4, 2), (4, 100, 32, 1)])
+def test_recurrence_one_token_a_sequence(dtype, lengths, heads, dim, vdim, groups):
+    g = torch.Generator().manual_seed(dim + vdim)
+    n, inner, shared = lengths, heads * vdim, groups * dim
+    u = torch.randn(n, inner + 2 * shared, generator=g).to(dtype)
+    raw, bias, rates = torch.randn(n, heads, generator=g).to(dtype), torch.randn(heads, generator=g), -torch.rand(heads, generator=g)
+    state = torch.randn(n + 2, heads * dim * vdim, generator=g)
+    starts, slots = ints([0 if i == 3 else 7 + i for i in range(n)]), ints([n + 1 - i for i in range(n)])
+    columns = dict(mode='step', heads=heads, dim=dim, vdim=vdim, groups=groups, v_offset=0, k_offset=inner, q_offset=inner + shared)
+    want_state, got_state = state.clone(), state.cuda()
+    index = dict(cu_seqlens=ints(range(n + 1)), seq_starts=starts, seq_slots=slots)
+    want, _ = refs.state_scan(u, gates=raw, gate_bias=bias, decay=rates, state=want_state, n_seqs=n, **index, **columns)
+    got, _ = ops.state_scan(u.cuda(), gates=raw.cuda(), gate_bias=bias.cuda(), decay=rates.cuda(), state=got_state, n_seqs=n,
+                            max_query=1, **{k: v.cuda() for k, v in index.items()}, **columns)
+    scale = want.abs().max().item()
+    torch.testing.assert_close(got.cpu(), want, atol=1e-5 * scale, rtol=1e-4)
+    torch.testing.assert_close(got_state.cpu(), want_state, atol=1e-5, rtol=1e-5)
 
 
 @pytest.mark.parametrize('dtype', DTYPES)
