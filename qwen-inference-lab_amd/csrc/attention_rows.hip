@@ -23,6 +23,7 @@
 // lane; a wave handles 64 / TG tokens at a time.
 #include "common.h"
 #include "key_span.h"
+#include "operand.h"
 
 #define ATT_THREADS 256
 #define ATT_WAVES (ATT_THREADS / QIL_WAVE)
@@ -245,7 +246,8 @@ __global__ void __launch_bounds__(QIL_WAVE)
 attn_rows_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_m,
                        const float* __restrict__ part_l, const int* __restrict__ positions,
                        const int* __restrict__ row_index, T* __restrict__ out, int heads, int d,
-                       int window, int P, int parts, int tg, const float* __restrict__ sinks, int keep) {
+                       int window, int P, int parts, int tg, const float* __restrict__ sinks, int keep, Operand gate,
+                       int gate_row) {
   const int slot_row = blockIdx.x;
   const int head = blockIdx.y * (QIL_WAVE / tg) + threadIdx.x / tg, e = (threadIdx.x % tg) * 4;
   const bool head_there = head < heads;                    // the same for the tg lanes of a head; all of them take part in the maximum
@@ -286,6 +288,13 @@ attn_rows_merge_kernel(const float* __restrict__ part_acc, const float* __restri
     }
   }
   T* to = out + ((size_t)row * heads + head) * d + e;
+  if (gate.data) {                                         // an output gate: the result times sigmoid of the gate's logits
+    const float r = sinks ? sink_reciprocal(denom, m, sinks[head]) : 1.f / denom;
+    const float4 g = operand_at4(gate, (size_t)row * gate_row + (size_t)head * d + e);
+    st4(to, make_float4(numer.x * r / (1.f + expf(-g.x)), numer.y * r / (1.f + expf(-g.y)), numer.z * r / (1.f + expf(-g.z)),
+                        numer.w * r / (1.f + expf(-g.w))));
+    return;
+  }
   if (sinks) {                                             // the sink joins the divisor once, here
     const float r = sink_reciprocal(denom, m, sinks[head]);
     st(to, numer.x * r); st(to + 1, numer.y * r); st(to + 2, numer.z * r); st(to + 3, numer.w * r);
@@ -341,7 +350,7 @@ static int launch_rows(const void* q, int q_stride, const void* k_cache, const v
   dim3 merge_grid;
   merge_shape(rows, heads, d, &tg, &merge_grid);
   hipLaunchKernelGGL(attn_rows_merge_kernel<T>, merge_grid, dim3(QIL_WAVE), 0, s, part_acc, part_m, part_l, positions,
-                     row_index, (T*)out, heads, d, window, P, parts, tg, sinks, keep);
+                     row_index, (T*)out, heads, d, window, P, parts, tg, sinks, keep, Operand{}, 0);
   return (int)hipGetLastError();
 }
 
@@ -406,9 +415,16 @@ int qil_attn_rows_unmerged(const void* q, int q_stride, const void* k_cache, con
 
 // Merge of partial results written by a partial kernel (this file's or the matrix-core decode kernel's).
 // sinks: null, or float32 [heads]: exp(sink) joins every head's divisor once.  keep: the kept first keys (key_span.h).
+// gate: null, or an operand of rows of gate_row elements (total_rows of them, split stride their product) whose first
+// heads * d columns are the logits of an output gate: a row's result is multiplied by their sigmoids before it is rounded.
 int qil_attn_merge(const void* workspace, const int* positions, const int* row_index, void* out, int rows, int heads,
-                   int d, int window, int P, int parts, int dtype, const float* sinks, int keep, hipStream_t s) {
+                   int d, int window, int P, int parts, int dtype, const float* sinks, int keep, const void* gate,
+                   int gate_code, int gate_splits, int gate_row, int total_rows, hipStream_t s) {
   if (rows == 0 || parts <= 1) return 0;
+  const Operand operand{gate, gate_code, gate_splits, (size_t)total_rows * gate_row};
+  if (gate && (gate_splits < 1 || (gate_code == QIL_BF16 && gate_splits != 1) || gate_row < heads * d || gate_row % 4 ||
+               ((uintptr_t)gate % 16)))
+    return -1;
   const float* acc = (const float*)workspace;
   const float* m = acc + (size_t)rows * heads * parts * d;
   const float* l = m + (size_t)rows * heads * parts;
@@ -419,10 +435,10 @@ int qil_attn_merge(const void* workspace, const int* positions, const int* row_i
   const dim3 block(QIL_WAVE);
   if (dtype == QIL_F32)
     hipLaunchKernelGGL(attn_rows_merge_kernel<float>, grid, block, 0, s, acc, m, l, positions, row_index, (float*)out,
-                       heads, d, window, P, parts, tg, sinks, keep);
+                       heads, d, window, P, parts, tg, sinks, keep, operand, gate_row);
   else
     hipLaunchKernelGGL(attn_rows_merge_kernel<bf16_t>, grid, block, 0, s, acc, m, l, positions, row_index, (bf16_t*)out,
-                       heads, d, window, P, parts, tg, sinks, keep);
+                       heads, d, window, P, parts, tg, sinks, keep, operand, gate_row);
   QIL_RETURN_LAUNCH_STATUS();
 }
 

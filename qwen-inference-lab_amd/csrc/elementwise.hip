@@ -49,6 +49,27 @@ __global__ void embed_pairs_kernel(const int* __restrict__ tokens, const int* __
   }
 }
 
+// The same for bfloat16 rows in whole pieces of eight elements, 16-byte aligned.
+__global__ void embed_pairs_bf16x8_kernel(const int* __restrict__ tokens, const int* __restrict__ previous,
+                                          const bf16_t* __restrict__ table, const bf16_t* __restrict__ pairs,
+                                          float* __restrict__ stream, float* __restrict__ copy, int width, float scale,
+                                          int buckets, long long mul_prev, long long mul_cur) {
+  const int n = blockIdx.x, token = tokens[n], before = previous[n];
+  const size_t row = before < 0 ? (size_t)buckets : (size_t)((before * mul_prev + token * mul_cur) % buckets);
+  const size_t at = (size_t)n * width;
+  for (int i = threadIdx.x * 8; i < width; i += blockDim.x * 8) {
+    float a[8], b[8];
+    ld8(table + (size_t)token * width + i, a);
+    ld8(pairs + row * width + i, b);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) a[e] = a[e] * scale + b[e];
+    const float4 lo = make_float4(a[0], a[1], a[2], a[3]), hi = make_float4(a[4], a[5], a[6], a[7]);
+    st4(stream + at + i, lo);
+    st4(stream + at + i + 4, hi);
+    if (copy) { st4(copy + at + i, lo); st4(copy + at + i + 4, hi); }
+  }
+}
+
 __device__ __forceinline__ float4 load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 __device__ __forceinline__ float4 load4(const bf16_t* p) {
   const uint2 raw = *reinterpret_cast<const uint2*>(p);
@@ -254,6 +275,9 @@ int qil_embed_pairs(const int* tokens, const int* previous, const void* table, c
   if (dtype == QIL_F32)
     hipLaunchKernelGGL(embed_pairs_kernel<float>, dim3(n), dim3(threads), 0, s, tokens, previous, (const float*)table,
                        (const float*)pairs, stream, copy, width, scale, buckets, mul_prev, mul_cur);
+  else if (width % 8 == 0 && (((uintptr_t)table | (uintptr_t)pairs | (uintptr_t)stream | (uintptr_t)copy) % 16) == 0)
+    hipLaunchKernelGGL(embed_pairs_bf16x8_kernel, dim3(n), dim3(width >= 2048 ? 256 : 64), 0, s, tokens, previous,
+                       (const bf16_t*)table, (const bf16_t*)pairs, stream, copy, width, scale, buckets, mul_prev, mul_cur);
   else
     hipLaunchKernelGGL(embed_pairs_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, tokens, previous, (const bf16_t*)table,
                        (const bf16_t*)pairs, stream, copy, width, scale, buckets, mul_prev, mul_cur);

@@ -83,6 +83,9 @@ OWN_LARGE_PRODUCTS = False
 WIDE_GEMM_FEWEST_ROWS = 512           # from here on the 256 x 256 block kernel, below the 32 x 32 tile kernel
 
 
+_NO_GATE = (None, 0, 1, 0, 0)         # the merge kernel's arguments for no output gate
+
+
 class UnsupportedShape(ValueError):
     pass
 
@@ -181,7 +184,7 @@ class Unmerged:
     def merge(self):
         _check(library.load().qil_attn_merge(_ptr(self.workspace), _ptr(self.positions), None, _ptr(self.out),
                                              self.shape[0], self.heads, self.head_dim, self.window, self.part,
-                                             self.parts, _code(self.dtype), None, 0, _stream()), 'attn_merge')
+                                             self.parts, _code(self.dtype), None, 0, *_NO_GATE, _stream()), 'attn_merge')
         return self.out
 
 
@@ -856,7 +859,7 @@ def decode_attention_takes(qkv, *, heads, kv_heads, head_dim, page_size, rotatio
 def decode_attention(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps, rotation, positions, writes, k_cache,
                      v_cache, page_size, block_tables, row_seq, max_context, scale, window, unmerged=False,
                      rotate_first=False, softcap=None, has_kv=True, extra_columns=0, bias=None, q_temperature=None, sinks=None,
-                     values_are_keys=False, slopes=None, keep_first=0):
+                     values_are_keys=False, slopes=None, keep_first=0, gate=None):
     """``qk_norm_rope_store`` and ``paged_attention`` in one kernel for a step whose rows are all alone in their
     sequences: queries, the new key and the new value are made from the partial sums ``qkv`` inside the
     attention kernel (bit for bit what the two kernels make), the new key and value are written into the
@@ -864,7 +867,8 @@ def decode_attention(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps,
     ``paged_attention``.  ``has_kv=False`` (with ``writes`` False): the rows of ``qkv`` hold queries only;
     ``extra_columns``, ``bias``, ``q_temperature`` as in ``qk_norm_rope_store``, ``sinks`` as in ``paged_attention``
     (a step with sinks comes back merged); ``values_are_keys`` as in ``qk_norm_rope_store``, ``slopes`` and
-    ``keep_first`` as in ``paged_attention``.  Returns what ``paged_attention`` returns."""
+    ``keep_first`` as in ``paged_attention``.  ``gate`` [N, heads * d] (a tensor, Partials or Columns): the result is
+    multiplied by its sigmoid (before the rounding, where parts are merged), and comes back merged.  Returns what ``paged_attention`` returns."""
     n = qkv.shape[0]
     dtype = torch.bfloat16
     stored = kv_heads if has_kv else 0
@@ -906,14 +910,16 @@ def decode_attention(qkv, *, heads, kv_heads, head_dim, q_weight, k_weight, eps,
                                      _ptr(bias), float(coef), int(every), _ptr(sinks), int(bool(values_are_keys)),
                                      _ptr(slopes), keep, _stream()), 'attn_decode_fused')
     if parts > 1:
-        if sinks is not None or keep:                   # the merge adds the sinks' term; its parts count places
+        if sinks is not None or keep or gate is not None:
+            # the merge adds the sinks' term and multiplies by the gate; its parts count places
+            columns_of_gate = _NO_GATE if gate is None else (*_row_operand(gate, 'gate', n, heads * head_dim), n)
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), None, _ptr(out), n, heads, head_dim, window_arg,
-                                      part, parts, _code(dtype), _ptr(sinks), keep, _stream()), 'attn_merge')
+                                      part, parts, _code(dtype), _ptr(sinks), keep, *columns_of_gate, _stream()), 'attn_merge')
             return out
         result = Unmerged(workspace, positions, out, heads=heads, head_dim=head_dim, window=window_arg, part=part,
                           parts=parts)
         return result if unmerged else result.merge()
-    return out
+    return out if gate is None else sigmoid_gate(out, gate, offset=0)
 
 
 TILE_KEY_PARTS = None   # tests: (keys per part, parts) forces the tile kernel's key split where it takes the sizes
@@ -1031,8 +1037,8 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
                                                   part, parts, _code(qkv.dtype), _ptr(slopes), _stream()),
                        'attn_tile_in_parts')
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), None, _ptr(out), merged, heads, head_dim,
-                                      int(window or 0), part, parts, _code(qkv.dtype), _ptr(sinks), 0, _stream()),
-                   'attn_merge')
+                                      int(window or 0), part, parts, _code(qkv.dtype), _ptr(sinks), 0, *_NO_GATE,
+                                      _stream()), 'attn_merge')
         else:
             _check(lib.qil_attn_tile(_ptr(qkv), qkv.shape[1], _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                      block_tables.shape[1], _ptr(cu_seqlens), _ptr(seq_starts), _ptr(out), n_seqs,
@@ -1059,8 +1065,8 @@ def paged_attention(q, *, heads, kv_heads, head_dim, k_cache, v_cache, page_size
                 return Unmerged(workspace, positions, out, heads=heads, head_dim=head_dim, window=window_arg,
                                 part=part, parts=parts)
             _check(lib.qil_attn_merge(_ptr(workspace), _ptr(positions), _ptr(single_rows), _ptr(out), rows, heads,
-                                      head_dim, window_arg, part, parts, _code(qkv.dtype), _ptr(sinks), keep, _stream()),
-                   'attn_merge')
+                                      head_dim, window_arg, part, parts, _code(qkv.dtype), _ptr(sinks), keep,
+                                      *_NO_GATE, _stream()), 'attn_merge')
         else:
             part = _rows_part(rows, kv_heads, places)
             parts = max(1, -(-places // part))

@@ -217,7 +217,7 @@ def _declare(lib):
     lib.qil_attn_rows_workspace.argtypes = [i, i, i, i]
     lib.qil_attn_rows_workspace.restype = z
     lib.qil_attn_rows.argtypes = [p, i, p, p, p, i, p, p, p, p, p, i, i, i, i, i, i, f, f, i, i, i, p, p, i, p]
-    lib.qil_attn_merge.argtypes = [p, p, p, p, i, i, i, i, i, i, i, p, i, p]
+    lib.qil_attn_merge.argtypes = [p, p, p, p, i, i, i, i, i, i, i, p, i, p, i, i, i, i, p]
     lib.qil_attn_decode_fused_takes.argtypes = [i, i, i, i, i]
     lib.qil_attn_decode_fused_takes.restype = i
     lib.qil_attn_decode_fused.argtypes = [p, i, p, p, f, p, p, i, i, p, p, p, i, p, p, p, p, i, i, i, i, i, i, f, i, i, i, i, i, f, i, i, p, f, i, p, i, p, i, p]

@@ -265,22 +265,23 @@ class Attention(Mixer):
                 page_size=cache.page_size, block_tables=cache.block_tables, row_seq=ctx.row_seq,
                 max_context=ctx.max_context, unmerged=False, rotate_first=self.norm_after_rotation, has_kv=self.own_kv,
                 extra_columns=gate_columns, bias=self.b_qkv_own, q_temperature=self.q_temperature,
-                values_are_keys=self.values_are_keys, **masks, **sizes, **norms)
+                values_are_keys=self.values_are_keys,
+                gate=ops.columns(qkv, own, gate_columns) if self.gate else None, **masks, **sizes, **norms)
+            return ops.linear(attended, p['o_proj.weight'], p.get('o_proj.bias'), partials=True)
+        store = dict(rotation=rotation, positions=ctx.positions, slots=cache.slots if cache.writes else None,
+                     k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size, dtype=self.dtype, heads=self.heads,
+                     kv_heads=stored, head_dim=self.padded_dim, extra_columns=gate_columns,
+                     values_are_keys=self.values_are_keys, **norms)
+        if rows:
+            q = ops.qk_row_norm_store(qkv, q_elems=self.heads * self.head_dim, k_elems=self.kv_heads * self.head_dim, **store)
         else:
-            store = dict(rotation=rotation, positions=ctx.positions, slots=cache.slots if cache.writes else None,
-                         k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size, dtype=self.dtype, heads=self.heads,
-                         kv_heads=stored, head_dim=self.padded_dim, extra_columns=gate_columns,
-                         values_are_keys=self.values_are_keys, **norms)
-            if rows:
-                q = ops.qk_row_norm_store(qkv, q_elems=self.heads * self.head_dim, k_elems=self.kv_heads * self.head_dim, **store)
-            else:
-                q = ops.qk_norm_rope_store(qkv, norm_dim=self.head_dim, rotate_first=self.norm_after_rotation,
-                                           q_temperature=self.q_temperature, bias=self.b_qkv_own, **store)
-            attended = ops.paged_attention(
-                q, k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size,
-                block_tables=cache.block_tables, row_seq=ctx.row_seq, positions=ctx.positions,
-                cu_seqlens=ctx.cu_seqlens, seq_starts=ctx.seq_starts, single_rows=ctx.single_rows, n_seqs=ctx.n_seqs,
-                max_query=ctx.max_query, max_context=ctx.max_context, tile_seqs=ctx.tile_seqs, unmerged=False, **masks, **sizes)
+            q = ops.qk_norm_rope_store(qkv, norm_dim=self.head_dim, rotate_first=self.norm_after_rotation,
+                                       q_temperature=self.q_temperature, bias=self.b_qkv_own, **store)
+        attended = ops.paged_attention(
+            q, k_cache=cache.k, v_cache=cache.v, page_size=cache.page_size,
+            block_tables=cache.block_tables, row_seq=ctx.row_seq, positions=ctx.positions,
+            cu_seqlens=ctx.cu_seqlens, seq_starts=ctx.seq_starts, single_rows=ctx.single_rows, n_seqs=ctx.n_seqs,
+            max_query=ctx.max_query, max_context=ctx.max_context, tile_seqs=ctx.tile_seqs, unmerged=False, **masks, **sizes)
         if self.gate:
             attended = ops.sigmoid_gate(attended, qkv, offset=own)
         return ops.linear(attended, p['o_proj.weight'], p.get('o_proj.bias'), partials=True)

@@ -181,6 +181,14 @@ def test_decoding_with_queries_made_inside_is_the_two_kernels(lengths, page_size
     torch.testing.assert_close(got, want, atol=0, rtol=0)
     same = lambda a, b: torch.equal(a.view(torch.int16), b.view(torch.int16))          # NaN-filled pages: compare the bits
     assert same(k_one, k_two) and same(v_one, v_two), 'the pages differ'
+    # with an output gate, from columns of the same product: the gate multiplies before the rounding
+    logits = ops.columns(wide, 8, heads * d) if extra else ops.Partials((torch.randn(2, rows, heads * d, generator=g)).cuda())
+    k_gated, v_gated = k_cache.clone(), v_cache.clone()
+    gated = ops.decode_attention(qkv, writes=True, k_cache=k_gated, v_cache=v_gated, block_tables=table, row_seq=row_seq,
+                                 max_context=max(lengths), gate=logits, **masks, **common)
+    source = logits.source.sum()[:, 8:8 + heads * d] if extra else logits.sum()
+    close(gated, want.float().cpu() * torch.sigmoid(source).cpu(), dtype, 0.3)
+    assert same(k_gated, k_two) and same(v_gated, v_two), 'the pages differ'
 
 
 # ------------------------------------------------------------------------------------------------ the recurrence
