@@ -321,6 +321,96 @@ qk_row_norm_store_kernel(const TD* __restrict__ qkv, int splits, size_t split_st
   }
 }
 
+// The same without a rotation, the row in registers: a block a row of queries (up to JQ chunks of 8 a thread), a wave a
+// row of keys (up to JK chunks a lane, four tokens a block), then the values as above.
+template <typename TD, typename T, int JQ, int JK>
+__global__ void __launch_bounds__(256)
+qk_row_norm_store_vec_kernel(const TD* __restrict__ qkv, int splits, size_t split_stride, T* __restrict__ q_out,
+                             const float* __restrict__ q_weight, const float* __restrict__ k_weight,
+                             const int* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache, int n, int heads,
+                             int kv_heads, int d, int page_size, float eps, float q_elems, float k_elems, int row_elems,
+                             int v_head, int k_blocks) {
+  __shared__ float scratch[16];
+  const int chunks = d / 8, lane = threadIdx.x & (QIL_WAVE - 1), wave_in_block = threadIdx.x / QIL_WAVE;
+  if ((int)blockIdx.x < n) {                             // queries
+    const int token = blockIdx.x, count = heads * chunks;
+    const size_t src = (size_t)token * row_elems;
+    float x[JQ][8], sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < JQ; ++j) {
+      const int c = min((int)threadIdx.x + j * 256, count - 1);
+      load8_sum(qkv, src + (size_t)c * 8, splits, split_stride, x[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < JQ; ++j)
+      if ((int)threadIdx.x + j * 256 < count) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += x[j][e] * x[j][e];
+      }
+    sum = block_sum(sum, scratch);
+    const float rstd = 1.f / sqrtf(sum / q_elems + eps);
+#pragma unroll
+    for (int j = 0; j < JQ; ++j) {
+      const int c = threadIdx.x + j * 256;
+      if (c < count) {
+        float w[8];
+        ld8(q_weight + (size_t)c * 8, w);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[j][e] = x[j][e] * rstd * w[e];
+        store8(q_out + (size_t)token * heads * d + (size_t)c * 8, x[j]);
+      }
+    }
+    return;
+  }
+  if ((int)blockIdx.x < n + k_blocks) {                  // keys
+    const int token = ((int)blockIdx.x - n) * 4 + wave_in_block, count = kv_heads * chunks;
+    if (token >= n) return;
+    const size_t src = (size_t)token * row_elems + (size_t)heads * d;
+    float x[JK][8], sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < JK; ++j) {
+      const int c = min(lane + j * QIL_WAVE, count - 1);
+      load8_sum(qkv, src + (size_t)c * 8, splits, split_stride, x[j]);
+    }
+    const int slot = slots[token];
+    const size_t page = slot / page_size, offset = slot % page_size;
+#pragma unroll
+    for (int j = 0; j < JK; ++j)
+      if (lane + j * QIL_WAVE < count) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += x[j][e] * x[j][e];
+      }
+    sum = wave_sum(sum);
+    const float rstd = 1.f / sqrtf(sum / k_elems + eps);
+#pragma unroll
+    for (int j = 0; j < JK; ++j) {
+      const int c = lane + j * QIL_WAVE;
+      if (c < count) {
+        float w[8];
+        ld8(k_weight + (size_t)c * 8, w);
+        const int head = c / chunks, e0 = (c - head * chunks) * 8;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[j][e] = x[j][e] * rstd * w[e];
+        store8(k_cache + ((page * kv_heads + head) * page_size + offset) * (size_t)d + e0, x[j]);
+      }
+    }
+    return;
+  }
+  const int quads = (chunks + 3) / 4;                    // values: copied, transposed within the page
+  const size_t wave = (size_t)((int)blockIdx.x - n - k_blocks) * 4 + wave_in_block;
+  const int quad = (int)(wave % quads), kvh = (int)(wave / quads % kv_heads);
+  const size_t token = wave / quads / kv_heads * 16 + (lane >> 2);
+  const int chunk = quad * 4 + (lane & 3);
+  if (token >= (size_t)n || chunk >= chunks) return;
+  float x[8];
+  load8_sum(qkv, token * row_elems + (size_t)(v_head + kvh) * d + chunk * 8, splits, split_stride, x);
+  const int slot = slots[token];
+  const size_t page = slot / page_size, offset = slot % page_size;
+  T* column = v_cache + ((page * kv_heads + kvh) * (size_t)d + chunk * 8) * page_size + offset;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) st(column + (size_t)e * page_size, x[e]);
+}
+
 // qkv, caches, slots, rotation, shared_kv, extra_columns: as in qil_qk_norm_rope_store (no bias, no temperature).
 // q_weight float32 [heads * d], k_weight float32 [kv_heads * d]; q_elems, k_elems: the numbers of elements the two means
 // run over (fewer than heads * d where the heads are padded with zeros).  d % 8 == 0 and 16-byte aligned rows.
@@ -342,6 +432,27 @@ extern "C" int qil_qk_row_norm_store(
   const size_t v_waves = slots ? (size_t)((n + 15) / 16) * kv_heads * ((d / 8 + 3) / 4) : 0;
   const dim3 grid((unsigned)(2 * (size_t)n + (v_waves + 3) / 4));
   const size_t stride = (size_t)n * row_elems;
+  const int q_chunks = heads * d / 8, k_chunks = kv_heads * d / 8;
+  if ((!cos_table || rot == 0) && q_chunks <= 1024 && k_chunks <= 256) {
+    const int k_blocks = slots ? (n + 3) / 4 : 0;
+    const dim3 blocks((unsigned)((size_t)n + k_blocks + (v_waves + 3) / 4));
+#define QIL_ROW_VEC(TD, T, JQ, JK)                                                                                    \
+  hipLaunchKernelGGL((qk_row_norm_store_vec_kernel<TD, T, JQ, JK>), blocks, dim3(256), 0, s, (const TD*)qkv, splits,   \
+                     stride, (T*)q_out, q_weight, k_weight, slots, (T*)k_cache, (T*)v_cache, n, heads, kv_heads, d,    \
+                     page_size, eps, (float)q_elems, (float)k_elems, row_elems, v_head, k_blocks)
+#define QIL_ROW_VEC_J(TD, T)                                                                                          \
+  do {                                                                                                                \
+    if (q_chunks <= 256 && k_chunks <= 64) QIL_ROW_VEC(TD, T, 1, 1);                                                   \
+    else if (q_chunks <= 512 && k_chunks <= 128) QIL_ROW_VEC(TD, T, 2, 2);                                             \
+    else QIL_ROW_VEC(TD, T, 4, 4);                                                                                     \
+  } while (0)
+    if (dtype == QIL_F32) QIL_ROW_VEC_J(float, float);
+    else if (in_dtype == QIL_F32) QIL_ROW_VEC_J(float, bf16_t);
+    else QIL_ROW_VEC_J(bf16_t, bf16_t);
+#undef QIL_ROW_VEC_J
+#undef QIL_ROW_VEC
+    QIL_RETURN_LAUNCH_STATUS();
+  }
 #define QIL_ROW_NORM(TD, T)                                                                                           \
   do {                                                                                                                \
     if (lds > 60 * 1024) {                                                                                            \

@@ -104,7 +104,8 @@ def rotation_of(rot):
 @pytest.mark.parametrize('dtype', DTYPES)
 @pytest.mark.parametrize('heads,kv_heads,d,true_d,rot,extra,splits,shared', [
     (4, 2, 64, 64, 32, 256, 0, False), (6, 3, 56, 50, 0, 0, 3, False), (16, 4, 128, 128, 128, 64, 5, True), (5, 5, 16, 11, 6, 80, 1, True),
-    (1, 1, 8, 8, 0, 0, 0, False), (32, 8, 256, 256, 0, 0, 2, False)])
+    (1, 1, 8, 8, 0, 0, 0, False), (32, 8, 256, 256, 0, 0, 2, False), (12, 3, 128, 128, 0, 40, 0, False), (32, 8, 128, 128, 0, 0, 0, False),
+    (40, 20, 128, 128, 0, 0, 2, False), (3, 3, 56, 56, 10, 0, 2, False)])
 def test_a_norm_over_whole_rows(dtype, heads, kv_heads, d, true_d, rot, extra, splits, shared):
     g = torch.Generator().manual_seed(heads * d)
     positions, slots, qkv, (kc, vc) = qk_inputs(37, 12, 8, heads, kv_heads, d, extra, splits, shared, dtype, g)
