@@ -6,6 +6,7 @@ from .gerivik import GerivikConfig
 from .zinesun import ZinesunConfig
 from .dogozen import DogozenConfig
 from .tinuzen import TinuzenConfig
+from .kebudra import KebudraConfig
 
 __all__ = ['ConfigError', 'read_config_json', 'Qwen3Config', 'FubapelConfig', 'GerivikConfig', 'ZinesunConfig', 'DogozenConfig',
-           'TinuzenConfig']
+           'TinuzenConfig', 'KebudraConfig']

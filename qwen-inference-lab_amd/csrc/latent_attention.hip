@@ -15,6 +15,7 @@
 // with W_uv,h, so it is applied here, to the weighted sum of latents.
 #include "common.h"
 #include "partials.h"
+#include "operand.h"
 
 // ---------------------------------------------------------------------------------------------------------------
 // Step 1 of the mixer, after the stacked down products x = [W_dq h ; W_dkv h] (q_rank + rank + rot columns):
@@ -28,11 +29,11 @@ __global__ void latent_prepare_kernel(const TD* __restrict__ x, int splits, size
                                       const float* __restrict__ wc, const float* __restrict__ freq,
                                       const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ cq_out,
                                       T* __restrict__ latent, T* __restrict__ rope, float* __restrict__ gate_out, int q_rank,
-                                      int rank, int rot, int gates, float eps, int held) {
+                                      int rank, int rot, int gates, float eps, int held, int x_row) {
   extern __shared__ float sums[];                     // [q_rank + rank + rot + gates] when `held`: the row, its partial sums added
   __shared__ float scratch[16];
   const int n = blockIdx.x, total = q_rank + rank + rot + gates;
-  const size_t at = (size_t)n * total;
+  const size_t at = (size_t)n * x_row;
   if (held) {                                         // every element is read from memory once, all reads side by side
     for (int i = threadIdx.x; i < total; i += blockDim.x) sums[i] = parts_sum(x, at + i, splits, split_stride);
     __syncthreads();
@@ -64,11 +65,13 @@ __global__ void latent_prepare_kernel(const TD* __restrict__ x, int splits, size
 
 // ---------------------------------------------------------------------------------------------------------------
 // A product per head: out[n, h, o] = sum_k W[h, k, o] x[n, h, k]   (W "k-major": the outputs of one k side by side).
+// With a gate (an operand of rows of g_row elements) the result is multiplied by sigmoid(gate[n, h * o_dim + o]).
 // x: row stride x_row, head stride x_head (elements); out likewise.  A block takes ROWS rows of one head and 256
 // outputs; x passes through LDS, every W element is read once a block.
 template <typename TX, typename TW, typename TO, int ROWS>
 __global__ void head_product_kernel(const TX* __restrict__ x, int x_row, int x_head, const TW* __restrict__ w,
-                                    TO* __restrict__ out, int out_row, int out_head, int n_rows, int k_dim, int o_dim) {
+                                    TO* __restrict__ out, int out_row, int out_head, int n_rows, int k_dim, int o_dim,
+                                    Operand gate, int g_row) {
   extern __shared__ float xs[];                       // [ROWS][k_dim]
   const int row0 = blockIdx.x * ROWS, h = blockIdx.y, o = blockIdx.z * blockDim.x + threadIdx.x;
   for (int idx = threadIdx.x; idx < ROWS * k_dim; idx += blockDim.x) {
@@ -88,7 +91,11 @@ __global__ void head_product_kernel(const TX* __restrict__ x, int x_row, int x_h
   }
 #pragma unroll
   for (int r = 0; r < ROWS; ++r)
-    if (row0 + r < n_rows) st(out + (size_t)(row0 + r) * out_row + (size_t)h * out_head + o, acc[r]);
+    if (row0 + r < n_rows) {
+      float v = acc[r];
+      if (gate.data) v /= 1.f + expf(-operand_at(gate, (size_t)(row0 + r) * g_row + (size_t)h * o_dim + o));
+      st(out + (size_t)(row0 + r) * out_row + (size_t)h * out_head + o, v);
+    }
 }
 
 // The same product for few rows (decoding): the weights of a head are then read by too few blocks for the chip, so a
@@ -98,7 +105,7 @@ __global__ void head_product_kernel(const TX* __restrict__ x, int x_row, int x_h
 template <typename TX, typename TW, typename TO, int OT>
 __global__ void __launch_bounds__(256)
 head_product_few_kernel(const TX* __restrict__ x, int x_row, int x_head, const TW* __restrict__ w, TO* __restrict__ out,
-                        int out_row, int out_head, int n_rows, int k_dim, int o_dim) {
+                        int out_row, int out_head, int n_rows, int k_dim, int o_dim, Operand gate, int g_row) {
   constexpr int OB = OT * 8, KG = 256 / OT;           // outputs a block, k groups
   extern __shared__ float xs[];                       // [8][k_dim], then [4 waves][8 rows][OB outputs]
   float* sums = xs + 8 * k_dim;
@@ -144,9 +151,31 @@ head_product_few_kernel(const TX* __restrict__ x, int x_row, int x_head, const T
   __syncthreads();
   for (int idx = tid; idx < 8 * OB; idx += 256) {
     const int r = idx / OB, j = idx % OB, o = blockIdx.z * OB + j;
-    if (row0 + r < n_rows && o < o_dim)
-      st(out + (size_t)(row0 + r) * out_row + (size_t)h * out_head + o,
-         sums[r * OB + j] + sums[(8 + r) * OB + j] + sums[(16 + r) * OB + j] + sums[(24 + r) * OB + j]);
+    if (row0 + r < n_rows && o < o_dim) {
+      float v = sums[r * OB + j] + sums[(8 + r) * OB + j] + sums[(16 + r) * OB + j] + sums[(24 + r) * OB + j];
+      if (gate.data) v /= 1.f + expf(-operand_at(gate, (size_t)(row0 + r) * g_row + (size_t)h * o_dim + o));
+      st(out + (size_t)(row0 + r) * out_row + (size_t)h * out_head + o, v);
+    }
+  }
+}
+
+// out[n, h * o_dim + o] = x[h, n, o] * sigmoid(gate[n, h * o_dim + o]): the batches of a product per head turned back into
+// rows, with the gate.  V neighbouring elements a thread.
+template <int V>
+__global__ void gated_heads_kernel(const bf16_t* __restrict__ x, Operand gate, int g_row, bf16_t* __restrict__ out, int n_rows,
+                                   int columns, int o_dim, size_t items) {
+  const size_t item = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (item >= items) return;
+  const int per_row = columns / V;
+  const size_t n = item / per_row;
+  const int c = (int)(item - n * per_row) * V, h = c / o_dim;
+  const bf16_t* from = x + ((size_t)h * n_rows + n) * o_dim + (c - h * o_dim);
+  if constexpr (V == 4) {
+    const float4 v = ld4(from), g = operand_at4(gate, n * g_row + c);
+    st4(out + n * columns + c, make_float4(v.x / (1.f + expf(-g.x)), v.y / (1.f + expf(-g.y)), v.z / (1.f + expf(-g.z)),
+                                           v.w / (1.f + expf(-g.w))));
+  } else {
+    st(out + n * columns + c, ld(from) / (1.f + expf(-operand_at(gate, n * g_row + c))));
   }
 }
 
@@ -282,14 +311,15 @@ static void latent_plan(int heads, int rank, int rot, int* group, int* kt, size_
 
 extern "C" {
 
-int qil_latent_prepare(const void* x, int x_dtype, int splits, const float* wq, const float* wc, const float* freq,
+// x: rows of x_row elements (split stride n * x_row), the first q_rank + rank + rot + gates of them meant.
+int qil_latent_prepare(const void* x, int x_dtype, int splits, int x_row, const float* wq, const float* wc, const float* freq,
                        const int* positions, const int* slots, void* cq_out, void* latent, void* rope, float* gate_out,
                        int n, int q_rank, int rank, int rot, int gates, float eps, int dtype, hipStream_t s) {
   if (n == 0) return 0;
   if (q_rank < 1 || rank < 1 || rot < 2 || rot % 2 || splits < 1 || (x_dtype == QIL_BF16 && splits != 1) || gates < 0 ||
-      (gates > 0 && !gate_out))
+      (gates > 0 && !gate_out) || x_row < q_rank + rank + rot + gates)
     return -1;
-  const size_t stride = (size_t)n * (q_rank + rank + rot + gates);
+  const size_t stride = (size_t)n * x_row;
   const size_t row_bytes = (size_t)(q_rank + rank + rot + gates) * sizeof(float);
   const int held = row_bytes <= 48 * 1024;            // the row's sums fit in LDS
   // a thread's loads of the row come one after the other: with few rows (too few blocks to hide that) wide rows get
@@ -297,7 +327,7 @@ int qil_latent_prepare(const void* x, int x_dtype, int splits, const float* wq, 
   const int total = q_rank + rank + rot + gates, threads = n > 64 ? 256 : total >= 2048 ? 1024 : total >= 1024 ? 512 : 256;
 #define QIL_LP(TD, T)                                                                                               \
   hipLaunchKernelGGL((latent_prepare_kernel<TD, T>), dim3(n), dim3(threads), held ? row_bytes : 0, s, (const TD*)x, splits, \
-                     stride, wq, wc, freq, positions, slots, (T*)cq_out, (T*)latent, (T*)rope, gate_out, q_rank, rank, rot, gates, eps, held)
+                     stride, wq, wc, freq, positions, slots, (T*)cq_out, (T*)latent, (T*)rope, gate_out, q_rank, rank, rot, gates, eps, held, x_row)
   if (dtype == QIL_F32) {
     if (x_dtype != QIL_F32) return -1;
     QIL_LP(float, float);
@@ -313,9 +343,12 @@ int qil_latent_prepare(const void* x, int x_dtype, int splits, const float* wq, 
 // out[n, h, o] = sum_k w[h, k, o] x[n, h, k]; x_dtype / w_dtype / out_dtype element codes; strides in elements.
 // Combinations: all float32; x bfloat16, w bfloat16, out float32; x float32, w bfloat16, out bfloat16.
 int qil_head_product(const void* x, int x_dtype, int x_row, int x_head, const void* w, int w_dtype, void* out,
-                     int out_dtype, int out_row, int out_head, int n, int heads, int k_dim, int o_dim, hipStream_t s) {
+                     int out_dtype, int out_row, int out_head, int n, int heads, int k_dim, int o_dim, const void* gate,
+                     int gate_code, int gate_splits, int gate_row, hipStream_t s) {
   if (n == 0 || heads == 0 || o_dim == 0) return 0;
-  if (k_dim < 1) return -1;
+  if (k_dim < 1 || (gate && (gate_splits < 1 || (gate_code == QIL_BF16 && gate_splits != 1) || gate_row < heads * o_dim)))
+    return -1;
+  const Operand g{gate, gate_code, gate_splits, (size_t)n * gate_row};
   const int rows = 8;
   const size_t lds = (size_t)rows * k_dim * sizeof(float);
   if (lds > 64 * 1024) return -1;
@@ -330,19 +363,39 @@ int qil_head_product(const void* x, int x_dtype, int x_row, int x_head, const vo
   do {                                                                                                                  \
     if (few && narrow)                                                                                                  \
       hipLaunchKernelGGL((head_product_few_kernel<TX, TW, TO, 4>), grid_narrow, dim3(256), lds + 4 * 8 * 32 * sizeof(float), s, \
-                         (const TX*)x, x_row, x_head, (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim);       \
+                         (const TX*)x, x_row, x_head, (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim, g, gate_row);       \
     else if (few)                                                                                                       \
       hipLaunchKernelGGL((head_product_few_kernel<TX, TW, TO, 8>), grid_few, dim3(256), lds + 4 * 8 * 64 * sizeof(float), s, \
-                         (const TX*)x, x_row, x_head, (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim);       \
+                         (const TX*)x, x_row, x_head, (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim, g, gate_row);       \
     else                                                                                                                \
       hipLaunchKernelGGL((head_product_kernel<TX, TW, TO, 8>), grid, dim3(threads), lds, s, (const TX*)x, x_row, x_head, \
-                         (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim);                                    \
+                         (const TW*)w, (TO*)out, out_row, out_head, n, k_dim, o_dim, g, gate_row);                                    \
   } while (0)
   if (x_dtype == QIL_F32 && w_dtype == QIL_F32 && out_dtype == QIL_F32) QIL_HP(float, float, float);
   else if (x_dtype == QIL_BF16 && w_dtype == QIL_BF16 && out_dtype == QIL_F32) QIL_HP(bf16_t, bf16_t, float);
   else if (x_dtype == QIL_F32 && w_dtype == QIL_BF16 && out_dtype == QIL_BF16) QIL_HP(float, bf16_t, bf16_t);
   else return -1;
 #undef QIL_HP
+  QIL_RETURN_LAUNCH_STATUS();
+}
+
+// x bfloat16 [heads, n, o_dim] -> out bfloat16 [n, heads * o_dim], times the sigmoid of the gate's logits (an operand of rows of
+// gate_row elements).
+int qil_gated_heads(const void* x, const void* gate, int gate_code, int gate_splits, int gate_row, void* out, int n, int heads,
+                    int o_dim, hipStream_t s) {
+  if (n == 0 || heads == 0 || o_dim == 0) return 0;
+  if (!gate || gate_splits < 1 || (gate_code == QIL_BF16 && gate_splits != 1) || gate_row < heads * o_dim) return -1;
+  const Operand g{gate, gate_code, gate_splits, (size_t)n * gate_row};
+  const int columns = heads * o_dim;
+  const bool vec = o_dim % 4 == 0 && gate_row % 4 == 0 && (((uintptr_t)x | (uintptr_t)gate | (uintptr_t)out) % 16) == 0;
+  const size_t items = (size_t)n * columns / (vec ? 4 : 1);
+  const dim3 grid((unsigned)((items + 255) / 256));
+  if (vec)
+    hipLaunchKernelGGL(gated_heads_kernel<4>, grid, dim3(256), 0, s, (const bf16_t*)x, g, gate_row, (bf16_t*)out, n, columns,
+                       o_dim, items);
+  else
+    hipLaunchKernelGGL(gated_heads_kernel<1>, grid, dim3(256), 0, s, (const bf16_t*)x, g, gate_row, (bf16_t*)out, n, columns,
+                       o_dim, items);
   QIL_RETURN_LAUNCH_STATUS();
 }
 

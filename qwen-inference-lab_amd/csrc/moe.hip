@@ -11,7 +11,8 @@
 //            cut into tiles of TM pairs: tile -> (expert, first place, pairs), a fixed number of tiles of which the
 //            unused ones hold no pair.  One block; the order inside an expert's run is whatever the atomics give,
 //            which no result depends on (every pair's row is a product of its own).
-//   gate_up  hidden[place] = act(W_gate,e h, W_up,e h) for the pairs of a tile, one wave per 16 hidden columns
+//   gate_up  hidden[place] = act(W_gate,e h, W_up,e h) for the pairs of a tile, one wave per 16 hidden columns; or, for
+//            experts without a gate branch, hidden[place] = act(W_up,e h), one wave per 32
 //   down     y[pair] = W_down,e hidden[place], float32
 //   combine  out[token] = sum over the token's slots, in slot order, of weight * (y[pair], or h for an identity expert)
 //
@@ -309,10 +310,12 @@ moe_gate_up_kernel(const T* __restrict__ x, int width, const T* __restrict__ w, 
 
 // grid (tiles, ceil(width / 128)); a wave: the tile's rows by 32 output columns.  w: [experts][width][ff].
 // y: [pairs][width] float32, a pair's row at the pair's own index.
-template <typename T, int MT, bool ALIGNED>
+// UP: the first product of experts without a gate branch: `hidden` are the rows of x (by the pair's token, of which there
+// are `top` pairs), ff their length, width the experts' inner size, and act(result) goes to the places' rows of `to`.
+template <typename T, int MT, bool ALIGNED, bool UP>
 __global__ void __launch_bounds__(256)
 moe_down_kernel(const T* __restrict__ hidden, int ff, const T* __restrict__ w, int width, const int* __restrict__ tiles,
-                int max_tiles, const int* __restrict__ places, float* __restrict__ y) {
+                int max_tiles, const int* __restrict__ places, float* __restrict__ y, T* __restrict__ to, int top, int act) {
   constexpr int EPL = Frag<T>::EPL, KC = 4 * EPL;
   const int tile = blockIdx.x, rows = tiles[2 * max_tiles + tile];
   if (rows == 0) return;
@@ -323,7 +326,10 @@ moe_down_kernel(const T* __restrict__ hidden, int ff, const T* __restrict__ w, i
   const int r = lane & 15, kq = lane >> 4;
   const T* a_row[MT];
 #pragma unroll
-  for (int m = 0; m < MT; ++m) a_row[m] = hidden + (size_t)(begin + min(m * 16 + r, rows - 1)) * ff;
+  for (int m = 0; m < MT; ++m) {
+    const int place = begin + min(m * 16 + r, rows - 1);
+    a_row[m] = hidden + (size_t)(UP ? places[place] / top : place) * ff;
+  }
   const T* b_row[2];
 #pragma unroll
   for (int t = 0; t < 2; ++t) b_row[t] = w + ((size_t)e * width + min(col0 + t * 16 + r, width - 1)) * ff;
@@ -356,10 +362,17 @@ moe_down_kernel(const T* __restrict__ hidden, int ff, const T* __restrict__ w, i
     for (int i = 0; i < 4; ++i) {
       const int local = m * 16 + 4 * kq + i;
       if (local >= rows) continue;
-      float* out = y + (size_t)places[begin + local] * width;
+      if constexpr (UP) {
+        T* out = to + (size_t)(begin + local) * width;
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
-        if (col0 + t * 16 + r < width) out[col0 + t * 16 + r] = acc[m][t][i];
+        for (int t = 0; t < 2; ++t)
+          if (col0 + t * 16 + r < width) st(out + col0 + t * 16 + r, ungated_act(acc[m][t][i], act));
+      } else {
+        float* out = y + (size_t)places[begin + local] * width;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+          if (col0 + t * 16 + r < width) out[col0 + t * 16 + r] = acc[m][t][i];
+      }
     }
 }
 
@@ -371,17 +384,21 @@ moe_down_kernel(const T* __restrict__ hidden, int ff, const T* __restrict__ w, i
 // (rows 144 bytes apart, so that the 16 rows of a fragment read fall on all banks) and the waves read their fragments
 // from there: a weight is read from memory once a block, a pair's row once a block.
 // GATED: A rows are the pairs' rows of x, the result columns are 128 gate columns and the same 128 up columns of the
-// expert (a wave owns 32 of each), and the block writes act(gate, up) for 128 hidden columns.  Otherwise A rows are the
-// places' rows of hidden, the result columns are 256 of the expert's down matrix, written to the pairs' rows of y.
+// expert (a wave owns 32 of each), and the block writes act(gate, up) for 128 hidden columns.  DOWN: A rows are the
+// places' rows of hidden, the result columns are 256 of the expert's down matrix, written to the pairs' rows of y.  UP:
+// the first product of experts without a gate branch, A rows as for GATED, 256 columns of the expert's up matrix, and
+// act(result) goes to hidden.
 #define MOE_TILE_ROW 144                                  // bytes of a staged row: 128 and 16 to spread the banks
 #define MOE_TILE_LDS ((64 + 256) * MOE_TILE_ROW)
 #define MOE_TILE_THREADS 512
 struct MoeFetched { qil_u32x4 a, b[4]; };                 // a thread's pieces of one stage: one of A, four of B
-template <bool GATED>
+enum { MOE_DOWN = 0, MOE_GATED = 1, MOE_UP = 2 };
+template <int MODE>
 __global__ void __launch_bounds__(MOE_TILE_THREADS, 2)
 moe_tile_kernel(const bf16_t* __restrict__ a_base, const bf16_t* __restrict__ w, int K, int columns,
                 const int* __restrict__ tiles, int max_tiles, const int* __restrict__ places, int top,
                 bf16_t* __restrict__ hidden, float* __restrict__ y, int act, float limit, float alpha, int column_blocks) {
+  constexpr bool GATED = MODE == MOE_GATED;
   extern __shared__ __align__(16) unsigned char tile_lds[];
   unsigned char* a_lds = tile_lds;
   unsigned char* b_lds = tile_lds + 64 * MOE_TILE_ROW;
@@ -403,7 +420,7 @@ moe_tile_kernel(const bf16_t* __restrict__ a_base, const bf16_t* __restrict__ w,
   // what this thread fetches of a stage: piece tid % 8 of row tid / 8 of A and of the rows tid / 8 + 64 j of B
   const int piece = tid & 7, row0 = tid >> 3;
   const int local0 = min(row0, rows - 1);
-  const bf16_t* a_src = GATED ? a_base + (size_t)(places[begin + local0] / top) * K : a_base + (size_t)(begin + local0) * K;
+  const bf16_t* a_src = MODE != MOE_DOWN ? a_base + (size_t)(places[begin + local0] / top) * K : a_base + (size_t)(begin + local0) * K;
   const bf16_t* b_src[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
@@ -479,6 +496,12 @@ moe_tile_kernel(const bf16_t* __restrict__ a_base, const bf16_t* __restrict__ w,
           const int col = c0 + quarter * 32 + t * 16 + r;
           if (col < columns) st(hidden + (size_t)(begin + local) * columns + col, gated_act(acc[m][t][i], acc[m][2 + t][i], act, limit, alpha));
         }
+      } else if (MODE == MOE_UP) {
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+          const int col = c0 + quarter * 64 + t * 16 + r;
+          if (col < columns) st(hidden + (size_t)(begin + local) * columns + col, ungated_act(acc[m][t][i], act));
+        }
       } else {
         float* out = y + (size_t)places[begin + local] * columns;
 #pragma unroll
@@ -550,13 +573,15 @@ int qil_moe_max_tiles(int pairs, int experts, int tile_rows) { return (pairs + t
 // The experts' work on the routed pairs: x [n, width], chosen/weights [n, top]; w_gate_up [experts][2][ff][width],
 // w_down [experts][width][ff] (dtype); scratch: tiles int32 [3 * max_tiles], places int32 [n * top], hidden (dtype)
 // [n * top, ff], y float32 [n * top, width].  out float32 [n, width], or null: the pairs' rows stay in y for a consumer
-// that makes the weighted sum itself.
+// that makes the weighted sum itself.  act from QIL_ACT_RELU_SQUARED on: the experts have no gate branch, w_gate_up is
+// [experts][ff][width].
 int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* weights, const void* w_gate_up,
                     const void* w_down, int* tiles, int* places, void* hidden, float* y, float* out, int n, int width,
                     int ff, int experts, int top, int tile_rows, int max_tiles, int act, float limit, float alpha,
                     hipStream_t s) {
   if (n == 0) return 0;
   const int pairs = n * top;
+  const bool gated = act < QIL_ACT_RELU_SQUARED;
   if (experts > MOE_MAX_OUTPUTS || (tile_rows != 16 && tile_rows != 64) ||
       max_tiles < qil_moe_max_tiles(pairs, experts, tile_rows) || width < 1 || ff < 1)
     return -1;
@@ -566,29 +591,42 @@ int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* we
     const int epl = dtype == QIL_F32 ? 4 : 8;
     const bool aligned = width % epl == 0 && ff % epl == 0 &&
                          (((uintptr_t)x | (uintptr_t)w_gate_up | (uintptr_t)w_down | (uintptr_t)hidden) % 16) == 0;
-    const dim3 g_up(max_tiles, (ff + 63) / 64), g_down(max_tiles, (width + 127) / 128);
+    const dim3 g_up(max_tiles, gated ? (ff + 63) / 64 : (ff + 127) / 128), g_down(max_tiles, (width + 127) / 128);
     if (dtype == QIL_BF16 && tile_rows == 64 && aligned && width % 8 == 0 && ff % 8 == 0) {
-      static bool granted = false;                        // (both instantiations, once)
+      static bool granted = false;                        // (all instantiations, once)
       if (!granted) {
-        hipError_t a = hipFuncSetAttribute((const void*)moe_tile_kernel<true>, hipFuncAttributeMaxDynamicSharedMemorySize, MOE_TILE_LDS);
-        hipError_t b = hipFuncSetAttribute((const void*)moe_tile_kernel<false>, hipFuncAttributeMaxDynamicSharedMemorySize, MOE_TILE_LDS);
-        if (a != hipSuccess || b != hipSuccess) return (int)(a != hipSuccess ? a : b);
+        const void* kernels[3] = {(const void*)moe_tile_kernel<MOE_GATED>, (const void*)moe_tile_kernel<MOE_UP>,
+                                  (const void*)moe_tile_kernel<MOE_DOWN>};
+        for (const void* kernel : kernels) {
+          hipError_t error = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, MOE_TILE_LDS);
+          if (error != hipSuccess) return (int)error;
+        }
         granted = true;
       }
-      const int up_blocks = (ff + 127) / 128, down_blocks = (width + 255) / 256;
-      hipLaunchKernelGGL(moe_tile_kernel<true>, dim3(((size_t)max_tiles * up_blocks + 7) / 8 * 8), dim3(MOE_TILE_THREADS),
-                         MOE_TILE_LDS, s, (const bf16_t*)x, (const bf16_t*)w_gate_up, width, ff, tiles, max_tiles, places,
-                         top, (bf16_t*)hidden, (float*)nullptr, act, limit, alpha, up_blocks);
-      hipLaunchKernelGGL(moe_tile_kernel<false>, dim3(((size_t)max_tiles * down_blocks + 7) / 8 * 8), dim3(MOE_TILE_THREADS),
+      const int up_blocks = gated ? (ff + 127) / 128 : (ff + 255) / 256, down_blocks = (width + 255) / 256;
+      const dim3 up_grid(((size_t)max_tiles * up_blocks + 7) / 8 * 8);
+      if (gated)
+        hipLaunchKernelGGL(moe_tile_kernel<MOE_GATED>, up_grid, dim3(MOE_TILE_THREADS), MOE_TILE_LDS, s, (const bf16_t*)x,
+                           (const bf16_t*)w_gate_up, width, ff, tiles, max_tiles, places, top, (bf16_t*)hidden,
+                           (float*)nullptr, act, limit, alpha, up_blocks);
+      else
+        hipLaunchKernelGGL(moe_tile_kernel<MOE_UP>, up_grid, dim3(MOE_TILE_THREADS), MOE_TILE_LDS, s, (const bf16_t*)x,
+                           (const bf16_t*)w_gate_up, width, ff, tiles, max_tiles, places, top, (bf16_t*)hidden,
+                           (float*)nullptr, act, limit, alpha, up_blocks);
+      hipLaunchKernelGGL(moe_tile_kernel<MOE_DOWN>, dim3(((size_t)max_tiles * down_blocks + 7) / 8 * 8), dim3(MOE_TILE_THREADS),
                          MOE_TILE_LDS, s, (const bf16_t*)hidden, (const bf16_t*)w_down, ff, width, tiles, max_tiles, places,
                          top, (bf16_t*)nullptr, y, act, limit, alpha, down_blocks);
     } else {
 #define QIL_MOE(T, MT, ALIGNED)                                                                                       \
   do {                                                                                                                \
-    hipLaunchKernelGGL((moe_gate_up_kernel<T, MT, ALIGNED>), g_up, dim3(256), 0, s, (const T*)x, width,                \
-                       (const T*)w_gate_up, ff, tiles, max_tiles, places, top, (T*)hidden, act, limit, alpha);         \
-    hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED>), g_down, dim3(256), 0, s, (const T*)hidden, ff,               \
-                       (const T*)w_down, width, tiles, max_tiles, places, y);                                          \
+    if (gated)                                                                                                        \
+      hipLaunchKernelGGL((moe_gate_up_kernel<T, MT, ALIGNED>), g_up, dim3(256), 0, s, (const T*)x, width,              \
+                         (const T*)w_gate_up, ff, tiles, max_tiles, places, top, (T*)hidden, act, limit, alpha);       \
+    else                                                                                                              \
+      hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, true>), g_up, dim3(256), 0, s, (const T*)x, width,           \
+                         (const T*)w_gate_up, ff, tiles, max_tiles, places, (float*)nullptr, (T*)hidden, top, act);    \
+    hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, false>), g_down, dim3(256), 0, s, (const T*)hidden, ff,        \
+                       (const T*)w_down, width, tiles, max_tiles, places, y, (T*)nullptr, top, act);                   \
   } while (0)
 #define QIL_MOE_T(T)                                                                                                  \
   do {                                                                                                                \

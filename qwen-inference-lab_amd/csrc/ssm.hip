@@ -7,7 +7,8 @@
 //    position (cached length) - (taps - 1) + k, float32.  grid (rows, pieces of the channels); the thread of a
 //    sequence's first row computes its first taps - 1 rows and then writes the state's new contents for its channel
 //    (ascending: entry k takes what entry k + rows held, or a row of this step), so every read of a state element
-//    comes before its write; the threads of rows 1 .. taps - 2 leave at once.
+//    comes before its write; the threads of rows 1 .. taps - 2 leave at once.  Other columns of the same rows may be passed
+//    on as they are (their partial sums added, rounded once) to a second array, which a product can then read.
 //
 // 2. The scan, a sequence's rows in order:
 //      dt = softplus(dt_raw[t, c] + dt_bias[c])
@@ -38,9 +39,14 @@ template <typename T>
 __global__ void channel_conv_kernel(Operand x, int x_columns, const float* __restrict__ w, const float* __restrict__ bias,
                                     float* state, const int* __restrict__ cu_seqlens, const int* __restrict__ seq_starts,
                                     const int* __restrict__ seq_slots, const int* __restrict__ row_seq,
-                                    T* __restrict__ out, int channels, int taps, int act) {
+                                    T* __restrict__ out, int channels, int taps, int act, int pass_from, int passed,
+                                    T* __restrict__ passed_out) {
   const int c = blockIdx.y * blockDim.x + threadIdx.x, n = blockIdx.x;
-  if (c >= channels) return;
+  if (c >= channels) {
+    const int i = c - channels;
+    if (i < passed) st(passed_out + (size_t)n * passed + i, operand_at(x, (size_t)n * x_columns + pass_from + i));
+    return;
+  }
   const int keep = taps - 1;
   const int s = row_seq[n], row0 = cu_seqlens[s], t = n - row0;
   if (t > 0 && t < keep) return;                       // computed with the sequence's first row
@@ -106,9 +112,18 @@ __global__ void channel_conv_vec_kernel(const TI* __restrict__ x, int splits, si
                                         const float* __restrict__ w, const float* __restrict__ bias, float* state,
                                         const int* __restrict__ cu_seqlens, const int* __restrict__ seq_starts,
                                         const int* __restrict__ seq_slots, const int* __restrict__ row_seq,
-                                        T* __restrict__ out, int channels, int taps, int act) {
+                                        T* __restrict__ out, int channels, int taps, int act, int pass_from, int passed,
+                                        T* __restrict__ passed_out) {
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V, n = blockIdx.x;
-  if (c >= channels) return;
+  if (c >= channels) {
+    const int i = c - channels;
+    if (i < passed) {
+      float v[V];
+      conv_in<TI, V>::load(x, (size_t)n * x_columns + pass_from + i, splits, split_stride, v);
+      store_floats<V>(passed_out + (size_t)n * passed + i, v);
+    }
+    return;
+  }
   const int keep = taps - 1;
   const int s = row_seq[n], row0 = cu_seqlens[s], t = n - row0;
   if (t > 0 && t < keep) return;                       // computed with the sequence's first row
@@ -362,41 +377,47 @@ int qil_selective_scan_takes(int channels, int states, int taps) {
 
 // x: [n, x_columns] (x_code QIL_F32 with x_splits partial sums, or QIL_BF16), its first `channels` columns are the
 // convolution's input; w float32 [taps, channels]; bias float32 [channels] or null; state float32 [slots][taps - 1]
-// [channels] (null only for one tap); out [n, channels] of out_dtype; act: 0 none, 1 silu.
+// [channels] (null only for one tap); out [n, channels] of out_dtype; act: 0 none, 1 silu.  passed > 0: the columns
+// [pass_from, pass_from + passed) go to passed_out [n, passed] of out_dtype.
 int qil_channel_conv(const void* x, int x_code, int x_splits, int x_columns, const float* w, const float* bias, float* state,
                      const int* cu_seqlens, const int* seq_starts, const int* seq_slots, const int* row_seq, void* out,
-                     int out_dtype, int n, int channels, int taps, int act, hipStream_t s) {
+                     int out_dtype, int n, int channels, int taps, int act, int pass_from, int passed, void* passed_out,
+                     hipStream_t s) {
   if (n == 0) return 0;
+  if (passed < 0 || (passed && (!passed_out || pass_from < 0 || pass_from + passed > x_columns))) return -1;
   if (channels < 1 || channels > x_columns || taps < 1 || (taps > 1 && !state) || x_splits < 1 ||
       (x_code == QIL_BF16 && x_splits != 1)) return -1;
   const int V = x_code == QIL_BF16 ? 8 : 4;
-  if (channels % V == 0 && x_columns % V == 0 &&
+  if (channels % V == 0 && x_columns % V == 0 && pass_from % V == 0 && passed % V == 0 && ((uintptr_t)passed_out % 16) == 0 &&
       (((uintptr_t)x | (uintptr_t)w | (uintptr_t)bias | (uintptr_t)state | (uintptr_t)out) % 16) == 0 &&
       !(x_code == QIL_BF16 && out_dtype == QIL_F32)) {
-    const int lanes = channels / V;
+    const int lanes = (channels + passed) / V;
     const int threads = lanes >= 128 ? 128 : (lanes + 63) / 64 * 64;
     const dim3 grid(n, (lanes + threads - 1) / threads);
     const size_t stride = (size_t)n * x_columns;
     if (x_code == QIL_BF16)
       hipLaunchKernelGGL((channel_conv_vec_kernel<bf16_t, bf16_t, 8>), grid, dim3(threads), 0, s, (const bf16_t*)x, 1, stride,
-                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act);
+                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act, pass_from, passed,
+                         (bf16_t*)passed_out);
     else if (out_dtype == QIL_F32)
       hipLaunchKernelGGL((channel_conv_vec_kernel<float, float, 4>), grid, dim3(threads), 0, s, (const float*)x, x_splits, stride,
-                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (float*)out, channels, taps, act);
+                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (float*)out, channels, taps, act, pass_from, passed,
+                         (float*)passed_out);
     else
       hipLaunchKernelGGL((channel_conv_vec_kernel<float, bf16_t, 4>), grid, dim3(threads), 0, s, (const float*)x, x_splits, stride,
-                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act);
+                         x_columns, w, bias, state, cu_seqlens, seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act, pass_from, passed,
+                         (bf16_t*)passed_out);
     QIL_RETURN_LAUNCH_STATUS();
   }
   const Operand in{x, x_code, x_splits, (size_t)n * x_columns};
-  const int threads = channels >= 256 ? 256 : (channels + 63) / 64 * 64;
-  const dim3 grid(n, (channels + threads - 1) / threads);
+  const int lanes = channels + passed, threads = lanes >= 256 ? 256 : (lanes + 63) / 64 * 64;
+  const dim3 grid(n, (lanes + threads - 1) / threads);
   if (out_dtype == QIL_F32)
     hipLaunchKernelGGL(channel_conv_kernel<float>, grid, dim3(threads), 0, s, in, x_columns, w, bias, state, cu_seqlens,
-                       seq_starts, seq_slots, row_seq, (float*)out, channels, taps, act);
+                       seq_starts, seq_slots, row_seq, (float*)out, channels, taps, act, pass_from, passed, (float*)passed_out);
   else
     hipLaunchKernelGGL(channel_conv_kernel<bf16_t>, grid, dim3(threads), 0, s, in, x_columns, w, bias, state, cu_seqlens,
-                       seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act);
+                       seq_starts, seq_slots, row_seq, (bf16_t*)out, channels, taps, act, pass_from, passed, (bf16_t*)passed_out);
   QIL_RETURN_LAUNCH_STATUS();
 }
 

@@ -5,3 +5,4 @@ from . import gerivik  # noqa: F401
 from . import zinesun  # noqa: F401
 from . import dogozen  # noqa: F401
 from . import tinuzen  # noqa: F401
+from . import kebudra  # noqa: F401

@@ -244,6 +244,16 @@ class PostNormed:
         self.shape, self.device = tuple(value.shape), value.device
 
 
+class StreamUpdate:
+    """A sub-layer's output that joins several residual streams, not added yet: x_t <- sum_s mix[s, t] x_s + out[t] value, all
+    t at once.  ``value``: a tensor of the model's type, float32, ``Partials`` or ``RoutedSum``; ``mix`` float32 [S, S]
+    (from, to), ``out`` float32 [S]."""
+
+    def __init__(self, value, mix, out):
+        self.value, self.mix, self.out = value, mix, out
+        self.shape, self.device = tuple(value.shape), value.device
+
+
 class RoutedSum:
     """The result of a routed feed-forward before its weighted sum: ``pairs`` float32 [N * top, width] (every (token,
     slot) pair's expert output), ``weights`` and ``chosen`` [N, top], and the feed-forward's input ``x`` (what an
@@ -395,13 +405,18 @@ def _check_caches(k_cache, v_cache, dtype, kv_heads, page_size, head_dim):
         raise ValueError(f'v_cache must be [pages, {kv_heads}, {head_dim}, {page_size}]')
 
 
-def embed(token_ids, table, scale=1.0):
-    """int32 [N], T [V, H] -> float32 stream [N, H] = table[token] * scale."""
+def embed(token_ids, table, scale=1.0, streams=1):
+    """int32 [N], T [V, H] -> float32 stream [N, H] = table[token] * scale; ``streams`` > 1: [N, streams * H], a row's
+    copies one behind another."""
     library.check_device()                                 # every step begins here
     _require(token_ids, 'token_ids', torch.int32)
     _require(table, 'table')
     n, width = token_ids.shape[0], table.shape[1]
-    stream = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    stream = torch.empty((n, streams * width), dtype=torch.float32, device=table.device)
+    if streams > 1:
+        _check(library.load().qil_embed_streams(_ptr(token_ids), _ptr(table), _ptr(stream), n, width, int(streams), float(scale),
+                                                _code(table.dtype), _stream()), 'embed_streams')
+        return stream
     _check(library.load().qil_embed(_ptr(token_ids), _ptr(table), _ptr(stream), n, width, float(scale), _code(table.dtype),
                                     _stream()), 'embed')
     return stream
@@ -458,6 +473,56 @@ def residual_join(stream, pending, weight, eps, out_dtype, rows=None):
         _ptr(pending.plus), _ptr(pending.step), _ptr(rows), _ptr(weight), _ptr(out), count, n, width, float(eps),
         int(rows is None), _code(out_dtype), _stream()), 'residual_join')
     return out
+
+
+def check_streams(streams):
+    """Numbers of residual streams the kernels take; called when a block is built."""
+    if type(streams) is not int or not 1 <= streams <= 16:
+        raise UnsupportedShape(f'{streams!r} residual streams: from 1 to 16')
+
+
+def stream_join(stream, pending, *, streams, out_dtype, read=None, norm=None, rows=None):
+    """What is pending joins the float32 residual streams [N, streams * H] in place (a ``StreamUpdate``; with one stream
+    also a tensor of ``out_dtype``, ``Partials`` or a ``RoutedSum``, which is added; None: nothing), and the next sub-layer's input
+    comes back, [N, H] of ``out_dtype``: u = sum_s read[s] x_s (``read`` float32 [streams], None: the plain sum), then, with
+    ``norm`` (alpha, weight, bias; float32 [1], [H], [H]), tanh(alpha u) * weight + bias.  float32 until the one rounding.
+    ``rows``: for the selected rows only, the streams are left as they are."""
+    n, width = stream.shape[0], stream.shape[1] // streams
+    _require(stream, 'stream', torch.float32, (n, streams * width))
+    mix = out_weights = None
+    if isinstance(pending, StreamUpdate):
+        mix, out_weights, pending = pending.mix, pending.out, pending.value
+        _require(mix, 'mix', torch.float32, (streams, streams))
+        _require(out_weights, 'out', torch.float32, (streams,))
+    elif pending is not None and streams > 1:
+        raise TypeError('several streams take a StreamUpdate')
+    if isinstance(pending, RoutedSum) and pending.dtype != out_dtype:
+        pending = _plain_delta(pending)
+    value, routed = (None, 0, 1, width), (None, None, None, None, 0, 0)
+    if isinstance(pending, RoutedSum):
+        top = pending.chosen.shape[1]
+        _require(pending.x, 'routed input', out_dtype, (n, width))
+        _require(pending.pairs, 'routed pairs', torch.float32, (n * top, width))
+        _require(pending.chosen, 'chosen', torch.int32, (n, top))
+        _require(pending.weights, 'weights', torch.float32, (n, top))
+        routed = (_ptr(pending.pairs), _ptr(pending.weights), _ptr(pending.chosen), _ptr(pending.x), top, pending.experts)
+    elif pending is not None:
+        value = _row_operand(pending, 'delta', n, width)
+    if read is not None:
+        _require(read, 'read', torch.float32, (streams,))
+    alpha, weight, bias = norm if norm is not None else (None, None, None)
+    if norm is not None:
+        _require(alpha, 'alpha', torch.float32)
+        _require(weight, 'weight', torch.float32, (width,))
+        _require(bias, 'bias', torch.float32, (width,))
+    if rows is not None:
+        _require(rows, 'rows', torch.int32)
+    count = n if rows is None else rows.shape[0]
+    result = torch.empty((count, width), dtype=out_dtype, device=stream.device)
+    _check(library.load().qil_stream_join(_ptr(stream), streams, *value, *routed, _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(rows),
+                                          _ptr(alpha), _ptr(weight), _ptr(bias), _ptr(result), count, n, width, int(rows is None),
+                                          _code(out_dtype), _stream()), 'stream_join')
+    return result
 
 
 def add_rmsnorm(stream, delta, weight, eps, out_dtype):
@@ -1257,12 +1322,12 @@ def short_conv(x, weight, *, state, cu_seqlens, seq_starts, seq_slots, row_seq, 
 # Attention over a cached latent
 def latent_prepare(down, *, q_rank, rank, rot, q_weight, c_weight, eps, frequencies, positions, slots, latent, rope,
                    dtype, gates=0):
-    """From the stacked down products ``down`` [N, q_rank + rank + rot (+ gates)] (tensor of ``dtype`` or Partials):
+    """From the stacked down products ``down`` [N, q_rank + rank + rot (+ gates)] (tensor of ``dtype``, Partials or Columns):
     the RMS-normed query latent [N, q_rank] (returned); the RMS-normed key/value latent and the rotated shared key
     part go into the caches ``latent`` [.., rank] / ``rope`` [.., rot] at ``slots`` (None: nothing is stored).  With
     ``gates`` more columns the result is (query latent, float32 [N, gates] of their sigmoids)."""
     n = down.shape[0]
-    pointer, code, splits = _operand(down, 'down', dtype, (n, q_rank + rank + rot + gates))
+    pointer, code, splits, row = _row_operand(down, 'down', n, q_rank + rank + rot + gates, (dtype, torch.float32))
     _require(q_weight, 'q_weight', torch.float32, (q_rank,))
     _require(c_weight, 'c_weight', torch.float32, (rank,))
     _require(frequencies, 'frequencies', torch.float32, (rot // 2,))
@@ -1275,7 +1340,7 @@ def latent_prepare(down, *, q_rank, rank, rot, q_weight, c_weight, eps, frequenc
             raise ValueError('latent_prepare: caches must be [.., rank] and [.., rot] over the same slots')
     out = torch.empty((n, q_rank), dtype=dtype, device=down.device)
     gate = torch.empty((n, gates), dtype=torch.float32, device=down.device) if gates else None
-    _check(library.load().qil_latent_prepare(pointer, code, splits, _ptr(q_weight), _ptr(c_weight), _ptr(frequencies),
+    _check(library.load().qil_latent_prepare(pointer, code, splits, row, _ptr(q_weight), _ptr(c_weight), _ptr(frequencies),
                                              _ptr(positions), _ptr(slots), _ptr(out), _ptr(latent), _ptr(rope), _ptr(gate),
                                              n, q_rank, rank, rot, gates, float(eps), _code(dtype), _stream()),
            'latent_prepare')
@@ -1285,12 +1350,12 @@ def latent_prepare(down, *, q_rank, rank, rot, q_weight, c_weight, eps, frequenc
 HEAD_PRODUCT_BLAS_ROWS = 256     # rows from which a bfloat16 product per head goes to the GPU BLAS in one batch
 
 
-def head_product(x, weight, *, heads, out_dtype, out=None, out_columns=None):
+def head_product(x, weight, *, heads, out_dtype, out=None, out_columns=None, gate=None):
     """A product per head: x [N, heads * X] (head h's K inputs lead its X columns), weight [heads, K, O] (for every k
     its O outputs side by side) -> [N, heads * O] of ``out_dtype``, or into the leading O of every head's
     ``out_columns`` columns of ``out``.  Own kernels for few rows (k split in a block) and in float32; bfloat16 weights
     with ``HEAD_PRODUCT_BLAS_ROWS`` rows or more take one batched product of the GPU BLAS, float32 inputs rounded to
-    bfloat16 first."""
+    bfloat16 first.  ``gate`` [N, heads * O] (tensor, Partials or Columns): the result is multiplied by its sigmoid."""
     n = x.shape[0]
     _require(x, 'x')
     _require(weight, 'weight')
@@ -1301,17 +1366,23 @@ def head_product(x, weight, *, heads, out_dtype, out=None, out_columns=None):
         out_columns = o
         out = torch.empty((n, heads * o), dtype=out_dtype, device=x.device)
     _require(out, 'out', out_dtype, (n, heads * out_columns))
+    gate_operand = (None, 0, 1, 0) if gate is None else _row_operand(gate, 'gate', n, heads * o)
     if n >= HEAD_PRODUCT_BLAS_ROWS and weight.dtype == torch.bfloat16:
         # many rows: one batched matrix-core product of the GPU BLAS (bfloat16 operands, float32 sums), a batch per head
         inputs = x.view(n, heads, x.shape[1] // heads)[:, :, :k]
         if inputs.dtype != torch.bfloat16:
             inputs = inputs.to(torch.bfloat16)
         product = torch.bmm(inputs.transpose(0, 1), weight)                    # [heads, N, O]
+        if gate is not None and out_columns == o and out_dtype == torch.bfloat16:
+            _check(library.load().qil_gated_heads(_ptr(product), *gate_operand, _ptr(out), n, heads, o, _stream()), 'gated_heads')
+            return out
+        if gate is not None:
+            raise UnsupportedShape('a gated product per head of many rows has a bfloat16 result in whole rows')
         out.view(n, heads, out_columns)[:, :, :o].copy_(product.transpose(0, 1))
         return out
     _check(library.load().qil_head_product(_ptr(x), _code(x.dtype), x.shape[1], x.shape[1] // heads, _ptr(weight),
                                            _code(weight.dtype), _ptr(out), _code(out_dtype), heads * out_columns,
-                                           out_columns, n, heads, k, o, _stream()), 'head_product')
+                                           out_columns, n, heads, k, o, *gate_operand, _stream()), 'head_product')
     return out
 
 
@@ -1580,11 +1651,16 @@ def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bi
     return chosen, weights
 
 
+# Activations of experts without a gate branch: name -> code of the kernels.  'relu_squared': max(z, 0)^2.
+EXPERT_ACTIVATIONS = {'relu_squared': 16}
+
+
 def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alpha=1.0, lazy=False):
     """The weighted sum of the chosen experts' outputs, float32 [N, width]; with ``lazy`` a ``RoutedSum`` (the pairs'
     rows, for a norm that makes the sum while it loads them).  ``gate_up`` [experts, 2, ff, width] (an
     expert's gate rows, then its up rows), ``down`` [experts, width, ff], both of x's type; an expert computes
-    down(act(gate x, up x)) with ``activation`` of ``GATE_FUNCTIONS``.  A chosen index from ``experts`` on is an
+    down(act(gate x, up x)) with ``activation`` of ``GATE_FUNCTIONS``; with an ``activation`` of ``EXPERT_ACTIVATIONS`` there is no
+    gate branch, ``gate_up`` is [experts, 1, ff, width] and an expert computes down(act(up x)).  A chosen index from ``experts`` on is an
     identity expert: its output is x itself.  The pairs (token, chosen expert) are grouped by expert on the device;
     the host sees no routing result, so a step may be captured into a graph."""
     n, width = x.shape
@@ -1593,7 +1669,8 @@ def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alp
     _require(chosen, 'chosen', torch.int32, (n, top))
     _require(weights, 'weights', torch.float32, (n, top))
     experts, ff = gate_up.shape[0], gate_up.shape[2]
-    _require(gate_up, 'gate_up', x.dtype, (experts, 2, ff, width))
+    act = GATE_FUNCTIONS[activation] if activation in GATE_FUNCTIONS else EXPERT_ACTIVATIONS[activation]
+    _require(gate_up, 'gate_up', x.dtype, (experts, 2 if activation in GATE_FUNCTIONS else 1, ff, width))
     _require(down, 'down', x.dtype, (experts, width, ff))
     lib = library.load()
     pairs = n * top
@@ -1605,7 +1682,7 @@ def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alp
     out = None if lazy else torch.empty((n, width), dtype=torch.float32, device=x.device)
     _check(lib.qil_moe_experts(_ptr(x), _code(x.dtype), _ptr(chosen), _ptr(weights), _ptr(gate_up), _ptr(down),
                                _ptr(scratch), scratch[3 * max_tiles:].data_ptr(), _ptr(hidden), _ptr(y), _ptr(out), n, width,
-                               ff, experts, top, tile_rows, max_tiles, GATE_FUNCTIONS[activation], float(limit),
+                               ff, experts, top, tile_rows, max_tiles, act, float(limit),
                                float(alpha), _stream()), 'moe_experts')
     return RoutedSum(x, y, chosen, weights, experts) if lazy else out
 
@@ -1670,13 +1747,14 @@ CONV_ACTIVATIONS = {None: 0, 'silu': 1}
 
 
 def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq_slots, row_seq, n_seqs, activation,
-                 out_dtype):
+                 out_dtype, pass_from=0, passed=0):
     """act(bias + causal convolution over time) on the first ``columns`` columns of ``x`` [N, W] (tensor of the
     model's type, Partials or Columns): out[t, c] = act(bias[c] + sum_j weight[j, c] * x[t - taps + 1 + j, c]) over the rows of
     every sequence of the step and the taps - 1 inputs before them, which are the sequence's state (``state`` float32
     [slots, taps - 1, columns]: read unless the sequence starts at position 0, and left holding the sequence's last
     taps - 1 inputs).  ``weight`` float32 [taps, columns], ``bias`` float32 [columns] or None.  -> [N, columns] of
-    ``out_dtype``; float32 arithmetic, one rounding."""
+    ``out_dtype``; float32 arithmetic, one rounding.  ``passed``: so many columns of x from ``pass_from`` on come back as
+    they are beside it, (result, [N, passed] of ``out_dtype``)."""
     n, width = x.shape
     taps = weight.shape[0]
     _require(weight, 'weight', torch.float32, (taps, columns))
@@ -1692,11 +1770,13 @@ def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq
     _require(row_seq, 'row_seq', torch.int32, (n,))
     pointer, code, splits, width = _row_operand(x, 'x', n, width)
     out = torch.empty((n, columns), dtype=out_dtype, device=weight.device)
+    through = torch.empty((n, passed), dtype=out_dtype, device=weight.device) if passed else None
     _check(library.load().qil_channel_conv(pointer, code, splits, width, _ptr(weight), _ptr(bias),
                                            _ptr(state) if taps > 1 else None, _ptr(cu_seqlens), _ptr(seq_starts),
                                            _ptr(seq_slots), _ptr(row_seq), _ptr(out), _code(out_dtype), n, columns, taps,
-                                           CONV_ACTIVATIONS[activation], _stream()), 'channel_conv')
-    return out
+                                           CONV_ACTIVATIONS[activation], int(pass_from), int(passed), _ptr(through), _stream()),
+           'channel_conv')
+    return (out, through) if passed else out
 
 
 def selective_scan(u, dt, bc, gate, *, dt_bias, a, d, state, gate_offset, cu_seqlens, seq_starts, seq_slots, n_seqs,
@@ -1742,3 +1822,106 @@ def selective_scan(u, dt, bc, gate, *, dt_bias, a, d, state, gate_offset, cu_seq
                                   _ptr(seq_slots), _ptr(y), _code(out_dtype), n, n_seqs, channels, states, int(max_query),
                                   _ptr(workspace), _stream()), 'selective_scan')
     return y
+
+
+# ---------------------------------------------------------------------------------------------------------------
+# Attention with two maps a head over the same values
+def pair_store(qkv, *, heads, kv_heads, dim, vdim, padded, slots, k_cache, v_cache, page_size, dtype):
+    """The rows [heads * 2 dim queries | kv_heads * 2 dim keys | kv_heads * vdim values | ..] of ``qkv`` (tensor of ``dtype``,
+    Partials or Columns; ``kv_heads`` 0: queries only) as the attention kernels take them: a key head's two keys are one
+    cached key [k1 | k2 | 0] of ``padded`` elements, its value is cached beside it (at ``slots``; None: not stored), and a
+    head's two queries come back as the rows [q1 | 0 | 0] and [0 | q2 | 0] of two query heads: [N, 2 heads * padded]."""
+    n = qkv.shape[0]
+    pointer, code, splits, row = _row_operand(qkv, 'qkv', n, qkv.shape[1], (dtype, torch.float32))
+    if slots is not None:
+        _require(slots, 'slots', torch.int32, (n,))
+        _check_caches(k_cache, v_cache, dtype, kv_heads, page_size, padded)
+    q = torch.empty((n, 2 * heads * padded), dtype=dtype, device=qkv.device)
+    _check(library.load().qil_pair_store(pointer, code, splits, row, _ptr(q), _ptr(slots), _ptr(k_cache), _ptr(v_cache), n, heads,
+                                         kv_heads, dim, vdim, padded, page_size, _code(dtype), _stream()), 'pair_store')
+    return q
+
+
+def difference_combine(maps, gate, *, heads, vdim, padded, factor, post, eps, dtype):
+    """o = a1 - factor * a2 of every head's two results (``maps`` [N, 2 heads * padded] of ``dtype``, or ``Unmerged`` parts of
+    them), o / sqrt(mean(o^2) + eps) over its ``vdim`` elements, times ``post`` and sigmoid(gate[:, head]) (``gate`` [N, heads]: tensor,
+    Partials or Columns).  float32 and one rounding.  -> [N, heads * vdim] of ``dtype``."""
+    n = maps.shape[0]
+    gate_operand = _row_operand(gate, 'gate', n, heads)
+    out = torch.empty((n, heads * vdim), dtype=dtype, device=maps.device)
+    parts = (None, None, 0, 1, 1)
+    tensor = None
+    if isinstance(maps, Unmerged):
+        if (maps.heads, maps.head_dim) != (2 * heads, padded):
+            raise ValueError('difference_combine: the parts are of other heads')
+        parts = (_ptr(maps.workspace), _ptr(maps.positions), maps.window, maps.part, maps.parts)
+    else:
+        _require(maps, 'maps', dtype, (n, 2 * heads * padded))
+        tensor = maps
+    _check(library.load().qil_difference_combine(_ptr(tensor), *parts, *gate_operand, float(factor), float(post), float(eps), _ptr(out),
+                                                 n, heads, vdim, padded, _code(dtype), _stream()), 'difference_combine')
+    return out
+
+
+# ---------------------------------------------------------------------------------------------------------------
+# The gated delta rule
+DELTA_CHUNKS_FROM = 32          # rows of one sequence from which a step's recurrence runs in chunks of 64 on the matrix cores
+
+
+def check_delta_geometry(*, heads, kv_heads, dim, vdim):
+    """Sizes the delta rule's kernels take; called when the part is built."""
+    if heads < 1 or kv_heads < 1 or heads % kv_heads or not 1 <= dim <= 256 or vdim < 1:
+        raise UnsupportedShape(f'delta rule: {heads} heads over {kv_heads}, dim {dim} (up to 256), vdim {vdim}')
+
+
+def delta_rule(u, decays, steps, *, heads, kv_heads, dim, vdim, q_offset, k_offset, v_offset, decay_bias, rates, state, cu_seqlens,
+               seq_starts, seq_slots, n_seqs, max_query, gate, weight, eps, tile_seqs=None):
+    """Per head, with unit vectors k, q (x / sqrt(sum(x^2) + 1e-6); q also times dim^(-1/2)), over every sequence's rows:
+
+        S <- diag(g) S;   w = beta (v - S^T k);   S <- S + k w^T;   o = S^T q
+        g = exp(rates[h] softplus(decays + decay_bias)) per key channel, beta = sigmoid(steps)
+
+    then o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate) per head.  ``u`` [N, U]: queries and keys of ``kv_heads`` heads
+    (head h reads h // (heads / kv_heads)) and values of ``heads`` from the offsets on.  ``decays`` [N, heads * dim], ``steps``
+    [N, heads], ``gate`` [N, heads * vdim]: tensors, Partials or Columns.  ``state`` float32 [slots, heads * dim * vdim], read
+    unless a sequence starts at position 0 and left holding S.  float32 until the one rounding of the result, [N, heads *
+    vdim] of u's type.  From ``DELTA_CHUNKS_FROM`` rows of a sequence on the sequences of several rows (the first ``tile_seqs``; None:
+    all) run in chunks, the others token by token: they differ by rounding only."""
+    n = u.shape[0]
+    _require(u, 'u')
+    dtype, lib = u.dtype, library.load()
+    if not lib.qil_delta_takes(dim, vdim):
+        raise UnsupportedShape(f'delta_rule: dim {dim} (up to 256), vdim {vdim}')
+    _require(decay_bias, 'decay_bias', torch.float32, (heads * dim,))
+    _require(rates, 'rates', torch.float32, (heads,))
+    _require(weight, 'weight', torch.float32, (vdim,))
+    _require(state, 'state', torch.float32)
+    if state.ndim != 2 or state.shape[1] != heads * dim * vdim:
+        raise ValueError(f'delta_rule: state must be [slots, {heads * dim * vdim}]')
+    _require(cu_seqlens, 'cu_seqlens', torch.int32, (n_seqs + 1,))
+    _require(seq_starts, 'seq_starts', torch.int32, (n_seqs,))
+    _require(seq_slots, 'seq_slots', torch.int32, (n_seqs,))
+    rows = (_ptr(u), _code(dtype), u.shape[1], q_offset, k_offset, v_offset, *_row_operand(decays, 'decays', n, heads * dim),
+            _ptr(decay_bias), _ptr(rates), *_row_operand(steps, 'steps', n, heads), _ptr(state))
+    gate_operand = _row_operand(gate, 'gate', n, heads * vdim)
+    sizes = (heads, kv_heads, dim, vdim)
+    out = torch.empty((n, heads * vdim), dtype=dtype, device=u.device)
+    chunked = 0
+    if max_query >= DELTA_CHUNKS_FROM and lib.qil_delta_chunked_takes(dim, vdim, u.shape[1], q_offset, k_offset, _code(dtype)):
+        chunked = n_seqs if tile_seqs is None else tile_seqs
+    if not chunked and lib.qil_delta_ends(vdim):
+        _check(lib.qil_delta_tokens(*rows, _ptr(cu_seqlens), _ptr(seq_starts), _ptr(seq_slots), None, _ptr(out), _ptr(weight),
+                                    *gate_operand, float(eps), n, n_seqs, *sizes, _stream()), 'delta_tokens')
+        return out
+    raw = torch.empty((n, heads * vdim), dtype=torch.float32, device=u.device)
+    if chunked:
+        scratch = torch.empty(lib.qil_delta_chunked_workspace(n, chunked, heads, dim, vdim), dtype=torch.float32, device=u.device)
+        _check(lib.qil_delta_chunked(*rows, _ptr(cu_seqlens), _ptr(seq_starts), _ptr(seq_slots), _ptr(raw), _ptr(scratch), n,
+                                     chunked, int(max_query), *sizes, _stream()), 'delta_chunked')
+    if n_seqs > chunked:
+        _check(lib.qil_delta_tokens(*rows, cu_seqlens[chunked:].data_ptr(), seq_starts[chunked:].data_ptr(),
+                                    seq_slots[chunked:].data_ptr(), _ptr(raw), None, None, None, 0, 1, 0, 0.0, n, n_seqs - chunked,
+                                    *sizes, _stream()), 'delta_tokens')
+    _check(lib.qil_delta_end(_ptr(raw), _ptr(weight), *gate_operand, float(eps), _ptr(out), n, heads, vdim, _code(dtype), _stream()),
+           'delta_end')
+    return out

@@ -290,8 +290,10 @@ def _declare(lib):
     lib.qil_gemm_bf16_wide_gated.argtypes = [p, p, p, i, i, i, i, p]
     lib.qil_add_norm.argtypes = [p, p, i, i, i, f, p, p, p, p, i, i, f, i, i, i, p]
     lib.qil_gated_act.argtypes = [p, i, i, i, p, i, i, i, i, i, f, f, p]
-    lib.qil_latent_prepare.argtypes = [p, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, f, i, p]
-    lib.qil_head_product.argtypes = [p, i, i, i, p, i, p, i, i, i, i, i, i, i, p]
+    lib.qil_latent_prepare.argtypes = [p, i, i, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, f, i, p]
+    lib.qil_head_product.argtypes = [p, i, i, i, p, i, p, i, i, i, i, i, i, i, p, i, i, i, p]
+    lib.qil_gated_heads.argtypes = [p, p, i, i, i, p, i, i, i, p]
+    lib.qil_gated_heads.restype = i
     lib.qil_rotate_tail.argtypes = [p, i, i, i, i, p, p, p, i, i, i, i, i, i, p]
     lib.qil_latent_attention_takes.argtypes = [i, i, i]
     lib.qil_latent_attention_takes.restype = i
@@ -331,7 +333,7 @@ def _declare(lib):
     lib.qil_scaled_sum.argtypes = [p, i, i, p, i, i, f, f, p, i, i, p]
     lib.qil_sigmoid_gate.argtypes = [p, p, i, i, i, i, p, i, i, i, p]
     lib.qil_soft_cap.argtypes = [p, f, z, p]
-    lib.qil_channel_conv.argtypes = [p, i, i, i, p, p, p, p, p, p, p, p, i, i, i, i, i, p]
+    lib.qil_channel_conv.argtypes = [p, i, i, i, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p, p]
     lib.qil_selective_scan_takes.argtypes = [i, i, i]
     lib.qil_selective_scan.argtypes = [p, p, i, i, p, p, p, i, i, p, p, i, i, i, i, p, p, p, p, p, i, i, i, i, i, i, p, p]
     lib.qil_selective_scan_workspace.argtypes = [i, i, i, i]
@@ -364,6 +366,24 @@ def _declare(lib):
     lib.qil_step_scan.argtypes = [p, i, i, i, i, p, i, i, i, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
     lib.qil_step_token.argtypes = [p, i, i, i, i, i, p, i, i, i, p, p, p, p, p, p, p, i, i, i, i, i, i, p]
     for name in ('qil_step_scan_takes', 'qil_step_token_takes', 'qil_step_scan', 'qil_step_token', 'qil_embed_pairs', 'qil_gated_group_norm', 'qil_residual_join', 'qil_qk_row_norm_store'):
+        getattr(lib, name).restype = i
+    lib.qil_stream_join_takes.argtypes = [i]
+    lib.qil_stream_join.argtypes = [p, i, p, i, i, i, p, p, p, p, i, i, p, p, p, p, p, p, p, p, i, i, i, i, i, p]
+    lib.qil_embed_streams.argtypes = [p, p, p, i, i, i, f, i, p]
+    lib.qil_pair_store.argtypes = [p, i, i, i, p, p, p, p, i, i, i, i, i, i, i, i, p]
+    lib.qil_difference_combine.argtypes = [p, p, p, i, i, i, p, i, i, i, f, f, f, p, i, i, i, i, i, p]
+    lib.qil_delta_takes.argtypes = [i, i]
+    lib.qil_delta_ends.argtypes = [i]
+    operands = [p, i, i, i, i, i, p, i, i, i, p, p, p, i, i, i, p, p, p, p]      # rows, raw decays, step sizes, state and sequences
+    lib.qil_delta_tokens.argtypes = operands + [p, p, p, p, i, i, i, f, i, i, i, i, i, i, p]
+    lib.qil_delta_end.argtypes = [p, p, p, i, i, i, f, p, i, i, i, i, p]
+    lib.qil_delta_chunked_takes.argtypes = [i, i, i, i, i, i]
+    lib.qil_delta_chunked_workspace.argtypes = [i, i, i, i, i]
+    lib.qil_delta_chunked_workspace.restype = z
+    lib.qil_delta_chunked.argtypes = operands + [p, p, i, i, i, i, i, i, i, p]
+    for name in ('qil_stream_join_takes', 'qil_stream_join', 'qil_embed_streams', 'qil_pair_store', 'qil_difference_combine',
+                 'qil_delta_takes', 'qil_delta_ends', 'qil_delta_tokens', 'qil_delta_end', 'qil_delta_chunked_takes',
+                 'qil_delta_chunked'):
         getattr(lib, name).restype = i
     lib.qil_sample.argtypes = [p, p, p, p, p, p, p, i, i, p]
     lib.qil_sample_workspace.argtypes = [i, i]

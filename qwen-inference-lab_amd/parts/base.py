@@ -129,6 +129,15 @@ class Norm(Part):
         raise NotImplementedError
 
 
+    def forward_streams(self, stream, pending, out_dtype, *, streams, read):
+        """Several residual streams [N, streams * width]: what is pending (``ops.StreamUpdate`` or None) joins them in place,
+        and the norm of u = sum_s read[s] x_s comes back.  This form makes u first; a norm with a kernel for it overrides it."""
+        from .. import ops
+        import torch
+        joined = ops.stream_join(stream, pending, streams=streams, read=read, out_dtype=torch.float32)
+        return self.forward(joined, None, out_dtype)
+
+
 class PositionEncoding(Part):
     """Something the mixer applies to queries and keys by absolute position.
 

@@ -262,3 +262,50 @@ class ParallelBlock(Block):
         ffn = self.ffn.forward(shared if self.ffn.input_matrices() else h) if self.ffn is not None else None
         gates = ops.linear(shared, self.p['gates.weight'], None, partials=True) if self.gated else None
         return ops.Joined(mixed, ffn, gates, self.p.get('gates.bias'))
+
+
+class StreamsBlock(Block):
+    """Several residual streams x_1 .. x_S side by side (hyper-connections), mixer then feed-forward (or the mixer alone).
+    For each sub-layer, with stored weights of its own:
+
+        u = sum_s in[s] x_s;   y = sublayer(norm(u));   x_t <- sum_s mix[s, t] x_s + out[t] y     (all t from the old x)
+
+    (tensors ``mixer_in``, ``mixer_mix``, ``mixer_out``, and ``ffn_*``).  The stream is float32 [N, S * width], a row's streams one
+    behind another.  A sub-layer's output leaves as an ``ops.StreamUpdate``, and the norm that follows, this block's, the next
+    one's or the model's last, joins it to the streams, mixes them and makes its own input in one kernel, in float32."""
+
+    def __init__(self, *, mixer_norm, mixer, ffn_norm=None, ffn=None, streams, dtype, names=None):
+        super().__init__()
+        if (ffn is None) != (ffn_norm is None):
+            raise ValueError('a feed-forward and its norm come together')
+        ops.check_streams(streams)
+        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+        self.streams, self.dtype = streams, dtype
+        self._names = names or dict(mixer_norm='mixer_norm', mixer='mixer', ffn_norm='ffn_norm', ffn='ffn')
+
+    def parts(self):
+        n = self._names
+        out = {n['mixer_norm']: self.mixer_norm, n['mixer']: self.mixer}
+        if self.ffn is not None:
+            out.update({n['ffn_norm']: self.ffn_norm, n['ffn']: self.ffn})
+        return out
+
+    def param_specs(self):
+        s, specs = self.streams, {}
+        for name in ('mixer',) + (('ffn',) if self.ffn is not None else ()):
+            specs[f'{name}_in'] = ParamSpec((s,), 'vector', 'one_plus_normal')
+            specs[f'{name}_mix'] = ParamSpec((s, s), 'vector')
+            specs[f'{name}_out'] = ParamSpec((s,), 'vector', 'one_plus_normal')
+        return specs
+
+    def _enter(self, name, norm, stream, pending):
+        return norm.forward_streams(stream, pending, self.dtype, streams=self.streams, read=self.p[f'{name}_in'])
+
+    def _leave(self, name, value):
+        return ops.StreamUpdate(value, self.p[f'{name}_mix'], self.p[f'{name}_out'])
+
+    def forward(self, stream, pending, ctx, cache):
+        mixed = self._leave('mixer', self.mixer.forward(self._enter('mixer', self.mixer_norm, stream, pending), ctx, cache))
+        if self.ffn is None:
+            return mixed
+        return self._leave('ffn', self.ffn.forward(self._enter('ffn', self.ffn_norm, stream, mixed)))

@@ -4,16 +4,20 @@ from .. import ops
 
 
 class Embedding(Part):
-    """stream[n] = float32(table[token[n]]) * scale; no scaling (scale 1) in qil/model.py:126."""
+    """stream[n] = float32(table[token[n]]) * scale; no scaling (scale 1) in qil/model.py:126.  ``streams``: so many
+    copies of it, for a model with several residual streams."""
 
-    def __init__(self, vocab, width, scale=1.0):
+    def __init__(self, vocab, width, scale=1.0, streams=1):
         super().__init__()
-        self.vocab, self.width, self.scale = vocab, width, float(scale)
+        ops.check_streams(streams)
+        self.vocab, self.width, self.scale, self.streams = vocab, width, float(scale), streams
 
     def param_specs(self):
         return {'weight': ParamSpec((self.vocab, self.width))}
 
     def forward(self, token_ids):
+        if self.streams > 1:
+            return ops.embed(token_ids, self.p['weight'], self.scale, streams=self.streams)
         return ops.embed(token_ids, self.p['weight'], self.scale)
 
     def forward_step(self, ctx):

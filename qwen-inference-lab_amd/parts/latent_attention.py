@@ -20,8 +20,10 @@ class LatentAttention(Mixer):
     ``position``: a ``RotaryFrequencies`` over ``rot_dim`` elements.
     ``window`` w: row i sees the keys j with 0 <= i - j < w only, and the cache gives pages back that no later row
     sees (None: every key j <= i).
-    ``gate``: head h's result is multiplied by sigmoid(W_g x)_h (tensor ``g_proj.weight`` [heads, width]; the
-    sigmoid in float32); W_g is stacked under the two down projections, so the gate costs no product of its own.
+    ``gate``: 'head' (or True), head h's result is multiplied by sigmoid(W_g x)_h (tensor ``g_proj.weight`` [heads, width];
+    the sigmoid in float32); 'element', the heads' values are multiplied element by element by sigmoid(W_g x) before the
+    output projection (``g_proj.weight`` [heads * vdim, width]), in the kernel that expands them.  W_g is stacked under the two
+    down projections, so the gate costs no product of its own.
     ``pairing``: which elements of the rotated parts a rotation pairs: 'halves', (i, i + rot_dim / 2), which is what
     the kernels do, or 'neighbours', (2 i, 2 i + 1) with the same frequency f_i.  A score does not change when the
     elements of the query's and the key's rotated part are reordered alike, so for 'neighbours' the rows of W_uq
@@ -47,7 +49,9 @@ class LatentAttention(Mixer):
             raise ops.UnsupportedShape(f'window must be a positive integer or None, not {window!r}')
         if pairing not in ('halves', 'neighbours'):
             raise ValueError(f"pairing must be 'halves' or 'neighbours', not {pairing!r}")
-        self.window, self.gate, self.pairing = window, bool(gate), pairing
+        if gate not in (False, True, None, 'head', 'element'):
+            raise ValueError(f"gate must be 'head', 'element' or False, not {gate!r}")
+        self.window, self.gate, self.pairing = window, 'head' if gate is True else gate or None, pairing
 
     def param_specs(self):
         h, d, r = self.heads, self.dim, self.rot_dim
@@ -62,7 +66,7 @@ class LatentAttention(Mixer):
         if self.sink:
             specs['sink'] = ParamSpec((h,), 'vector', 'normal')
         if self.gate:
-            specs['g_proj.weight'] = ParamSpec((h, self.width))
+            specs['g_proj.weight'] = ParamSpec((h if self.gate == 'head' else h * self.vdim, self.width))
         return specs
 
     def cache_need(self):
@@ -77,8 +81,20 @@ class LatentAttention(Mixer):
             p['q_up.weight'] = torch.cat([q_up[:, :d], q_up[:, d:][:, order]], dim=1).reshape(-1, self.q_rank).contiguous()
             kv_down = p['kv_down.weight']
             p['kv_down.weight'] = torch.cat([kv_down[:self.kv_rank], kv_down[self.kv_rank:][order]]).contiguous()
-        # the down products in one: [q_rank + kv_rank + rot_dim (+ heads), width]
-        stacked = [p.pop('q_down.weight'), p.pop('kv_down.weight')] + ([p.pop('g_proj.weight')] if self.gate else [])
+        # the down products in one: [q_rank + kv_rank + rot_dim (+ the gate's rows), width]
+        stacked = [p.pop('q_down.weight'), p.pop('kv_down.weight')]
+        self.own_rows = self.gate_offset = self.q_rank + self.kv_rank + self.rot_dim
+        if self.gate == 'head':
+            stacked.append(p.pop('g_proj.weight'))
+            self.own_rows += self.heads
+        elif self.gate == 'element':                    # at a multiple of 8 rows, the stack too
+            for piece in (None, p.pop('g_proj.weight')):
+                if piece is not None:
+                    self.gate_offset = sum(matrix.shape[0] for matrix in stacked)
+                    stacked.append(piece)
+                pad = -sum(matrix.shape[0] for matrix in stacked) % 8
+                if pad:
+                    stacked.append(stacked[0].new_zeros((pad, self.width)))
         self.w_down = torch.cat(stacked).contiguous()
         p['down.weight'] = self.w_down
         # W_uk as [heads, dim, kv_rank] is the layout the query's product reads (a pure view); W_uv per head transposed
@@ -90,12 +106,13 @@ class LatentAttention(Mixer):
         p = self.p
         frequencies = self.position.frequencies()
         down = ops.linear(h, self.w_down, None, partials=True)
-        cq = ops.latent_prepare(down, q_rank=self.q_rank, rank=self.kv_rank, rot=self.rot_dim, q_weight=p['q_norm.weight'],
+        own = down if self.gate != 'element' else ops.columns(down, 0, self.own_rows)
+        cq = ops.latent_prepare(own, q_rank=self.q_rank, rank=self.kv_rank, rot=self.rot_dim, q_weight=p['q_norm.weight'],
                                 c_weight=p['kv_norm.weight'], eps=self.eps, frequencies=frequencies,
                                 positions=ctx.positions, slots=cache.slots if cache.writes else None,
                                 latent=cache.tensors['latent'], rope=cache.tensors['rope'], dtype=self.dtype,
-                                gates=self.heads if self.gate else 0)
-        cq, gate = cq if self.gate else (cq, None)
+                                gates=self.heads if self.gate == 'head' else 0)
+        cq, gate = cq if self.gate == 'head' else (cq, None)
         q = ops.linear(cq, p['q_up.weight'], None)
         q = ops.latent_query(q, self.k_up, heads=self.heads, dim=self.dim, rot=self.rot_dim, rank=self.kv_rank,
                              frequencies=frequencies, positions=ctx.positions)
@@ -105,5 +122,9 @@ class LatentAttention(Mixer):
                                      rank=self.kv_rank, rot=self.rot_dim, cu_seqlens=ctx.cu_seqlens,
                                      seq_starts=ctx.seq_starts, n_seqs=ctx.n_seqs, max_query=ctx.max_query,
                                      max_context=ctx.max_context, window=self.window, gate=gate)
-        values = ops.head_product(mixed, p['v_up.weight'], heads=self.heads, out_dtype=self.dtype)
+        if self.gate == 'element':
+            values = ops.head_product(mixed, p['v_up.weight'], heads=self.heads, out_dtype=self.dtype,
+                                      gate=ops.columns(down, self.gate_offset, self.heads * self.vdim))
+        else:
+            values = ops.head_product(mixed, p['v_up.weight'], heads=self.heads, out_dtype=self.dtype)
         return ops.linear(values, p['o_proj.weight'], None, partials=True)

@@ -1,4 +1,4 @@
-"""A routed feed-forward: a router chooses a few experts per token, each a small gated feed-forward."""
+"""A routed feed-forward: a router chooses a few experts per token, each a small feed-forward (gated or not)."""
 import torch
 
 from .base import FeedForward, ParamSpec
@@ -24,6 +24,9 @@ class RoutedExperts(FeedForward):
     ``shared``: a feed-forward part that every token passes and whose result is added to the routed sum (in float32,
     by one kernel); its tensors are this part's own under the prefix ``shared.``.
 
+    ``activation`` may name a function of ``ops.EXPERT_ACTIVATIONS``: the experts then have no gate branch, down(act(up x)),
+    and no gate tensors ([experts, 1, ff, width] below).
+
     The experts' matrices are stacked at ``finalize`` into [experts, 2, ff, width] (gate rows, then up rows) and
     [experts, width, ff], ff padded with zeros to a multiple of 16 (a zero gate and up row give act = 0, which meets a
     zero column of the down matrix): pure re-layouts.
@@ -42,7 +45,8 @@ class RoutedExperts(FeedForward):
         outputs = experts + identity
         if outputs % groups or keep > groups or top > keep * (outputs // groups):
             raise ValueError(f'{outputs} router outputs do not split into {groups} groups of which {keep} hold {top} choices')
-        if activation not in ops.GATE_FUNCTIONS:
+        self.gated = activation in ops.GATE_FUNCTIONS
+        if not self.gated and activation not in ops.EXPERT_ACTIVATIONS:
             raise ValueError(f'no kernel for activation {activation!r}')
         if activation == 'clamped_swish' and not (limit is not None and limit > 0):
             raise ValueError('clamped_swish needs a positive limit')
@@ -70,7 +74,8 @@ class RoutedExperts(FeedForward):
         if self.correction:
             specs['router.correction'] = ParamSpec((self.outputs,), 'vector')
         for e in range(self.experts):
-            specs[f'experts.{e}.gate_proj.weight'] = ParamSpec((self.intermediate, self.width))
+            if self.gated:
+                specs[f'experts.{e}.gate_proj.weight'] = ParamSpec((self.intermediate, self.width))
             specs[f'experts.{e}.up_proj.weight'] = ParamSpec((self.intermediate, self.width))
             specs[f'experts.{e}.down_proj.weight'] = ParamSpec((self.width, self.intermediate))
         if self.shared is not None:
@@ -82,12 +87,13 @@ class RoutedExperts(FeedForward):
             self.shared.finalize()
         p = self.p
         ff, padded = self.intermediate, -(-self.intermediate // 16) * 16
-        first = p['experts.0.gate_proj.weight']
-        gate_up = first.new_zeros((self.experts, 2, padded, self.width))
+        first = p['experts.0.up_proj.weight']
+        gate_up = first.new_zeros((self.experts, 2 if self.gated else 1, padded, self.width))
         down = first.new_zeros((self.experts, self.width, padded))
         for e in range(self.experts):
-            gate_up[e, 0, :ff].copy_(p.pop(f'experts.{e}.gate_proj.weight'))
-            gate_up[e, 1, :ff].copy_(p.pop(f'experts.{e}.up_proj.weight'))
+            if self.gated:
+                gate_up[e, 0, :ff].copy_(p.pop(f'experts.{e}.gate_proj.weight'))
+            gate_up[e, -1, :ff].copy_(p.pop(f'experts.{e}.up_proj.weight'))
             down[e, :, :ff].copy_(p.pop(f'experts.{e}.down_proj.weight'))
         p['experts.gate_up_proj.weight'], p['experts.down_proj.weight'] = gate_up, down
 

@@ -1,4 +1,5 @@
-"""Norms with float32 statistics: RMSNorm (formula: qil/model.py:15-23) and a layer norm with or without a bias."""
+"""Norms with float32 statistics: RMSNorm (formula: qil/model.py:15-23) and a layer norm with or without a bias; and a
+hyperbolic tangent in a norm's place, which has no statistics."""
 import torch
 
 from .base import Norm, ParamSpec
@@ -65,3 +66,29 @@ class LayerNorm(Norm):
     def forward_rows(self, stream, delta, rows, out_dtype, delta_scale=1.0):
         return ops.rows_norm(stream, delta, rows, self.p['weight'], self.eps, out_dtype, centre=True,
                              delta_scale=delta_scale, bias=self.p.get('bias'))
+
+
+class TanhNorm(Norm):
+    """y = tanh(alpha * x) * weight + bias, element by element, ``alpha`` one stored number; float32 and one rounding.
+    ``streams``: the number of residual streams whose sum the norm of selected rows reads (a model's last norm)."""
+
+    def __init__(self, width, streams=1):
+        super().__init__()
+        ops.check_streams(streams)
+        self.width, self.streams = int(width), streams
+
+    def param_specs(self):
+        return {'weight': ParamSpec((self.width,), 'vector', 'one_plus_normal'), 'bias': ParamSpec((self.width,), 'vector'),
+                'alpha': ParamSpec((), 'vector', 'one_plus_normal')}
+
+    def _tensors(self):
+        return self.p['alpha'], self.p['weight'], self.p['bias']
+
+    def forward(self, stream, delta, out_dtype):
+        return ops.stream_join(stream, delta, streams=1, norm=self._tensors(), out_dtype=out_dtype)
+
+    def forward_streams(self, stream, pending, out_dtype, *, streams, read):
+        return ops.stream_join(stream, pending, streams=streams, read=read, norm=self._tensors(), out_dtype=out_dtype)
+
+    def forward_rows(self, stream, delta, rows, out_dtype):
+        return ops.stream_join(stream, delta, streams=self.streams, rows=rows, norm=self._tensors(), out_dtype=out_dtype)
