@@ -19,8 +19,82 @@ def _round(x, dtype):
     return x.to(dtype).to(torch.float32)
 
 
-def embed(token_ids, table, scale=1.0):
-    return table[token_ids.long()].to(torch.float32) * scale
+def embed(token_ids, table, scale=1.0, streams=1):
+    return (table[token_ids.long()].to(torch.float32) * scale).repeat(1, streams)
+
+
+def stream_join(stream, pending, *, streams, out_dtype, read=None, norm=None, rows=None):
+    n = stream.shape[0]
+    x = stream.view(n, streams, -1)
+    if pending is not None:
+        update = hasattr(pending, 'mix')
+        value = pending.value if update else pending
+        value = (value.materialize() if hasattr(value, 'materialize') else _value(value)).to(torch.float32)[:, None, :]
+        x = torch.einsum('st,nsw->ntw', pending.mix, x) + pending.out[None, :, None] * value if update else x + value
+    if rows is None:
+        stream.copy_(x.reshape(n, -1))
+    else:
+        x = x[rows.long()]
+    u = (x * read[None, :, None]).sum(1) if read is not None else x.sum(1)
+    if norm is not None:
+        alpha, weight, bias = norm
+        u = torch.tanh(alpha * u) * weight + bias
+    return u.to(out_dtype)
+
+
+def pair_store(qkv, *, heads, kv_heads, dim, vdim, padded, slots, k_cache, v_cache, page_size, dtype):
+    x = _value(qkv)
+    n = x.shape[0]
+    q = torch.zeros(n, heads, 2, padded)
+    given = x[:, :heads * 2 * dim].to(torch.float32).reshape(n, heads, 2, dim)
+    q[:, :, 0, :dim], q[:, :, 1, dim:2 * dim] = given[:, :, 0], given[:, :, 1]
+    if slots is not None:
+        at = heads * 2 * dim
+        k, v = torch.zeros(n, kv_heads, padded), torch.zeros(n, kv_heads, padded)
+        k[..., :2 * dim] = x[:, at:at + kv_heads * 2 * dim].reshape(n, kv_heads, 2 * dim)
+        at += kv_heads * 2 * dim
+        v[..., :vdim] = x[:, at:at + kv_heads * vdim].reshape(n, kv_heads, vdim)
+        page, offset = slots.long() // page_size, slots.long() % page_size
+        k_cache[page, :, offset] = k.to(dtype)
+        v_cache[page, :, :, offset] = v.to(dtype)
+    return q.reshape(n, -1).to(dtype)
+
+
+def difference_combine(maps, gate, *, heads, vdim, padded, factor, post, eps, dtype):
+    maps = maps.merge() if hasattr(maps, 'merge') else maps
+    n = maps.shape[0]
+    a = maps.to(torch.float32).reshape(n, heads, 2, padded)[..., :vdim]
+    o = a[:, :, 0] - factor * a[:, :, 1]
+    o = o / torch.sqrt(o.square().mean(dim=-1, keepdim=True) + eps) * post
+    return (o * torch.sigmoid(_value(gate).to(torch.float32))[:, :, None]).reshape(n, -1).to(dtype)
+
+
+def delta_rule(u, decays, steps, *, heads, kv_heads, dim, vdim, q_offset, k_offset, v_offset, decay_bias, rates, state, cu_seqlens,
+               seq_starts, seq_slots, n_seqs, gate, weight, eps, max_query=None, tile_seqs=None, accumulate=torch.float32):
+    """Token by token, whatever ``max_query`` says."""
+    n = u.shape[0]
+    x = u.to(accumulate)
+    share = torch.arange(heads) // (heads // kv_heads)
+    unit = lambda t: t / torch.sqrt(t.square().sum(dim=-1, keepdim=True) + 1e-6)
+    q = unit(x[:, q_offset:q_offset + kv_heads * dim].reshape(n, kv_heads, dim))[:, share] * dim ** -0.5
+    k = unit(x[:, k_offset:k_offset + kv_heads * dim].reshape(n, kv_heads, dim))[:, share]
+    v = x[:, v_offset:v_offset + heads * vdim].reshape(n, heads, vdim)
+    soft = torch.nn.functional.softplus(_value(decays).to(accumulate) + decay_bias, threshold=20.0).reshape(n, heads, dim)
+    keep = torch.exp(rates.to(accumulate)[None, :, None] * soft)
+    beta = torch.sigmoid(_value(steps).to(accumulate))
+    o = torch.zeros(n, heads, vdim, dtype=accumulate)
+    for s in range(n_seqs):
+        slot = int(seq_slots[s])
+        S = state[slot].view(heads, dim, vdim).to(accumulate) if int(seq_starts[s]) > 0 else torch.zeros(heads, dim, vdim, dtype=accumulate)
+        for t in range(int(cu_seqlens[s]), int(cu_seqlens[s + 1])):
+            S = keep[t][:, :, None] * S
+            w = beta[t][:, None] * (v[t] - torch.einsum('hdv,hd->hv', S, k[t]))
+            S = S + k[t][:, :, None] * w[:, None, :]
+            o[t] = torch.einsum('hdv,hd->hv', S, q[t])
+        if int(cu_seqlens[s + 1]) > int(cu_seqlens[s]):
+            state[slot] = S.reshape(-1).to(torch.float32)
+    o = o / torch.sqrt(o.square().mean(dim=-1, keepdim=True) + eps) * weight
+    return (o.reshape(n, -1) * torch.sigmoid(_value(gate).to(accumulate))).to(u.dtype)
 
 
 def _norm(x, weight, eps, out_dtype):
@@ -298,9 +372,11 @@ def latent_prepare(down, *, q_rank, rank, rot, q_weight, c_weight, eps, frequenc
     return (cq, torch.sigmoid(x[:, q_rank + rank + rot:])) if gates else cq
 
 
-def head_product(x, weight, *, heads, out_dtype, out=None, out_columns=None):
+def head_product(x, weight, *, heads, out_dtype, out=None, out_columns=None, gate=None):
     n, k, o = x.shape[0], weight.shape[1], weight.shape[2]
     result = torch.einsum('nhk,hko->nho', x.to(torch.float32).view(n, heads, -1)[:, :, :k], weight.to(torch.float32))
+    if gate is not None:
+        result = result * torch.sigmoid(_value(gate).to(torch.float32)).view(n, heads, o)
     if out is None:
         return result.reshape(n, heads * o).to(out_dtype)
     out.view(n, heads, out_columns)[:, :, :o] = result.to(out_dtype)
@@ -491,8 +567,9 @@ def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alp
             if e >= experts:
                 out[row] += weights[row, slot] * xf[row]
                 continue
-            g, u = gate_up[e, 0].to(torch.float32) @ xf[row], gate_up[e, 1].to(torch.float32) @ xf[row]
-            hidden = _round(_gate(g, u, activation, limit, alpha), x.dtype)
+            g, u = gate_up[e, 0].to(torch.float32) @ xf[row], gate_up[e, -1].to(torch.float32) @ xf[row]
+            hidden = u.clamp(min=0.0) ** 2 if activation == 'relu_squared' else _gate(g, u, activation, limit, alpha)
+            hidden = _round(hidden, x.dtype)
             out[row] += weights[row, slot] * (down[e].to(torch.float32) @ hidden)
     return out
 
@@ -517,7 +594,8 @@ def check_selective_scan_geometry(*, inner, state, taps):
 
 
 def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq_slots, row_seq, n_seqs, activation,
-                 out_dtype):
+                 out_dtype, pass_from=0, passed=0):
+    through = _value(x)[:, pass_from:pass_from + passed].to(out_dtype)
     x = _value(x)[:, :columns].to(torch.float32)
     taps, keep = weight.shape[0], weight.shape[0] - 1               # weight [taps, C]
     out = torch.empty_like(x)
@@ -535,7 +613,7 @@ def channel_conv(x, weight, bias, *, columns, state, cu_seqlens, seq_starts, seq
         out[first:last] = total * torch.sigmoid(total) if activation == 'silu' else total
         if keep:
             state[int(seq_slots[s])] = inputs[-keep:]
-    return out.to(out_dtype)
+    return (out.to(out_dtype), through) if passed else out.to(out_dtype)
 
 
 def selective_scan(u, dt, bc, gate, *, dt_bias, a, d, state, gate_offset, cu_seqlens, seq_starts, seq_slots, n_seqs,
@@ -564,4 +642,5 @@ ALL = dict(scaled_sum=scaled_sum, sigmoid_gate=sigmoid_gate, soft_cap=soft_cap, 
            latent_query=latent_query, latent_attention=latent_attention, state_scan_slot=state_scan_slot, state_scan=state_scan,
            head_norm_gate=head_norm_gate, plain_act=plain_act, post_norm_scale_add=post_norm_scale_add, short_conv=short_conv,
            qk_row_norm_store=qk_row_norm_store, gated_group_norm=gated_group_norm, embed_pairs=embed_pairs,
-           residual_join=residual_join)
+           residual_join=residual_join, stream_join=stream_join, pair_store=pair_store, difference_combine=difference_combine,
+           delta_rule=delta_rule)

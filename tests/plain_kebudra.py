@@ -219,9 +219,12 @@ def make_config(layers, *, vocab, width, streams, eps=1e-5, embedding_scale=1.0)
                 layers=layers, norm=dict(eps=eps))
 
 
-def random_weights(config, seed, spread=1.0, ranks=(5, 11)):
+def random_weights(config, seed, spread=1.0, ranks=(5, 11), clear_routers=False):
     """float64 tensors whose values bfloat16 holds exactly, by checkpoint name.  ``ranks``: inner sizes of the low-rank
-    products of the decays and of the gate."""
+    products of the decays and of the gate.  ``clear_routers``: no router is ever close to choosing otherwise (for engines that
+    round: an expert more or less is no rounding error).  Every token then has one of 16 sign patterns in the last four
+    channels, which no sub-layer writes to and which the routers read alone, and the routers are drawn until every pattern's
+    choice is clear."""
     g = torch.Generator().manual_seed(seed)
     width, streams = config['width'], config['streams']
     w = {}
@@ -295,6 +298,25 @@ def random_weights(config, seed, spread=1.0, ranks=(5, 11)):
             for e in range(f['router']['experts']):
                 matrix(p + f'e{e}.up', f['expert']['ff'], width)
                 matrix(p + f'e{e}.down', width, f['expert']['ff'], 1.5)
+    if clear_routers:
+        signs = torch.tensor([[1.0 if token >> bit & 1 else -1.0 for bit in range(4)] for token in range(config['vocab'])], dtype=F)
+        w['embed'][:, -4:] = held(3.0 / config['embedding']['scale'] * signs)
+        for name in w:
+            if name.endswith('.mix.o') or name.endswith('.down'):
+                w[name][-4:] = 0.0
+            elif name.endswith('.norm2'):
+                w[name][-4:], w[name + '.b'][-4:] = 1.0, 0.0
+        for i, layer in enumerate(config['layers']):
+            if layer['mlp'] is None:
+                continue
+            r = layer['mlp']['router']
+            while True:
+                router = held(normal(r['experts'], 4))
+                z = (signs[:16] @ router.T).sort(dim=-1, descending=True).values
+                if r['top'] == r['experts'] or (z[:, r['top'] - 1] - z[:, r['top']]).min() > 0.12:
+                    break
+            w[f'l{i}.mlp.router'] = torch.zeros(r['experts'], width, dtype=F)
+            w[f'l{i}.mlp.router'][:, -4:] = router
     return w
 
 
