@@ -309,6 +309,30 @@ def tinuzen_config(z, layers, vocab, window, kind='turns'):
     return out
 
 
+def kebudra_config(z, layers, vocab, kind='turns'):
+    """`layers` layers of the Kebudra design with four residual streams, a routed feed-forward behind each (32 experts
+    without a gate branch of which 4 are chosen, three eighths of the gated feed-forward's inner size each: a token's
+    experts have its weights): the delta rule with a decay per key channel (heads of 128 x 128, a state as large as that of the
+    other designs' memories), attention as the difference of two maps (two queries and two keys of half a head's size a
+    head), latent attention at the sizes of Fubapel's, or the three in turns (the second difference layer of six reads the
+    first one's cache)."""
+    moe = dict(kind='moe', expert=dict(ff=z['ff'] * 3 // 8), router=dict(experts=32, top=4))
+    heads = max(1, z['memory_heads'] * z['memory_vdim'] // 128)
+    delta = dict(type='channel_delta', mlp=moe, mixer=dict(heads=heads, kv_heads=heads, dim=128, vdim=128, conv=4))
+    difference = dict(type='attention', mlp=moe,
+                      mixer=dict(heads=z['heads'], kv_heads=max(1, z['heads'] // 4), dim=z['dim'] // 2, vdim=z['dim'],
+                                 scale=(z['dim'] // 2) ** -0.5, diff=0.5))
+    latent = dict(type='latent_attention', mlp=moe,
+                  mixer=dict(heads=z['heads'], dim=z['dim'], rot_dim=z['rot_dim'], vdim=z['dim'], kv_rank=z['kv_rank'], q_rank=z['q_rank'],
+                             rot=dict(base=10000.0, dims=z['rot_dim']), scale=(z['dim'] + z['rot_dim']) ** -0.5))
+    kinds = dict(turns=[delta, difference, latent], delta=[delta], difference=[difference], latent=[latent])[kind]
+    made = [kinds[i % len(kinds)] for i in range(layers)]
+    if kind == 'turns' and layers >= 5:
+        made[4] = dict(difference, mixer=dict(difference['mixer'], kv_from=1))
+    return dict(architecture='Kebudra', vocab=vocab, width=z['width'], streams=4, embedding=dict(scale=z['width'] ** 0.5),
+                layers=made, norm=dict(eps=1e-6))
+
+
 def designs_phase(args, torch, dtype):
     """Prefill tokens a second and decode milliseconds a step of a design's models whose layers are all of one kind
     (and of its kinds in turns), beside dense Qwen3 of the same width, feed-forward, depth and attention heads."""
@@ -344,6 +368,15 @@ def designs_phase(args, torch, dtype):
         models['dogozen (window beside a scan)'] = dogozen_config(z, layers, vocab, args.design_window, 'parallel')
         models['dogozen (gated attention)'] = dogozen_config(z, layers, vocab, args.design_window, 'attention')
         models['fubapel (decaying memory only)'] = dict(fubapel_config(z, layers, vocab), layers=[fubapel_config(z, 3, vocab)['layers'][2]] * layers)
+    elif args.design == 'kebudra':
+        # beside it the closest models of the engine: Gerivik's memory with a decay per row (a matrix state of the same size
+        # per layer, a routed feed-forward), its attention, and Fubapel's latent attention
+        names = (('turns', 'kinds in turns'), ('delta', 'delta rule'), ('difference', 'difference of two maps'), ('latent', 'latent attention'))
+        models = {f'kebudra ({name})': kebudra_config(z, layers, vocab, kind) for kind, name in names}
+        gerivik = gerivik_config(z, layers, vocab)
+        for index, name in enumerate(('gated linear attention', 'capped attention')):
+            models[f'gerivik ({name} only)'] = dict(gerivik, layers=[gerivik['layers'][index]] * layers)
+        models['fubapel (latent attention only)'] = dict(fubapel_config(z, layers, vocab), layers=[fubapel_config(z, 1, vocab)['layers'][0]] * layers)
     elif args.design == 'gerivik':
         mixed = gerivik_config(z, layers, vocab)
         models = {'gerivik (kinds in turns)': mixed}
@@ -425,7 +458,7 @@ def main():
                              'attention kernels alone, at the reference\'s own shapes and at the benchmark\'s.  products: a layer\'s '
                              'matrix products at --prefill-tokens rows alone, GPU BLAS against own kernel.  designs: prefill and decode of the '
                              'design named by --design at --design-sizes beside dense Qwen3 of equal sizes (--layers, default 6)')
-    parser.add_argument('--design', default='fubapel', choices=['fubapel', 'gerivik', 'zinesun', 'dogozen', 'tinuzen'], help='the design of --phase designs')
+    parser.add_argument('--design', default='fubapel', choices=['fubapel', 'gerivik', 'zinesun', 'dogozen', 'tinuzen', 'kebudra'], help='the design of --phase designs')
     parser.add_argument('--design-window', type=int, default=512, help='the attention window of --design zinesun, dogozen and tinuzen')
     parser.add_argument('--design-only', default=None, help='of the models of --phase designs, only those whose name holds this (for profiling)')
     parser.add_argument('--design-sizes', default='1b', choices=sorted(DESIGN_SIZES), help='layer sizes of --phase designs')

@@ -23,7 +23,11 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 #define DC_L 64                                            // tokens a chunk
 #define DC_THREADS 512
-#define DC_A_ROW 20                                        // floats between two rows of a 16 x 16 block in LDS
+#define DC_BLOCK 256                                       // floats of a 16 x 16 block in LDS
+
+// Where row i, column j of such a block lies: rows of 16 floats, their pieces of four turned so that the 16 rows a fragment
+// read touches fall on all banks.
+__device__ __forceinline__ int dc_in_block(int i, int j) { return i * 16 + ((((j >> 2) ^ (i >> 2)) & 3) << 2) + (j & 3); }
 
 __device__ __forceinline__ f32x4 dc_ld(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
 __device__ __forceinline__ f32x4 dc_ld(const bf16_t* p) { const float4 v = ld4(p); return (f32x4){v.x, v.y, v.z, v.w}; }
@@ -34,6 +38,18 @@ __device__ __forceinline__ f32x4 dc_mma(const f32x4& a, const f32x4& b, f32x4 ac
 }
 __device__ __forceinline__ float dc_exp2(float v) { return __builtin_amdgcn_exp2f(v); }
 
+// ln(1 + e^v) = max(v, 0) + ln(1 + t), t = e^(-|v|), with the hardware's exponential and logarithm; a small t by its series (the
+// logarithm of 1 + t would lose it).
+__device__ __forceinline__ float dc_softplus(float v) {
+  const float t = dc_exp2(-fabsf(v) * 1.44269504088896f);
+  const float series = t * (1.f - t * (0.5f - t * (0.33333333f - t * 0.25f)));
+  return fmaxf(v, 0.f) + (t < 0.015f ? series : __builtin_amdgcn_logf(1.f + t) * 0.69314718055995f);
+}
+
+// A barrier for what went through LDS: the waves' loads from memory stay on their way (the compiler's barrier would wait
+// for them as well).
+__device__ __forceinline__ void dc_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // Where chunk c of sequence seq keeps its operands: sequences before it took at most row0 / DC_L + seq places.
 __device__ __forceinline__ size_t dc_place(int row0, int seq, int c) { return (size_t)(row0 / DC_L + seq + c); }
 
@@ -42,7 +58,7 @@ __host__ __device__ __forceinline__ size_t dc_cell(int dp, int vp) { return (siz
 
 // grid (chunks of the longest sequence, sequences x heads), 8 waves.
 template <typename T, int DP>
-__global__ void __launch_bounds__(DC_THREADS)
+__global__ void __launch_bounds__(DC_THREADS, DP <= 128 ? 4 : 2)
 delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* __restrict__ scratch, int heads, int kv_heads,
                      int dim, int vdim, int vp) {
   constexpr int KROW = DP + 16 / (int)sizeof(T), LROW = DP + 4;
@@ -51,7 +67,7 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
   T* ks = reinterpret_cast<T*>(L + DC_L * LROW);           // [64][KROW]
   T* qs = ks + DC_L * KROW;
   float* A = reinterpret_cast<float*>(qs + DC_L * KROW);   // [10] blocks of -A (b >= j: b (b + 1) / 2 + j), the diagonal ones then inverted
-  float* units = A + 10 * 16 * DC_A_ROW;                   // [3][64]: 1 / |k|, dim^(-1/2) / |q|, beta
+  float* units = A + 10 * DC_BLOCK;                   // [3][64]: 1 / |k|, dim^(-1/2) / |q|, beta
   const int c = blockIdx.x, seq = blockIdx.y / heads, h = blockIdx.y % heads;
   const int row0 = cu_seqlens[seq], len = cu_seqlens[seq + 1] - row0;
   if (c * DC_L >= len) return;
@@ -72,27 +88,37 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
     const T* k = x + in.k_off + shared_head * dim;
     const T* q = x + in.q_off + shared_head * dim;
     float kk = 0.f, qq = 0.f;
-    for (int e0 = part * 4; e0 < DP; e0 += 32) {
-      float kv[4], qv[4];
+    constexpr int PIECES = DP / 32;
+    float4 kv[PIECES], qv[PIECES];
+    if (dim % 4 == 0) {                                    // (the host checked that rows and offsets are multiples of 4)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) { kv[e] = 0.f; qv[e] = 0.f; }
-      if (t < lc) {
-        if (dim % 4 == 0) {                                // (the host checked that rows and offsets are multiples of 4)
-          if (e0 < dim) {
-            const f32x4 a = dc_ld(k + e0), b = dc_ld(q + e0);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) { kv[e] = a[e]; qv[e] = b[e]; }
-          }
-        } else {
-#pragma unroll
-          for (int e = 0; e < 4; ++e)
-            if (e0 + e < dim) { kv[e] = ld(k + e0 + e); qv[e] = ld(q + e0 + e); }
-        }
+      for (int n = 0; n < PIECES; ++n) {
+        const int e0 = min(part * 4 + n * 32, dim - 4);
+        kv[n] = ld4(k + e0);
+        qv[n] = ld4(q + e0);
       }
-      st4(ks + t * KROW + e0, make_float4(kv[0], kv[1], kv[2], kv[3]));
-      st4(qs + t * KROW + e0, make_float4(qv[0], qv[1], qv[2], qv[3]));
+    } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) { kk += kv[e] * kv[e]; qq += qv[e] * qv[e]; }
+      for (int n = 0; n < PIECES; ++n) {
+        float v[2][4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int at = part * 4 + n * 32 + e;
+          v[0][e] = at < dim ? ld(k + at) : 0.f;
+          v[1][e] = at < dim ? ld(q + at) : 0.f;
+        }
+        kv[n] = make_float4(v[0][0], v[0][1], v[0][2], v[0][3]);
+        qv[n] = make_float4(v[1][0], v[1][1], v[1][2], v[1][3]);
+      }
+    }
+#pragma unroll
+    for (int n = 0; n < PIECES; ++n) {
+      const int e0 = part * 4 + n * 32;
+      if (t >= lc || e0 >= dim) kv[n] = qv[n] = make_float4(0.f, 0.f, 0.f, 0.f);
+      st4(ks + t * KROW + e0, kv[n]);
+      st4(qs + t * KROW + e0, qv[n]);
+      kk += kv[n].x * kv[n].x + kv[n].y * kv[n].y + kv[n].z * kv[n].z + kv[n].w * kv[n].w;
+      qq += qv[n].x * qv[n].x + qv[n].y * qv[n].y + qv[n].z * qv[n].z + qv[n].w * qv[n].w;
     }
 #pragma unroll
     for (int o = 1; o < 8; o <<= 1) { kk += __shfl_xor(kk, o, QIL_WAVE); qq += __shfl_xor(qq, o, QIL_WAVE); }
@@ -102,15 +128,31 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
       units[2 * DC_L + t] = t < lc ? delta_step_size(in, r0 + t, h) : 0.f;
     }
   }
-  for (int item = tid; item < DP * 4; item += DC_THREADS) {    // a thread a channel and block of 16 tokens
-    const int ch = item % DP, b = item / DP;
+  for (int item = tid; item < DP * 4; item += DC_THREADS) {    // a thread a channel and block of 16 tokens, all loads first
+    const int ch = item % DP, b = item / DP, own = min(ch, dim - 1);
     float raw[16], sum = 0.f;
+    const size_t first = (size_t)r0 * in.z_row + h * dim + own;
+    int at[16];
 #pragma unroll
-    for (int t = 0; t < 16; ++t)
-      raw[t] = ch < dim && b * 16 + t < lc ? delta_log_decay(in, r0 + b * 16 + t, h, dim, ch) : 0.f;
+    for (int t = 0; t < 16; ++t) at[t] = min(b * 16 + t, lc - 1) * in.z_row;
+    if (in.z.code == QIL_BF16) {
+      const bf16_t* base = reinterpret_cast<const bf16_t*>(in.z.data) + first;
+#pragma unroll
+      for (int t = 0; t < 16; ++t) raw[t] = ld(base + at[t]);
+    } else {
+      const float* base = reinterpret_cast<const float*>(in.z.data) + first;
+#pragma unroll
+      for (int t = 0; t < 16; ++t) raw[t] = base[at[t]];
+      for (int split = 1; split < in.z.splits; ++split) {
+        base += in.z.stride;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) raw[t] += base[at[t]];
+      }
+    }
+    const float bias = in.bias[h * dim + own], rate = in.rates[h] * 1.44269504088896f;
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-      sum += raw[t] * 1.44269504088896f;
+      if (ch < dim && b * 16 + t < lc) sum += rate * dc_softplus(raw[t] + bias);
       L[(b * 16 + t) * LROW + ch] = sum;
     }
   }
@@ -134,11 +176,11 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
         }
       }
     }
-    float* a = A + (b * (b + 1) / 2 + b) * 16 * DC_A_ROW;
+    float* a = A + (b * (b + 1) / 2 + b) * DC_BLOCK;
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
       const float uk = units[j + p];
-      a[(i - b * 16) * DC_A_ROW + j + p - b * 16] = i > j + p ? -kk[p] * units[i] * uk * units[2 * DC_L + i] : 0.f;
+      a[dc_in_block(r, j + p - b * 16)] = i > j + p ? -kk[p] * units[i] * uk * units[2 * DC_L + i] : 0.f;
       B[i * DC_L + j + p] = i >= j + p ? qk[p] * units[DC_L + i] * uk : 0.f;
     }
   }
@@ -162,30 +204,34 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
       kk = dc_mma(ki, kj, kk);
       qk = dc_mma(qi, kj, qk);
     }
-    float* a = A + (bi * (bi + 1) / 2 + bj) * 16 * DC_A_ROW;
+    float* a = A + (bi * (bi + 1) / 2 + bj) * DC_BLOCK;
     const float uk = units[bj * 16 + r];
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = bi * 16 + 4 * kb + e;
-      a[(4 * kb + e) * DC_A_ROW + r] = -kk[e] * units[i] * uk * units[2 * DC_L + i];
+      a[dc_in_block(4 * kb + e, r)] = -kk[e] * units[i] * uk * units[2 * DC_L + i];
       B[i * DC_L + bj * 16 + r] = qk[e] * units[DC_L + i] * uk;
     }
   }
   __syncthreads();
   if (wave < 4) {                                          // (I + A_bb)^(-1), a column a lane: x_i = delta_ij - sum_(m < i) A_im x_m
-    float* a = A + (wave * (wave + 1) / 2 + wave) * 16 * DC_A_ROW;
+    float* a = A + (wave * (wave + 1) / 2 + wave) * DC_BLOCK;
     float x[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float v = i == r ? 1.f : 0.f;
 #pragma unroll
-      for (int m = 0; m < i; ++m) v += a[i * DC_A_ROW + m] * x[m];
+      for (int m0 = 0; m0 < i; m0 += 4) {
+        const f32x4 row = dc_ld(a + dc_in_block(i, m0));
+#pragma unroll
+        for (int m = m0; m < i && m < m0 + 4; ++m) v += row[m - m0] * x[m];
+      }
       x[i] = v;
     }
     // (a wave's LDS operations are in order: every lane has read the block before any lane writes it)
     if (lane < 16) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) a[i * DC_A_ROW + r] = x[i];
+      for (int i = 0; i < 16; ++i) a[dc_in_block(i, r)] = x[i];
     }
   }
   __syncthreads();
@@ -208,8 +254,8 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
       }
       if (is_w) before += L[(b * 16 + 15) * LROW + col];
 #pragma unroll
-      for (int j = 0; j < b; ++j) acc = dc_mma(dc_ld(A + ((b * (b + 1) / 2 + j) * 16 + r) * DC_A_ROW + 4 * kb), x[j], acc);
-      x[b] = dc_mma(dc_ld(A + ((b * (b + 1) / 2 + b) * 16 + r) * DC_A_ROW + 4 * kb), acc, (f32x4){0.f, 0.f, 0.f, 0.f});
+      for (int j = 0; j < b; ++j) acc = dc_mma(dc_ld(A + (b * (b + 1) / 2 + j) * DC_BLOCK + dc_in_block(r, 4 * kb)), x[j], acc);
+      x[b] = dc_mma(dc_ld(A + (b * (b + 1) / 2 + b) * DC_BLOCK + dc_in_block(r, 4 * kb)), acc, (f32x4){0.f, 0.f, 0.f, 0.f});
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int t = b * 16 + 4 * kb + e;
@@ -219,12 +265,14 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
     }
   }
   // the queries with their decays from the chunk's start, the keys with theirs to its end (transposed), the whole decay
+#pragma unroll 4
   for (int item = tid; item < DC_L * DP; item += DC_THREADS) {
     const int t = item / DP, ch = item % DP;
     float from = L[t * LROW + ch];
     for (int m = 0; m < (t >> 4); ++m) from += L[(m * 16 + 15) * LROW + ch];
     Q[item] = ld(qs + t * KROW + ch) * units[DC_L + t] * dc_exp2(from);
   }
+#pragma unroll 4
   for (int item = tid; item < DC_L * DP; item += DC_THREADS) {
     const int t = item % DC_L, ch = item / DC_L;
     float upto = L[((t >> 4) * 16 + 15) * LROW + ch] - L[t * LROW + ch];
@@ -248,7 +296,8 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
   const int seq = blockIdx.x / heads, h = blockIdx.x % heads, j0 = blockIdx.y * 16;
   const int row0 = cu_seqlens[seq], len = cu_seqlens[seq + 1] - row0;
   if (len <= 0) return;
-  const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE, r = lane & 15, kb = lane >> 4;
+  const int lane = threadIdx.x & (QIL_WAVE - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / QIL_WAVE);
+  const int r = lane & 15, kb = lane >> 4;
   const bool column = j0 + r < vdim;
   float* mine = slots + ((size_t)seq_slots[seq] * heads + h) * dim * vdim + j0 + r;
   const bool fresh = seq_starts[seq] == 0;
@@ -279,8 +328,7 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
     for (int n = 0; n < DT; ++n) q[n] = dc_ld(p + DC_L * DP + t_row * DP + n * 16 + 4 * kb);
     const float* bo = p + 3 * DC_L * DP + DC_L * vp;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (j <= wave) b[j] = dc_ld(bo + t_row * DC_L + j * 16 + 4 * kb);
+    for (int j = 0; j < 4; ++j) b[j] = dc_ld(bo + t_row * DC_L + j * 16 + 4 * kb);      // (nobody wrote or uses those of j > wave)
   };
   auto load_k = [&](const float* p) {
     const float* eo = p + 3 * DC_L * DP + DC_L * vp + DC_L * DC_L;
@@ -294,7 +342,7 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
   load_w(at);
   load_q(at);
   load_k(at);
-  __syncthreads();
+  dc_barrier();
   for (int c = 0; c < chunks; ++c) {
     const float* next = at + (c + 1 < chunks ? stride : 0);
     f32x4 acc = write, acc2 = {0.f, 0.f, 0.f, 0.f};        // w = U - W S (two sums: the products of one wait for each other)
@@ -312,7 +360,7 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
       o = dc_mma(q[n], dc_ld(S + (n * 64 + lane) * 4), o);
       o2 = dc_mma(q[n + 1], dc_ld(S + ((n + 1) * 64 + lane) * 4), o2);
     }
-    __syncthreads();
+    dc_barrier();
 #pragma unroll
     for (int j = 0; j < 4; ++j)
       if (j <= wave) o = dc_mma(b[j], dc_ld(V + (j * 64 + lane) * 4), o);
@@ -334,7 +382,7 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
     load_k(next);
 #pragma unroll
     for (int n = 0; n < OWN; ++n) *reinterpret_cast<f32x4*>(S + ((wave + 4 * n) * 64 + lane) * 4) = s[n];   // (read before the barrier)
-    __syncthreads();
+    dc_barrier();
     at = next;
   }
 #pragma unroll
@@ -349,7 +397,7 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
 static int dc_padded(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : 256; }
 static size_t dc_lds(int dp, int dtype) {
   const size_t element = dtype == QIL_F32 ? 4 : 2;
-  return (size_t)DC_L * (dp + 4) * 4 + 2 * (size_t)DC_L * (dp + 16 / element) * element + 10 * 16 * DC_A_ROW * 4 + 3 * DC_L * 4;
+  return (size_t)DC_L * (dp + 4) * 4 + 2 * (size_t)DC_L * (dp + 16 / element) * element + 10 * DC_BLOCK * 4 + 3 * DC_L * 4;
 }
 
 extern "C" {

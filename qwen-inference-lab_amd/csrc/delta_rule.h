@@ -16,9 +16,9 @@ struct DeltaInputs {
 
 #define DELTA_UNIT_EPS 1e-6f                               // joins the sum of squares that makes unit vectors
 
+__device__ __forceinline__ float delta_softplus(float v) { return v > 20.f ? v : log1pf(expf(v)); }
 __device__ __forceinline__ float delta_log_decay(const DeltaInputs& in, int row, int h, int dim, int c) {
-  const float v = operand_at(in.z, (size_t)row * in.z_row + h * dim + c) + in.bias[h * dim + c];
-  return in.rates[h] * (v > 20.f ? v : log1pf(expf(v)));
+  return in.rates[h] * delta_softplus(operand_at(in.z, (size_t)row * in.z_row + h * dim + c) + in.bias[h * dim + c]);
 }
 __device__ __forceinline__ float delta_step_size(const DeltaInputs& in, int row, int h) {
   return 1.f / (1.f + expf(-operand_at(in.b, (size_t)row * in.b_row + h)));

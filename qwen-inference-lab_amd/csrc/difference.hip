@@ -78,52 +78,47 @@ pair_store_kernel(Operand x, size_t row_elems, T* __restrict__ q, const int* __r
   }
 }
 
-// A wave a (row, head): lanes 0 .. 31 take the first map's elements, lanes 32 .. 63 the second's, four at a time.
-// PARTS: the maps are the unmerged parts of a split context.
-template <typename T, bool PARTS>
+// A (row, head) takes 2 L lanes, the first L the first map's elements, the others the second's, eight a lane (L = 16 up to 128
+// elements, 32 up to 256): a lane and its partner L lanes away hold the same elements of both maps.  PARTS: the maps are the
+// unmerged parts of a split context.
+template <typename T, bool PARTS, int L>
 __global__ void __launch_bounds__(256)
 difference_combine_kernel(const T* __restrict__ maps, UnmergedA parts, Operand gate, size_t gate_row, float factor, float post,
                           float eps, T* __restrict__ out, int rows, int heads, int vdim, int padded, int vec_out) {
-  const int lane = threadIdx.x & (QIL_WAVE - 1);
-  const int item = blockIdx.x * (256 / QIL_WAVE) + threadIdx.x / QIL_WAVE;
-  if (item >= rows * heads) return;
-  const int row = item / heads, head = item - row * heads, map = lane >> 5, at = (lane & 31) * 4;
-  float o[2][4];                                            // padded <= 256: two rounds of 128 elements
+  const int item = blockIdx.x * (256 / (2 * L)) + threadIdx.x / (2 * L);
+  const bool there = item < rows * heads;                   // (every lane takes part in the exchanges)
+  const int row = there ? item / heads : 0, head = there ? item - row * heads : 0;
+  const int map = (threadIdx.x / L) & 1, e = (threadIdx.x % L) * 8;
+  const float g = operand_at(gate, (size_t)row * gate_row + head);
+  float v[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = 0.f;
+  if (e < padded) {
+    if constexpr (PARTS) merged_values<8>(parts, row, (head * 2 + map) * padded + e, v);
+    else ld8(maps + ((size_t)row * 2 * heads + head * 2 + map) * padded + e, v);
+  }
   float squares = 0.f;
 #pragma unroll
-  for (int round = 0; round < 2; ++round) {
-    const int e = round * 128 + at;
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    if (e < padded) {
-      if constexpr (PARTS) {
-        merged_values<4>(parts, row, (head * 2 + map) * padded + e, v);
-      } else {
-        const float4 a = ld4(maps + ((size_t)row * 2 * heads + head * 2 + map) * padded + e);
-        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
-      }
-    }
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float other = __shfl_xor(v[i], 32, QIL_WAVE);
-      const float d = map ? other - factor * v[i] : v[i] - factor * other;
-      o[round][i] = e + i < vdim ? d : 0.f;
-      squares += o[round][i] * o[round][i];
-    }
+  for (int i = 0; i < 8; ++i) {
+    const float other = __shfl_xor(v[i], L, QIL_WAVE);
+    const float d = map ? other - factor * v[i] : v[i] - factor * other;
+    v[i] = e + i < vdim ? d : 0.f;
+    squares += v[i] * v[i];
   }
-  squares = wave_sum(squares) * 0.5f;                       // (both halves hold the difference)
-  const float g = operand_at(gate, (size_t)row * gate_row + head);
+#pragma unroll
+  for (int o = 1; o < L; o <<= 1) squares += __shfl_xor(squares, o, QIL_WAVE);
   const float scale = post / sqrtf(squares / (float)vdim + eps) / (1.f + expf(-g));
-  // the first half of the wave stores round 0, the second half round 1
-  const int e = map * 128 + at;
-  T* to = out + ((size_t)row * heads + head) * vdim + e;
+  // both partners hold the difference: the first stores its first four elements, the second the last four
+  const int first = map * 4;
+  if (!there || e + first >= vdim) return;
+  T* to = out + ((size_t)row * heads + head) * vdim + e + first;
+  const float y[4] = {(map ? v[4] : v[0]) * scale, (map ? v[5] : v[1]) * scale, (map ? v[6] : v[2]) * scale, (map ? v[7] : v[3]) * scale};
   if (vec_out) {
-    if (e < vdim)
-      st4(to, make_float4((map ? o[1][0] : o[0][0]) * scale, (map ? o[1][1] : o[0][1]) * scale, (map ? o[1][2] : o[0][2]) * scale,
-                          (map ? o[1][3] : o[0][3]) * scale));
+    st4(to, make_float4(y[0], y[1], y[2], y[3]));
   } else {
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (e + i < vdim) st(to + i, (map ? o[1][i] : o[0][i]) * scale);
+      if (e + first + i < vdim) st(to + i, y[i]);
   }
 }
 
@@ -170,10 +165,17 @@ int qil_difference_combine(const void* maps, const float* workspace, const int* 
   }
   const Operand g{gate, gate_code, gate_splits, (size_t)rows * gate_row};
   const int vec_out = vdim % 4 == 0 && (uintptr_t)out % 16 == 0;
-  const dim3 grid((rows * heads + 3) / 4);
+  const int a_block = padded <= 128 ? 8 : 4;
+  const dim3 grid((rows * heads + a_block - 1) / a_block);
 #define QIL_DC(T, P)                                                                                                  \
-  hipLaunchKernelGGL((difference_combine_kernel<T, P>), grid, dim3(256), 0, s, (const T*)maps, u, g, (size_t)gate_row, factor, \
-                     post, eps, (T*)out, rows, heads, vdim, padded, vec_out)
+  do {                                                                                                                \
+    if (padded <= 128)                                                                                                \
+      hipLaunchKernelGGL((difference_combine_kernel<T, P, 16>), grid, dim3(256), 0, s, (const T*)maps, u, g, (size_t)gate_row, \
+                         factor, post, eps, (T*)out, rows, heads, vdim, padded, vec_out);                              \
+    else                                                                                                              \
+      hipLaunchKernelGGL((difference_combine_kernel<T, P, 32>), grid, dim3(256), 0, s, (const T*)maps, u, g, (size_t)gate_row, \
+                         factor, post, eps, (T*)out, rows, heads, vdim, padded, vec_out);                              \
+  } while (0)
   if (dtype == QIL_F32) { if (workspace) QIL_DC(float, true); else QIL_DC(float, false); }
   else { if (workspace) QIL_DC(bf16_t, true); else QIL_DC(bf16_t, false); }
 #undef QIL_DC

@@ -250,7 +250,35 @@ __device__ __forceinline__ typename Frag<T>::raw load_frag(const T* __restrict__
   return __builtin_bit_cast(typename Frag<T>::raw, e);
 }
 
-// grid (tiles, ceil(ff / 64)); a wave: the tile's rows by 16 gate and the same 16 up columns.
+// The same inside the row: no check.
+template <typename T, bool ALIGNED>
+__device__ __forceinline__ typename Frag<T>::raw load_inside(const T* __restrict__ at) {
+  if (ALIGNED) return *reinterpret_cast<const typename Frag<T>::raw*>(at);
+  T e[Frag<T>::EPL];
+#pragma unroll
+  for (int i = 0; i < Frag<T>::EPL; ++i) e[i] = at[i];
+  return __builtin_bit_cast(typename Frag<T>::raw, e);
+}
+
+// What a lane loads and what it multiplies are different places of a fragment: four neighbouring lanes load the four 16-byte
+// pieces of one row (lane 4 r + kq), so that a load touches a line of memory once; the matrix instruction wants row r's piece kq in
+// lane 16 kq + r (sixteen neighbouring lanes then ask for sixteen lines, and every load occupies the address path for 64
+// cycles: a block got 11 bytes a cycle).  The pieces change lanes in registers, by the data-parallel exchange that LDS's crossbar makes.
+template <typename T>
+__device__ __forceinline__ typename Frag<T>::raw to_operand(const typename Frag<T>::raw& loaded, int from) {
+  const qil_u32x4 in = __builtin_bit_cast(qil_u32x4, loaded);
+  qil_u32x4 out;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) out[i] = (uint32_t)__builtin_amdgcn_ds_bpermute(from, (int)in[i]);
+  return __builtin_bit_cast(typename Frag<T>::raw, out);
+}
+
+// Steps of K whose fragments are on their way while a step's products run: with few pairs (one tile of rows) the products
+// are few and the weights' way from memory is long.  The loads carry no condition (past the last whole step they repeat
+// it), or the compiler would wait for all of them at every use.
+template <int MT> struct Depth { static constexpr int of = MT == 1 ? 8 : 2; };
+
+// grid (tiles, column pieces of the block's waves); a wave: the tile's rows by 16 gate and the same 16 up columns.
 // w: [experts][2][ff][width] (an expert's gate rows, then its up rows).  hidden: [places][ff].
 template <typename T, int MT, bool ALIGNED>
 __global__ void __launch_bounds__(256)
@@ -262,41 +290,62 @@ moe_gate_up_kernel(const T* __restrict__ x, int width, const T* __restrict__ w, 
   if (rows == 0) return;
   const int e = tiles[tile], begin = tiles[max_tiles + tile];
   const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE;
-  const int col0 = (blockIdx.y * 4 + wave) * 16;
+  const int col0 = (blockIdx.y * (blockDim.x / QIL_WAVE) + wave) * 16;
   if (col0 >= ff) return;
-  const int r = lane & 15, kq = lane >> 4;
+  const int r = lane & 15, kq = lane >> 4, lr = lane >> 2, lq = lane & 3, from = (r * 4 + kq) * 4;
   const T* a_row[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
-    const int local = m * 16 + r;
+    const int local = m * 16 + lr;
     a_row[m] = x + (size_t)(places[begin + min(local, rows - 1)] / top) * width;
   }
-  const int col = min(col0 + r, ff - 1);
+  const int col = min(col0 + lr, ff - 1);
   const T* g_row = w + ((size_t)e * 2 * ff + col) * width;
   const T* u_row = g_row + (size_t)ff * width;
   moe_f32x4 acc_g[MT], acc_u[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) acc_g[m] = acc_u[m] = (moe_f32x4){0.f, 0.f, 0.f, 0.f};
-  // the fragments of the next step are on their way while this step's products run
-  typename Frag<T>::raw bg = load_frag<T, ALIGNED>(g_row, kq * EPL, width), bu = load_frag<T, ALIGNED>(u_row, kq * EPL, width);
-  typename Frag<T>::raw a[MT];
+  constexpr int DEPTH = Depth<MT>::of;
+  const int steps = width / KC;
+  typename Frag<T>::raw bg[DEPTH], bu[DEPTH], a[DEPTH][MT];
+  auto fetch = [&](int d, int step) {
+    const int k = min(step, steps - 1) * KC + lq * EPL;
+    bg[d] = load_inside<T, ALIGNED>(g_row + k);
+    bu[d] = load_inside<T, ALIGNED>(u_row + k);
 #pragma unroll
-  for (int m = 0; m < MT; ++m) a[m] = load_frag<T, ALIGNED>(a_row[m], kq * EPL, width);
-  for (int k0 = 0; k0 < width; k0 += KC) {
-    const int k = k0 + KC + kq * EPL;                    // (past the end: zeros, never used)
-    const typename Frag<T>::raw bg_next = load_frag<T, ALIGNED>(g_row, k, width), bu_next = load_frag<T, ALIGNED>(u_row, k, width);
-    typename Frag<T>::raw a_next[MT];
+    for (int m = 0; m < MT; ++m) a[d][m] = load_inside<T, ALIGNED>(a_row[m] + k);
+  };
+  if (steps > 0) {
 #pragma unroll
-    for (int m = 0; m < MT; ++m) a_next[m] = load_frag<T, ALIGNED>(a_row[m], k, width);
+    for (int d = 0; d < DEPTH; ++d) fetch(d, d);
+  }
+  for (int step = 0; step < steps; step += DEPTH) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      const typename Frag<T>::raw g = to_operand<T>(bg[d], from), u = to_operand<T>(bu[d], from);
+      typename Frag<T>::raw x_now[MT];
+#pragma unroll
+      for (int m = 0; m < MT; ++m) x_now[m] = to_operand<T>(a[d][m], from);
+      fetch(d, step + d + DEPTH);
+      if (step + d < steps) {
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+          Frag<T>::mma(acc_g[m], x_now[m], g);
+          Frag<T>::mma(acc_u[m], x_now[m], u);
+        }
+      }
+    }
+  }
+  if (steps * KC < width) {                                // what is left of K
+    const int k = steps * KC + lq * EPL;
+    const typename Frag<T>::raw g = to_operand<T>(load_frag<T, ALIGNED>(g_row, k, width), from);
+    const typename Frag<T>::raw u = to_operand<T>(load_frag<T, ALIGNED>(u_row, k, width), from);
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      Frag<T>::mma(acc_g[m], a[m], bg);
-      Frag<T>::mma(acc_u[m], a[m], bu);
+      const typename Frag<T>::raw x_now = to_operand<T>(load_frag<T, ALIGNED>(a_row[m], k, width), from);
+      Frag<T>::mma(acc_g[m], x_now, g);
+      Frag<T>::mma(acc_u[m], x_now, u);
     }
-    bg = bg_next;
-    bu = bu_next;
-#pragma unroll
-    for (int m = 0; m < MT; ++m) a[m] = a_next[m];
   }
   if (col0 + r >= ff) return;
 #pragma unroll
@@ -308,7 +357,7 @@ moe_gate_up_kernel(const T* __restrict__ x, int width, const T* __restrict__ w, 
     }
 }
 
-// grid (tiles, ceil(width / 128)); a wave: the tile's rows by 32 output columns.  w: [experts][width][ff].
+// grid (tiles, column pieces of the block's waves); a wave: the tile's rows by 32 output columns.  w: [experts][width][ff].
 // y: [pairs][width] float32, a pair's row at the pair's own index.
 // UP: the first product of experts without a gate branch: `hidden` are the rows of x (by the pair's token, of which there
 // are `top` pairs), ff their length, width the experts' inner size, and act(result) goes to the places' rows of `to`.
@@ -321,40 +370,62 @@ moe_down_kernel(const T* __restrict__ hidden, int ff, const T* __restrict__ w, i
   if (rows == 0) return;
   const int e = tiles[tile], begin = tiles[max_tiles + tile];
   const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE;
-  const int col0 = (blockIdx.y * 4 + wave) * 32;
+  const int col0 = (blockIdx.y * (blockDim.x / QIL_WAVE) + wave) * 32;
   if (col0 >= width) return;
-  const int r = lane & 15, kq = lane >> 4;
+  const int r = lane & 15, kq = lane >> 4, lr = lane >> 2, lq = lane & 3, from = (r * 4 + kq) * 4;
   const T* a_row[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
-    const int place = begin + min(m * 16 + r, rows - 1);
+    const int place = begin + min(m * 16 + lr, rows - 1);
     a_row[m] = hidden + (size_t)(UP ? places[place] / top : place) * ff;
   }
   const T* b_row[2];
 #pragma unroll
-  for (int t = 0; t < 2; ++t) b_row[t] = w + ((size_t)e * width + min(col0 + t * 16 + r, width - 1)) * ff;
+  for (int t = 0; t < 2; ++t) b_row[t] = w + ((size_t)e * width + min(col0 + t * 16 + lr, width - 1)) * ff;
   moe_f32x4 acc[MT][2];
 #pragma unroll
   for (int m = 0; m < MT; ++m) acc[m][0] = acc[m][1] = (moe_f32x4){0.f, 0.f, 0.f, 0.f};
-  typename Frag<T>::raw b0 = load_frag<T, ALIGNED>(b_row[0], kq * EPL, ff), b1 = load_frag<T, ALIGNED>(b_row[1], kq * EPL, ff);
-  typename Frag<T>::raw a[MT];
+  constexpr int DEPTH = Depth<MT>::of;
+  const int steps = ff / KC;
+  typename Frag<T>::raw b0[DEPTH], b1[DEPTH], a[DEPTH][MT];
+  auto fetch = [&](int d, int step) {
+    const int k = min(step, steps - 1) * KC + lq * EPL;
+    b0[d] = load_inside<T, ALIGNED>(b_row[0] + k);
+    b1[d] = load_inside<T, ALIGNED>(b_row[1] + k);
 #pragma unroll
-  for (int m = 0; m < MT; ++m) a[m] = load_frag<T, ALIGNED>(a_row[m], kq * EPL, ff);
-  for (int k0 = 0; k0 < ff; k0 += KC) {
-    const int k = k0 + KC + kq * EPL;
-    const typename Frag<T>::raw b0_next = load_frag<T, ALIGNED>(b_row[0], k, ff), b1_next = load_frag<T, ALIGNED>(b_row[1], k, ff);
-    typename Frag<T>::raw a_next[MT];
+    for (int m = 0; m < MT; ++m) a[d][m] = load_inside<T, ALIGNED>(a_row[m] + k);
+  };
+  if (steps > 0) {
 #pragma unroll
-    for (int m = 0; m < MT; ++m) a_next[m] = load_frag<T, ALIGNED>(a_row[m], k, ff);
+    for (int d = 0; d < DEPTH; ++d) fetch(d, d);
+  }
+  for (int step = 0; step < steps; step += DEPTH) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      const typename Frag<T>::raw first = to_operand<T>(b0[d], from), second = to_operand<T>(b1[d], from);
+      typename Frag<T>::raw x_now[MT];
+#pragma unroll
+      for (int m = 0; m < MT; ++m) x_now[m] = to_operand<T>(a[d][m], from);
+      fetch(d, step + d + DEPTH);
+      if (step + d < steps) {
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+          Frag<T>::mma(acc[m][0], x_now[m], first);
+          Frag<T>::mma(acc[m][1], x_now[m], second);
+        }
+      }
+    }
+  }
+  if (steps * KC < ff) {                                   // what is left of K
+    const int k = steps * KC + lq * EPL;
+    const typename Frag<T>::raw first = to_operand<T>(load_frag<T, ALIGNED>(b_row[0], k, ff), from);
+    const typename Frag<T>::raw second = to_operand<T>(load_frag<T, ALIGNED>(b_row[1], k, ff), from);
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      Frag<T>::mma(acc[m][0], a[m], b0);
-      Frag<T>::mma(acc[m][1], a[m], b1);
+      const typename Frag<T>::raw x_now = to_operand<T>(load_frag<T, ALIGNED>(a_row[m], k, ff), from);
+      Frag<T>::mma(acc[m][0], x_now, first);
+      Frag<T>::mma(acc[m][1], x_now, second);
     }
-    b0 = b0_next;
-    b1 = b1_next;
-#pragma unroll
-    for (int m = 0; m < MT; ++m) a[m] = a_next[m];
   }
 #pragma unroll
   for (int m = 0; m < MT; ++m)
@@ -591,7 +662,11 @@ int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* we
     const int epl = dtype == QIL_F32 ? 4 : 8;
     const bool aligned = width % epl == 0 && ff % epl == 0 &&
                          (((uintptr_t)x | (uintptr_t)w_gate_up | (uintptr_t)w_down | (uintptr_t)hidden) % 16) == 0;
-    const dim3 g_up(max_tiles, gated ? (ff + 63) / 64 : (ff + 127) / 128), g_down(max_tiles, (width + 127) / 128);
+    // Tiles of 16 pairs: a block is one wave (a CU takes about 12 bytes a cycle from memory however many waves ask, so the
+    // weights have to come through all of the CUs evenly); of 64: four waves, which share the rows of x.
+    const int waves = tile_rows == 16 ? 1 : 4, up_columns = (gated ? 16 : 32) * waves, down_columns = 32 * waves;
+    const dim3 g_up(max_tiles, (ff + up_columns - 1) / up_columns), g_down(max_tiles, (width + down_columns - 1) / down_columns);
+    const dim3 threads(waves * QIL_WAVE);
     if (dtype == QIL_BF16 && tile_rows == 64 && aligned && width % 8 == 0 && ff % 8 == 0) {
       static bool granted = false;                        // (all instantiations, once)
       if (!granted) {
@@ -620,12 +695,12 @@ int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* we
 #define QIL_MOE(T, MT, ALIGNED)                                                                                       \
   do {                                                                                                                \
     if (gated)                                                                                                        \
-      hipLaunchKernelGGL((moe_gate_up_kernel<T, MT, ALIGNED>), g_up, dim3(256), 0, s, (const T*)x, width,              \
+      hipLaunchKernelGGL((moe_gate_up_kernel<T, MT, ALIGNED>), g_up, threads, 0, s, (const T*)x, width,              \
                          (const T*)w_gate_up, ff, tiles, max_tiles, places, top, (T*)hidden, act, limit, alpha);       \
     else                                                                                                              \
-      hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, true>), g_up, dim3(256), 0, s, (const T*)x, width,           \
+      hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, true>), g_up, threads, 0, s, (const T*)x, width,           \
                          (const T*)w_gate_up, ff, tiles, max_tiles, places, (float*)nullptr, (T*)hidden, top, act);    \
-    hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, false>), g_down, dim3(256), 0, s, (const T*)hidden, ff,        \
+    hipLaunchKernelGGL((moe_down_kernel<T, MT, ALIGNED, false>), g_down, threads, 0, s, (const T*)hidden, ff,        \
                        (const T*)w_down, width, tiles, max_tiles, places, y, (T*)nullptr, top, act);                   \
   } while (0)
 #define QIL_MOE_T(T)                                                                                                  \

@@ -685,6 +685,15 @@ def test_sizes_beyond_the_kernels_are_refused_when_the_model_is_built():
             build_kebudra(KebudraConfig.from_dict(config), device='cpu')
 
 
+def test_the_bench_makes_valid_configurations():
+    """The configurations that ``bench.py --phase designs --design kebudra`` measures are ones the design accepts."""
+    import bench
+    from qil_amd.config import KebudraConfig
+    for sizes in bench.DESIGN_SIZES.values():
+        for kind in ('turns', 'delta', 'difference', 'latent'):
+            assert len(KebudraConfig.from_dict(bench.kebudra_config(sizes, 6, 100, kind)).layers) == 6
+
+
 def test_random_weights_load(tmp_path, cpu_kernels):
     """A folder written from a configuration and a seed holds every tensor of the design, and loads and runs; the inner sizes of
     the low-rank products are the folder's."""
