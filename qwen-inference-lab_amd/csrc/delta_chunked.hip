@@ -14,6 +14,8 @@
 // most zero) and A and B are matrix products; inside a block every pair's exponential is taken by itself.  The triangular
 // system goes block by block: the 16 x 16 diagonal blocks of I + A are inverted, a column a lane.
 //
+// The operands lie in the scratch memory tile by tile as the lanes of the walk hold them (64 lanes x 4 floats, a kilobyte in a
+// row): a load of 16 rows by 16 bytes would occupy the address path for 64 cycles, four times what the tile's product takes.
 // The layout trick throughout: a result tile holds rows 4 kb + e and column r in lane 16 kb + r; as the next product's
 // right operand, whose k-step e then stands for the rows 4 kb + e, it needs no move, and the left operand's 4 neighbouring
 // elements a lane are one 16-byte load.
@@ -50,10 +52,14 @@ __device__ __forceinline__ float dc_softplus(float v) {
 // for them as well).
 __device__ __forceinline__ void dc_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
+// Element (row i, column j) of a left operand's tile.
+__device__ __forceinline__ int dc_in_operand(int i, int j) { return (i + 16 * (j >> 2)) * 4 + (j & 3); }
+
 // Where chunk c of sequence seq keeps its operands: sequences before it took at most row0 / DC_L + seq places.
 __device__ __forceinline__ size_t dc_place(int row0, int seq, int c) { return (size_t)(row0 / DC_L + seq + c); }
 
-// Floats of one (place, head): W [64][DP] (negated), Q [64][DP], K^T [DP][64], U [64][VP], B [64][64], the decay e^(G_end) [DP].
+// Floats of one (place, head), in tiles: W (negated) and Q [4 token blocks][DP / 16], K^T [DP / 16][4], U [VP / 16][4] (result
+// tiles), B [4][4], and the decay e^(G_end) [DP].
 __host__ __device__ __forceinline__ size_t dc_cell(int dp, int vp) { return (size_t)3 * DC_L * dp + DC_L * vp + DC_L * DC_L + dp; }
 
 // grid (chunks of the longest sequence, sequences x heads), 8 waves.
@@ -181,7 +187,7 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
     for (int p = 0; p < 2; ++p) {
       const float uk = units[j + p];
       a[dc_in_block(r, j + p - b * 16)] = i > j + p ? -kk[p] * units[i] * uk * units[2 * DC_L + i] : 0.f;
-      B[i * DC_L + j + p] = i >= j + p ? qk[p] * units[DC_L + i] * uk : 0.f;
+      B[(b * 4 + b) * DC_BLOCK + dc_in_operand(r, j + p - b * 16)] = i >= j + p ? qk[p] * units[DC_L + i] * uk : 0.f;
     }
   }
   // between blocks: waves 0 .. 5 a pair (later block bi, earlier block bj) each
@@ -210,7 +216,7 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
     for (int e = 0; e < 4; ++e) {
       const int i = bi * 16 + 4 * kb + e;
       a[dc_in_block(4 * kb + e, r)] = -kk[e] * units[i] * uk * units[2 * DC_L + i];
-      B[i * DC_L + bj * 16 + r] = qk[e] * units[DC_L + i] * uk;
+      B[(bi * 4 + bj) * DC_BLOCK + dc_in_operand(4 * kb + e, r)] = qk[e] * units[DC_L + i] * uk;
     }
   }
   __syncthreads();
@@ -256,28 +262,41 @@ delta_prepare_kernel(DeltaInputs in, const int* __restrict__ cu_seqlens, float* 
 #pragma unroll
       for (int j = 0; j < b; ++j) acc = dc_mma(dc_ld(A + (b * (b + 1) / 2 + j) * DC_BLOCK + dc_in_block(r, 4 * kb)), x[j], acc);
       x[b] = dc_mma(dc_ld(A + (b * (b + 1) / 2 + b) * DC_BLOCK + dc_in_block(r, 4 * kb)), acc, (f32x4){0.f, 0.f, 0.f, 0.f});
+      if (is_w) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int t = b * 16 + 4 * kb + e;
-        if (is_w) W[t * DP + col] = -x[b][e];
-        else Uo[t * vp + col] = x[b][e];
+        for (int e = 0; e < 4; ++e) W[(b * (DP / 16) + tile) * DC_BLOCK + dc_in_operand(4 * kb + e, r)] = -x[b][e];
+      } else {
+        *reinterpret_cast<f32x4*>(Uo + (((tile - DP / 16) * 4 + b) * 64 + lane) * 4) = x[b];
       }
     }
   }
-  // the queries with their decays from the chunk's start, the keys with theirs to its end (transposed), the whole decay
-#pragma unroll 4
-  for (int item = tid; item < DC_L * DP; item += DC_THREADS) {
-    const int t = item / DP, ch = item % DP;
-    float from = L[t * LROW + ch];
-    for (int m = 0; m < (t >> 4); ++m) from += L[(m * 16 + 15) * LROW + ch];
-    Q[item] = ld(qs + t * KROW + ch) * units[DC_L + t] * dc_exp2(from);
-  }
-#pragma unroll 4
-  for (int item = tid; item < DC_L * DP; item += DC_THREADS) {
-    const int t = item % DC_L, ch = item / DC_L;
-    float upto = L[((t >> 4) * 16 + 15) * LROW + ch] - L[t * LROW + ch];
-    for (int m = (t >> 4) + 1; m < 4; ++m) upto += L[(m * 16 + 15) * LROW + ch];
-    KT[item] = ld(ks + t * KROW + ch) * units[t] * dc_exp2(fminf(upto, 0.f));
+  // the queries with their decays from the chunk's start, the keys with theirs to its end (transposed): a wave a channel tile
+  for (int n = wave; n < DP / 16; n += DC_THREADS / QIL_WAVE) {
+    f32x4 before = {0.f, 0.f, 0.f, 0.f};
+    const int ch = n * 16 + 4 * kb;
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+      const int t = b * 16 + r;
+      const f32x4 from = before + dc_ld(L + t * LROW + ch);
+      f32x4 q = dc_ld(qs + t * KROW + ch);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) q[e] *= units[DC_L + t] * dc_exp2(from[e]);
+      *reinterpret_cast<f32x4*>(Q + ((b * (DP / 16) + n) * 64 + lane) * 4) = q;
+      before += dc_ld(L + (b * 16 + 15) * LROW + ch);
+    }
+    float after = 0.f;
+#pragma unroll
+    for (int b = 3; b >= 0; --b) {
+      const float whole = L[(b * 16 + 15) * LROW + n * 16 + r];
+      f32x4 k;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = b * 16 + 4 * kb + e;
+        k[e] = ld(ks + t * KROW + n * 16 + r) * units[t] * dc_exp2(fminf(after + whole - L[t * LROW + n * 16 + r], 0.f));
+      }
+      *reinterpret_cast<f32x4*>(KT + ((n * 4 + b) * 64 + lane) * 4) = k;
+      after += whole;
+    }
   }
   for (int ch = tid; ch < DP; ch += DC_THREADS)
     end[ch] = dc_exp2(L[15 * LROW + ch] + L[31 * LROW + ch] + L[47 * LROW + ch] + L[63 * LROW + ch]);
@@ -313,29 +332,27 @@ delta_walk_kernel(const float* __restrict__ scratch, float* __restrict__ slots, 
   }
   const size_t cell = dc_cell(DP, vp), stride = cell * heads;
   const float* at = scratch + (dc_place(row0, seq, 0) * heads + h) * cell;
-  const int chunks = (len + DC_L - 1) / DC_L, t_row = wave * 16 + r;
+  const int chunks = (len + DC_L - 1) / DC_L;
   // this chunk's operands; each is asked for again, for the next chunk, as soon as it has been used
   f32x4 w[DT], q[DT], b[4], k[OWN][4], keep[OWN], write;
   auto load_w = [&](const float* p) {
 #pragma unroll
-    for (int n = 0; n < DT; ++n) w[n] = dc_ld(p + t_row * DP + n * 16 + 4 * kb);
-    const float* uo = p + 3 * DC_L * DP;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) write[e] = uo[(wave * 16 + 4 * kb + e) * vp + j0 + r];
+    for (int n = 0; n < DT; ++n) w[n] = dc_ld(p + ((wave * DT + n) * 64 + lane) * 4);
+    write = dc_ld(p + 3 * DC_L * DP + (((j0 >> 4) * 4 + wave) * 64 + lane) * 4);
   };
   auto load_q = [&](const float* p) {
 #pragma unroll
-    for (int n = 0; n < DT; ++n) q[n] = dc_ld(p + DC_L * DP + t_row * DP + n * 16 + 4 * kb);
+    for (int n = 0; n < DT; ++n) q[n] = dc_ld(p + DC_L * DP + ((wave * DT + n) * 64 + lane) * 4);
     const float* bo = p + 3 * DC_L * DP + DC_L * vp;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) b[j] = dc_ld(bo + t_row * DC_L + j * 16 + 4 * kb);      // (nobody wrote or uses those of j > wave)
+    for (int j = 0; j < 4; ++j) b[j] = dc_ld(bo + ((wave * 4 + j) * 64 + lane) * 4);   // (nobody wrote or uses those of j > wave)
   };
   auto load_k = [&](const float* p) {
     const float* eo = p + 3 * DC_L * DP + DC_L * vp + DC_L * DC_L;
 #pragma unroll
     for (int n = 0; n < OWN; ++n) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) k[n][j] = dc_ld(p + 2 * DC_L * DP + ((wave + 4 * n) * 16 + r) * DC_L + j * 16 + 4 * kb);
+      for (int j = 0; j < 4; ++j) k[n][j] = dc_ld(p + 2 * DC_L * DP + (((wave + 4 * n) * 4 + j) * 64 + lane) * 4);
       keep[n] = dc_ld(eo + (wave + 4 * n) * 16 + 4 * kb);
     }
   };

@@ -47,7 +47,9 @@ __device__ __forceinline__ float4 moe_load4(const bf16_t* p) {
   return make_float4(__uint_as_float(raw.x << 16), __uint_as_float(raw.x & 0xffff0000u), __uint_as_float(raw.y << 16),
                      __uint_as_float(raw.y & 0xffff0000u));
 }
-template <typename T, bool VEC>
+// DEPTH: pieces of a row that are on their way while one is multiplied (1: with many rows other waves hide the way); the sums
+// are the same.
+template <typename T, bool VEC, int DEPTH>
 __global__ void __launch_bounds__(MOE_ROUTE_THREADS)
 moe_logits_kernel(const T* __restrict__ x, int n, int width, const float* __restrict__ w_router, int outputs,
                   float* __restrict__ logits) {
@@ -59,13 +61,36 @@ moe_logits_kernel(const T* __restrict__ x, int n, int width, const float* __rest
 #pragma unroll
   for (int r = 0; r < 8; ++r) rows[r] = x + (size_t)min(row0 + r, n - 1) * width;
   float acc[8] = {};
-  if (VEC) {
+  if (VEC && DEPTH == 1) {
     for (int i = lane * 4; i < width; i += QIL_WAVE * 4) {
       const float4 wv = moe_load4(w + i);
 #pragma unroll
       for (int r = 0; r < 8; ++r) {
         const float4 xv = moe_load4(rows[r] + i);
         acc[r] += xv.x * wv.x + xv.y * wv.y + xv.z * wv.z + xv.w * wv.w;
+      }
+    }
+  } else if (VEC) {
+    const int pieces = (width + QIL_WAVE * 4 - 1) / (QIL_WAVE * 4);
+    float4 wv[DEPTH], xv[DEPTH][8];
+    auto fetch = [&](int d, int piece) {                // (past the row's end: any element, times zero)
+      const int i = (min(piece, pieces - 1) * QIL_WAVE + lane) * 4, at = min(i, width - 4);
+      wv[d] = moe_load4(w + at);
+      if (i >= width) wv[d] = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int r = 0; r < 8; ++r) xv[d][r] = moe_load4(rows[r] + at);
+    };
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) fetch(d, d);
+    for (int piece = 0; piece < pieces; piece += DEPTH) {
+#pragma unroll
+      for (int d = 0; d < DEPTH; ++d) {
+        if (piece + d < pieces) {
+#pragma unroll
+          for (int r = 0; r < 8; ++r)
+            acc[r] += xv[d][r].x * wv[d].x + xv[d][r].y * wv[d].y + xv[d][r].z * wv[d].z + xv[d][r].w * wv[d].w;
+        }
+        fetch(d, piece + d + DEPTH);
       }
     }
   } else {
@@ -82,22 +107,47 @@ moe_logits_kernel(const T* __restrict__ x, int n, int width, const float* __rest
   }
 }
 
-// The choice from the logits: a wave a row, four rows a block (every wave walks the same steps, so the barriers
-// between a wave's writes to its part of LDS and its reads are met by all).
-__global__ void __launch_bounds__(MOE_ROUTE_THREADS)
-moe_select_kernel(const float* __restrict__ logits, int n, const float* __restrict__ bias,
-                  const float* __restrict__ correction, int outputs, int groups,
-                  int keep, int top, int renormalize, int* __restrict__ chosen, float* __restrict__ weights,
-                  int sigmoid_scores, int group_top2, float weight_scale, float renormalize_eps) {
-  extern __shared__ float lds[];                        // per wave: [outputs] scores, [outputs] choice scores, [groups]
-  const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE;
-  float* score = lds + (size_t)wave * (2 * outputs + groups);
+// The choice of one row from its logits, by one wave (`live`: the row is there; every wave walks the same steps, so the
+// barriers between a wave's writes to its part of LDS and its reads are met by all).  lds: the wave's [outputs] scores,
+// [outputs] choice scores, [groups].  put(slot, output) is called by one lane, and weights go to weights[0 .. top).
+template <typename PUT>
+__device__ __forceinline__ void select_row(const float* __restrict__ z, bool live, float* lds, int lane, const float* __restrict__ bias,
+                                           const float* __restrict__ correction, int outputs, int groups, int keep, int top,
+                                           int renormalize, float* __restrict__ weights, int sigmoid_scores, int group_top2,
+                                           float weight_scale, float renormalize_eps, PUT put) {
+  float* score = lds;
   float* choice = score + outputs;
   float* group_best = choice + outputs;
-  const int n_row = blockIdx.x * (MOE_ROUTE_THREADS / QIL_WAVE) + wave;
-  const bool live = n_row < n;
-  const float* z = logits + (size_t)min(n_row, n - 1) * outputs;
   auto logit = [&](int e) { return z[e] + (bias ? bias[e] : 0.f); };
+  if (outputs <= QIL_WAVE && (groups <= 1 || keep >= groups)) {      // an output a lane: the same arithmetic in registers
+    const bool mine = lane < outputs;
+    const float v = mine ? logit(lane) : -INFINITY;
+    float s, c;
+    if (sigmoid_scores) {
+      s = 1.f / (1.f + expf(-v));
+      c = s;
+    } else {
+      const float top_logit = wave_max(v), e = mine ? expf(v - top_logit) : 0.f;
+      s = e / wave_sum(e);
+      c = v;
+    }
+    if (correction && mine) c = s + correction[lane];
+    bool open = mine && c == c && c != INFINITY;
+    float sum = 0.f, kept = 0.f;
+    for (int round = 0; round < top; ++round) {
+      float best = open ? c : -INFINITY;
+      int at = open ? lane : 0x7fffffff;
+      wave_argmax(best, at);
+      if (at == 0x7fffffff) at = 0;
+      const float chosen_score = __shfl(s, at, QIL_WAVE);
+      sum += chosen_score;
+      if (lane == round) kept = chosen_score;
+      if (lane == at) open = false;
+      if (lane == 0 && live) put(round, at);
+    }
+    if (live && lane < top) weights[lane] = (renormalize ? kept / (sum + renormalize_eps) : kept) * weight_scale;
+    return;
+  }
   if (sigmoid_scores) {                                 // every output by itself; the choice goes by the score
     for (int e = lane; e < outputs; e += QIL_WAVE) {
       const float s = 1.f / (1.f + expf(-logit(e)));
@@ -162,57 +212,111 @@ moe_select_kernel(const float* __restrict__ logits, int n, const float* __restri
     if (lane == round) mine = s;
     __syncthreads();
     if (lane == 0) {
-      if (live) chosen[(size_t)n_row * top + round] = at;
+      if (live) put(round, at);
       choice[at] = INFINITY;
     }
     __syncthreads();
   }
   if (live && lane < top)
-    weights[(size_t)n_row * top + lane] = (renormalize ? mine / (sum + renormalize_eps) : mine) * weight_scale;
+    weights[lane] = (renormalize ? mine / (sum + renormalize_eps) : mine) * weight_scale;
+}
+
+// A wave a row, four rows a block.
+__global__ void __launch_bounds__(MOE_ROUTE_THREADS)
+moe_select_kernel(const float* __restrict__ logits, int n, const float* __restrict__ bias,
+                  const float* __restrict__ correction, int outputs, int groups,
+                  int keep, int top, int renormalize, int* __restrict__ chosen, float* __restrict__ weights,
+                  int sigmoid_scores, int group_top2, float weight_scale, float renormalize_eps) {
+  extern __shared__ float lds[];
+  const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE;
+  const int row = blockIdx.x * (MOE_ROUTE_THREADS / QIL_WAVE) + wave;
+  int* mine = chosen + (size_t)row * top;
+  select_row(logits + (size_t)min(row, n - 1) * outputs, row < n, lds + (size_t)wave * (2 * outputs + groups), lane, bias, correction,
+             outputs, groups, keep, top, renormalize, weights + (size_t)row * top, sigmoid_scores, group_top2, weight_scale,
+             renormalize_eps, [&](int slot, int at) { mine[slot] = at; });
 }
 
 // ------------------------------------------------------------------------------------------------ align
-// tiles: [3][max_tiles] expert, first place, pairs.  places: [pairs] the pair at every place.
-__global__ void __launch_bounds__(1024)
-moe_align_kernel(const int* __restrict__ chosen, int pairs, int experts, int tile_rows, int max_tiles,
-                 int* __restrict__ tiles, int* __restrict__ places) {
-  __shared__ int count[MOE_MAX_OUTPUTS], first[MOE_MAX_OUTPUTS], first_tile[MOE_MAX_OUTPUTS + 1];
+// tiles: [3][max_tiles] expert, first place, pairs.  places: [pairs] the pair at every place.  By all of a block's threads.
+struct AlignLds { int count[MOE_MAX_OUTPUTS], first[MOE_MAX_OUTPUTS], first_tile[MOE_MAX_OUTPUTS + 1]; };
+__device__ __forceinline__ void align_pairs(const int* chosen, int pairs, int experts, int tile_rows, int max_tiles,
+                                            int* __restrict__ tiles, int* __restrict__ places, AlignLds& lds) {
   const int tid = threadIdx.x;
-  for (int e = tid; e < experts; e += blockDim.x) count[e] = 0;
+  for (int e = tid; e < experts; e += blockDim.x) lds.count[e] = 0;
   __syncthreads();
   for (int p = tid; p < pairs; p += blockDim.x) {
     const int e = chosen[p];
-    if (e < experts) atomicAdd(&count[e], 1);
+    if (e < experts) atomicAdd(&lds.count[e], 1);
   }
   __syncthreads();
-  if (tid == 0) {
+  if (tid < QIL_WAVE) {                                   // running sums over the experts, 64 at a time
     int place = 0, tile = 0;
-    for (int e = 0; e < experts; ++e) {
-      first[e] = place;
-      first_tile[e] = tile;
-      place += count[e];
-      tile += (count[e] + tile_rows - 1) / tile_rows;
+    for (int e0 = 0; e0 < experts; e0 += QIL_WAVE) {
+      const int e = e0 + tid, pairs_here = e < experts ? lds.count[e] : 0, tiles_here = (pairs_here + tile_rows - 1) / tile_rows;
+      int p = pairs_here, t = tiles_here;
+#pragma unroll
+      for (int o = 1; o < QIL_WAVE; o <<= 1) {
+        const int p_up = __shfl_up(p, o, QIL_WAVE), t_up = __shfl_up(t, o, QIL_WAVE);
+        if (tid >= o) { p += p_up; t += t_up; }
+      }
+      if (e < experts) {
+        lds.first[e] = place + p - pairs_here;
+        lds.first_tile[e] = tile + t - tiles_here;
+      }
+      place += __shfl(p, QIL_WAVE - 1, QIL_WAVE);
+      tile += __shfl(t, QIL_WAVE - 1, QIL_WAVE);
     }
-    first_tile[experts] = tile;
+    if (tid == 0) lds.first_tile[experts] = tile;
   }
   __syncthreads();
   for (int t = tid; t < max_tiles; t += blockDim.x) tiles[2 * max_tiles + t] = 0;
   __syncthreads();
   for (int e = tid; e < experts; e += blockDim.x) {
-    const int n_tiles = first_tile[e + 1] - first_tile[e];
+    const int n_tiles = lds.first_tile[e + 1] - lds.first_tile[e];
     for (int t = 0; t < n_tiles; ++t) {
-      const int at = first_tile[e] + t;
+      const int at = lds.first_tile[e] + t;
       tiles[at] = e;
-      tiles[max_tiles + at] = first[e] + t * tile_rows;
-      tiles[2 * max_tiles + at] = min(tile_rows, count[e] - t * tile_rows);
+      tiles[max_tiles + at] = lds.first[e] + t * tile_rows;
+      tiles[2 * max_tiles + at] = min(tile_rows, lds.count[e] - t * tile_rows);
     }
-    count[e] = 0;                                       // from here on: the places of the expert's run already given out
+    lds.count[e] = 0;                                   // from here on: the places of the expert's run already given out
   }
   __syncthreads();
   for (int p = tid; p < pairs; p += blockDim.x) {
     const int e = chosen[p];
-    if (e < experts) places[first[e] + atomicAdd(&count[e], 1)] = p;
+    if (e < experts) places[lds.first[e] + atomicAdd(&lds.count[e], 1)] = p;
   }
+}
+
+__global__ void __launch_bounds__(1024)
+moe_align_kernel(const int* __restrict__ chosen, int pairs, int experts, int tile_rows, int max_tiles,
+                 int* __restrict__ tiles, int* __restrict__ places) {
+  __shared__ AlignLds lds;
+  align_pairs(chosen, pairs, experts, tile_rows, max_tiles, tiles, places, lds);
+}
+
+// The choice and the grouping of a step of few rows in one kernel, one block: sixteen rows at a time, then the pairs.
+#define MOE_FEW_PAIRS 1024
+__global__ void __launch_bounds__(1024)
+moe_select_align_kernel(const float* __restrict__ logits, int n, const float* __restrict__ bias, const float* __restrict__ correction,
+                        int outputs, int groups, int keep, int top, int renormalize, int* __restrict__ chosen,
+                        float* __restrict__ weights, int sigmoid_scores, int group_top2, float weight_scale, float renormalize_eps,
+                        int experts, int tile_rows, int max_tiles, int* __restrict__ tiles, int* __restrict__ places) {
+  extern __shared__ float lds[];
+  __shared__ AlignLds align;
+  __shared__ int picked[MOE_FEW_PAIRS];
+  const int lane = threadIdx.x & (QIL_WAVE - 1), wave = threadIdx.x / QIL_WAVE;
+  for (int row0 = 0; row0 < n; row0 += 1024 / QIL_WAVE) {
+    const int row = row0 + wave;
+    select_row(logits + (size_t)min(row, n - 1) * outputs, row < n, lds + (size_t)wave * (2 * outputs + groups), lane, bias, correction,
+               outputs, groups, keep, top, renormalize, weights + (size_t)row * top, sigmoid_scores, group_top2, weight_scale,
+               renormalize_eps, [&](int slot, int at) {
+                 chosen[(size_t)row * top + slot] = at;
+                 picked[row * top + slot] = at;
+               });
+  }
+  __syncthreads();
+  align_pairs(picked, n * top, experts, tile_rows, max_tiles, tiles, places, align);
 }
 
 // ------------------------------------------------------------------------------------------------ products
@@ -614,20 +718,37 @@ int qil_moe_takes(int width, int outputs, int experts, int groups, int keep, int
 // sigmoid_scores: scores are sigmoid(logit) instead of the softmax over all outputs.  group_top2: a group's score is
 // the sum of its two largest choice scores instead of its largest.  The weights are the chosen scores, divided by
 // (their sum + renormalize_eps) if renormalize, times weight_scale.
+// tiles and places (or null): the pairs' grouping for qil_moe_experts (experts, tile_rows and max_tiles as there), made by the
+// same kernel that chooses: for steps that qil_moe_aligns takes.
+int qil_moe_aligns(int n, int outputs, int groups, int top) {
+  return n * top <= MOE_FEW_PAIRS && n <= 64 && (size_t)16 * (2 * outputs + groups) * sizeof(float) <= 40 * 1024;
+}
 int qil_moe_route(const void* x, int dtype, const float* w_router, const float* bias, const float* correction,
                   float* logits, int* chosen,
                   float* weights, int n, int width, int outputs, int groups, int keep, int top, int renormalize,
-                  int sigmoid_scores, int group_top2, float weight_scale, float renormalize_eps, hipStream_t s) {
+                  int sigmoid_scores, int group_top2, float weight_scale, float renormalize_eps, int experts, int tile_rows,
+                  int max_tiles, int* tiles, int* places, hipStream_t s) {
   if (n == 0) return 0;
+  if (tiles && (!places || !qil_moe_aligns(n, outputs, groups, top) || experts < 1 || experts > outputs)) return -1;
   if (!qil_moe_takes(width, outputs, 0, groups, keep, top) || !logits) return -1;
   const dim3 g_logits((n + 7) / 8, (outputs + 3) / 4);
   const bool vec = width % 4 == 0 && (((uintptr_t)x | (uintptr_t)w_router) % 16) == 0;
 #define QIL_LOGITS(T, VEC)                                                                                            \
-  hipLaunchKernelGGL((moe_logits_kernel<T, VEC>), g_logits, dim3(MOE_ROUTE_THREADS), 0, s, (const T*)x, n, width,      \
+  if (n <= 64)                                                                                                        \
+    hipLaunchKernelGGL((moe_logits_kernel<T, VEC, 4>), g_logits, dim3(MOE_ROUTE_THREADS), 0, s, (const T*)x, n, width, \
+                       w_router, outputs, logits);                                                                    \
+  else                                                                                                                \
+    hipLaunchKernelGGL((moe_logits_kernel<T, VEC, 1>), g_logits, dim3(MOE_ROUTE_THREADS), 0, s, (const T*)x, n, width,      \
                      w_router, outputs, logits)
-  if (dtype == QIL_F32) { if (vec) QIL_LOGITS(float, true); else QIL_LOGITS(float, false); }
-  else { if (vec) QIL_LOGITS(bf16_t, true); else QIL_LOGITS(bf16_t, false); }
+  if (dtype == QIL_F32) { if (vec) { QIL_LOGITS(float, true); } else { QIL_LOGITS(float, false); } }
+  else { if (vec) { QIL_LOGITS(bf16_t, true); } else { QIL_LOGITS(bf16_t, false); } }
 #undef QIL_LOGITS
+  if (tiles) {
+    hipLaunchKernelGGL(moe_select_align_kernel, dim3(1), dim3(1024), (size_t)16 * (2 * outputs + groups) * sizeof(float), s, logits,
+                       n, bias, correction, outputs, groups, keep, top, renormalize, chosen, weights, sigmoid_scores, group_top2,
+                       weight_scale, renormalize_eps, experts, tile_rows, max_tiles, tiles, places);
+    QIL_RETURN_LAUNCH_STATUS();
+  }
   const int per_block = MOE_ROUTE_THREADS / QIL_WAVE;
   const size_t lds = (size_t)per_block * (2 * outputs + groups) * sizeof(float);
   hipLaunchKernelGGL(moe_select_kernel, dim3((n + per_block - 1) / per_block), dim3(MOE_ROUTE_THREADS), lds, s, logits, n,
@@ -649,7 +770,7 @@ int qil_moe_max_tiles(int pairs, int experts, int tile_rows) { return (pairs + t
 int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* weights, const void* w_gate_up,
                     const void* w_down, int* tiles, int* places, void* hidden, float* y, float* out, int n, int width,
                     int ff, int experts, int top, int tile_rows, int max_tiles, int act, float limit, float alpha,
-                    hipStream_t s) {
+                    int aligned_already, hipStream_t s) {
   if (n == 0) return 0;
   const int pairs = n * top;
   const bool gated = act < QIL_ACT_RELU_SQUARED;
@@ -657,8 +778,9 @@ int qil_moe_experts(const void* x, int dtype, const int* chosen, const float* we
       max_tiles < qil_moe_max_tiles(pairs, experts, tile_rows) || width < 1 || ff < 1)
     return -1;
   if (experts > 0) {
-    hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, s, chosen, pairs, experts, tile_rows, max_tiles, tiles,
-                       places);
+    if (!aligned_already)                                  // (else the route's kernel has made tiles and places)
+      hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, s, chosen, pairs, experts, tile_rows, max_tiles, tiles,
+                         places);
     const int epl = dtype == QIL_F32 ? 4 : 8;
     const bool aligned = width % epl == 0 && ff % epl == 0 &&
                          (((uintptr_t)x | (uintptr_t)w_gate_up | (uintptr_t)w_down | (uintptr_t)hidden) % 16) == 0;

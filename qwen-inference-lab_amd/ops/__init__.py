@@ -1621,7 +1621,7 @@ ROUTER_GROUP_SCORES = {'max': 0, 'top2': 1}
 
 
 def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bias=None, score='softmax',
-              group_score='max', weight_scale=1.0, renormalize_eps=0.0):
+              group_score='max', weight_scale=1.0, renormalize_eps=0.0, align_for=None):
     """x [N, width] (model type), router float32 [outputs, width], correction float32 [outputs] or None ->
     (chosen int32 [N, top], weights float32 [N, top]): softmax scores over all outputs in float32; the choice goes
     by score + correction among the outputs of the ``keep`` best of ``groups`` equal groups of neighbours (a group's
@@ -1629,7 +1629,9 @@ def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bi
     makes them the softmax over the chosen logits alone).  ``bias`` float32 [outputs]: added to the logits.
     ``score='sigmoid'``: scores are sigmoid(logit) and the choice goes by the score (+ correction);
     ``group_score='top2'``: a group's score is the sum of its two largest choice scores; with ``renormalize`` the
-    divisor is the chosen scores' sum + ``renormalize_eps``; ``weight_scale`` multiplies the weights last."""
+    divisor is the chosen scores' sum + ``renormalize_eps``; ``weight_scale`` multiplies the weights last.
+    ``align_for``: the number of experts with tensors; the result is then (chosen, weights, grouping), where the grouping is
+    the pairs' for ``moe_experts`` in a step of few rows, made by the kernel that chooses, and None otherwise."""
     n, width = x.shape
     _require(x, 'x')
     outputs = router.shape[0]
@@ -1644,25 +1646,44 @@ def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bi
     chosen = torch.empty((n, top), dtype=torch.int32, device=x.device)
     weights = torch.empty((n, top), dtype=torch.float32, device=x.device)
     logits = torch.empty((n, outputs), dtype=torch.float32, device=x.device)
+    grouping = _moe_grouping(lib, n * top, align_for, x.device) if align_for and n and lib.qil_moe_aligns(n, outputs, groups, top) else None
+    tail = (0, 0, 0, None, None) if grouping is None else (align_for, grouping.tile_rows, grouping.max_tiles, *grouping.pointers())
     _check(lib.qil_moe_route(_ptr(x), _code(x.dtype), _ptr(router), _ptr(bias), _ptr(correction), _ptr(logits), _ptr(chosen),
                              _ptr(weights), n, width, outputs, groups, keep, top, int(bool(renormalize)),
                              ROUTER_SCORES[score], ROUTER_GROUP_SCORES[group_score], float(weight_scale),
-                             float(renormalize_eps), _stream()), 'moe_route')
-    return chosen, weights
+                             float(renormalize_eps), *tail, _stream()), 'moe_route')
+    return (chosen, weights) if align_for is None else (chosen, weights, grouping)
+
+
+class _Grouping:
+    """Where the pairs (token, chosen expert) of a step lie once they are grouped by expert: device scratch memory."""
+
+    def __init__(self, scratch, pairs, experts, tile_rows, max_tiles):
+        self.scratch, self.pairs, self.experts, self.tile_rows, self.max_tiles = scratch, pairs, experts, tile_rows, max_tiles
+
+    def pointers(self):
+        return _ptr(self.scratch), self.scratch[3 * self.max_tiles:].data_ptr()
+
+
+def _moe_grouping(lib, pairs, experts, device):
+    tile_rows = lib.qil_moe_tile_rows(pairs, experts)
+    max_tiles = lib.qil_moe_max_tiles(pairs, experts, tile_rows)
+    return _Grouping(torch.empty(3 * max_tiles + pairs, dtype=torch.int32, device=device), pairs, experts, tile_rows, max_tiles)
 
 
 # Activations of experts without a gate branch: name -> code of the kernels.  'relu_squared': max(z, 0)^2.
 EXPERT_ACTIVATIONS = {'relu_squared': 16}
 
 
-def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alpha=1.0, lazy=False):
+def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alpha=1.0, lazy=False, grouping=None):
     """The weighted sum of the chosen experts' outputs, float32 [N, width]; with ``lazy`` a ``RoutedSum`` (the pairs'
     rows, for a norm that makes the sum while it loads them).  ``gate_up`` [experts, 2, ff, width] (an
     expert's gate rows, then its up rows), ``down`` [experts, width, ff], both of x's type; an expert computes
     down(act(gate x, up x)) with ``activation`` of ``GATE_FUNCTIONS``; with an ``activation`` of ``EXPERT_ACTIVATIONS`` there is no
     gate branch, ``gate_up`` is [experts, 1, ff, width] and an expert computes down(act(up x)).  A chosen index from ``experts`` on is an
     identity expert: its output is x itself.  The pairs (token, chosen expert) are grouped by expert on the device;
-    the host sees no routing result, so a step may be captured into a graph."""
+    the host sees no routing result, so a step may be captured into a graph.  ``grouping``: what ``moe_route`` made with
+    ``align_for``."""
     n, width = x.shape
     top = chosen.shape[1]
     _require(x, 'x')
@@ -1674,16 +1695,18 @@ def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alp
     _require(down, 'down', x.dtype, (experts, width, ff))
     lib = library.load()
     pairs = n * top
-    tile_rows = lib.qil_moe_tile_rows(pairs, experts)
-    max_tiles = lib.qil_moe_max_tiles(pairs, experts, tile_rows)
-    scratch = torch.empty(3 * max_tiles + pairs, dtype=torch.int32, device=x.device)
+    grouped = grouping is not None
+    if grouped and (grouping.pairs, grouping.experts) != (pairs, experts):
+        raise ValueError('moe_experts: the grouping is of another step')
+    if not grouped:
+        grouping = _moe_grouping(lib, pairs, experts, x.device)
     hidden = torch.empty((pairs, ff), dtype=x.dtype, device=x.device)
     y = torch.empty((pairs, width), dtype=torch.float32, device=x.device)
     out = None if lazy else torch.empty((n, width), dtype=torch.float32, device=x.device)
     _check(lib.qil_moe_experts(_ptr(x), _code(x.dtype), _ptr(chosen), _ptr(weights), _ptr(gate_up), _ptr(down),
-                               _ptr(scratch), scratch[3 * max_tiles:].data_ptr(), _ptr(hidden), _ptr(y), _ptr(out), n, width,
-                               ff, experts, top, tile_rows, max_tiles, act, float(limit),
-                               float(alpha), _stream()), 'moe_experts')
+                               *grouping.pointers(), _ptr(hidden), _ptr(y), _ptr(out), n, width, ff, experts, top,
+                               grouping.tile_rows, grouping.max_tiles, act, float(limit), float(alpha), int(grouped), _stream()),
+           'moe_experts')
     return RoutedSum(x, y, chosen, weights, experts) if lazy else out
 
 

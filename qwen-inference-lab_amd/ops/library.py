@@ -328,7 +328,9 @@ def _declare(lib):
     lib.qil_moe_combine.restype = i
     lib.qil_moe_takes.argtypes = [i, i, i, i, i, i]
     lib.qil_moe_takes.restype = i
-    lib.qil_moe_route.argtypes = [p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, f, f, p]
+    lib.qil_moe_route.argtypes = [p, i, p, p, p, p, p, p, i, i, i, i, i, i, i, i, i, f, f, i, i, i, p, p, p]
+    lib.qil_moe_aligns.argtypes = [i, i, i, i]
+    lib.qil_moe_aligns.restype = i
     lib.qil_moe_route.restype = i
     lib.qil_scaled_sum.argtypes = [p, i, i, p, i, i, f, f, p, i, i, p]
     lib.qil_sigmoid_gate.argtypes = [p, p, i, i, i, i, p, i, i, i, p]
@@ -345,7 +347,7 @@ def _declare(lib):
     lib.qil_moe_tile_rows.restype = i
     lib.qil_moe_max_tiles.argtypes = [i, i, i]
     lib.qil_moe_max_tiles.restype = i
-    lib.qil_moe_experts.argtypes = [p, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, f, f, p]
+    lib.qil_moe_experts.argtypes = [p, i, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, f, f, i, p]
     lib.qil_moe_experts.restype = i
     lib.qil_post_norm_scale_add.argtypes = [p, p, i, i, p, p, p, f, i, p, i, p, i, p, i, i, p]
     lib.qil_post_norm_scale_add.restype = i

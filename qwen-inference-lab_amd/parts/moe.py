@@ -99,12 +99,12 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h, add_to=None):
         p = self.p
-        chosen, weights = ops.moe_route(h, p['router.weight'], p.get('router.correction'), groups=self.groups,
+        chosen, weights, grouping = ops.moe_route(h, p['router.weight'], p.get('router.correction'), groups=self.groups,
                                         keep=self.keep, top=self.top, renormalize=self.renormalize, bias=p.get('router.bias'),
                                         score=self.score, group_score=self.group_score, weight_scale=self.weight_scale,
-                                        renormalize_eps=self.renormalize_eps)
+                                        renormalize_eps=self.renormalize_eps, align_for=self.experts)
         out = ops.moe_experts(h, chosen, weights, p['experts.gate_up_proj.weight'], p['experts.down_proj.weight'],
-                              activation=self.activation, limit=self.limit, alpha=self.alpha, lazy=self.shared is None)
+                              activation=self.activation, limit=self.limit, alpha=self.alpha, lazy=self.shared is None, grouping=grouping)
         if self.shared is not None:                     # routed sum + the shared expert's result, float32
             return ops.Partials(ops.scaled_sum(out, self.shared.forward(h), 1.0, 1.0).unsqueeze(0))
         if isinstance(out, ops.RoutedSum):              # the norm that follows makes the weighted sum as it loads the rows

@@ -531,7 +531,7 @@ def residual_join(stream, pending, weight, eps, out_dtype, rows=None):
 
 
 def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bias=None, score='softmax',
-              group_score='max', weight_scale=1.0, renormalize_eps=0.0):
+              group_score='max', weight_scale=1.0, renormalize_eps=0.0, align_for=None):
     logits = x.to(torch.float32) @ router.t() + (bias if bias is not None else 0.0)
     if score == 'sigmoid':
         scores = torch.sigmoid(logits)
@@ -552,10 +552,11 @@ def moe_route(x, router, correction, *, groups, keep, top, renormalize=False, bi
     weights = scores.gather(1, chosen)
     if renormalize:
         weights = weights / (weights.sum(dim=-1, keepdim=True) + renormalize_eps)
-    return chosen.to(torch.int32), weights * weight_scale
+    result = (chosen.to(torch.int32), weights * weight_scale)
+    return result if align_for is None else (*result, None)
 
 
-def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alpha=1.0, lazy=False):
+def moe_experts(x, chosen, weights, gate_up, down, *, activation, limit=0.0, alpha=1.0, lazy=False, grouping=None):
     """float32 [N, width]; the hidden activations pass through x's type as the kernel's do."""
     n, width = x.shape
     experts = gate_up.shape[0]

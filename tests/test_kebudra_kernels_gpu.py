@@ -295,3 +295,24 @@ def test_experts_without_a_gate_branch(dtype, n, width, ff, experts, top):
     arguments = (x.cuda(), chosen.cuda(), weights.cuda(), up.cuda(), down.cuda())
     close(ops.moe_experts(*arguments, activation='relu_squared'), want, dtype, 2.0)
     close(ops.moe_experts(*arguments, activation='relu_squared', lazy=True).materialize(), want, dtype, 2.0)
+
+
+@pytest.mark.parametrize('dtype', DTYPES)
+@pytest.mark.parametrize('n,outputs,identity,groups,keep,top', [(1, 32, 0, 1, 1, 4), (8, 16, 0, 1, 1, 2), (17, 40, 8, 4, 2, 6), (64, 7, 0, 1, 1, 7),
+                                                                (64, 300, 0, 1, 1, 16), (65, 16, 0, 1, 1, 2)])
+def test_choice_and_grouping_in_one_kernel(dtype, n, outputs, identity, groups, keep, top):
+    """Steps of few rows are chosen and grouped by one kernel: the same choices and weights as by the two, bit for bit, and the
+    experts' results from its grouping are those of the grouping made from the choices."""
+    g = torch.Generator().manual_seed(n + outputs)
+    width, ff, experts = 96, 32, outputs - identity
+    x, router = torch.randn(n, width, generator=g).to(dtype).cuda(), torch.randn(outputs, width, generator=g).cuda()
+    up = (torch.randn(experts, 1, ff, width, generator=g) / 10).to(dtype).cuda()
+    down = (torch.randn(experts, width, ff, generator=g) / 6).to(dtype).cuda()
+    rules = dict(groups=groups, keep=keep, top=top, renormalize=True)
+    chosen, weights = ops.moe_route(x, router, None, **rules)
+    same, share, grouping = ops.moe_route(x, router, None, align_for=experts, **rules)
+    assert (grouping is not None) == (n <= 64 and outputs <= 300)
+    assert torch.equal(chosen, same) and torch.equal(weights, share)
+    want = ops.moe_experts(x, chosen, weights, up, down, activation='relu_squared')
+    got = ops.moe_experts(x, same, share, up, down, activation='relu_squared', grouping=grouping)
+    assert torch.equal(want, got)
